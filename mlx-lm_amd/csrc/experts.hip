@@ -6,7 +6,8 @@
 //                   came out of one product as float rows
 //   expert_rows_up / expert_rows_down
 //                   a token's chosen experts read straight from the stacked expert weights, a
-//                   wave four features at once: act[t, j, :] = w_tj silu(Wg_e x_t) * (Wu_e x_t), then
+//                   wave four features at once: act[t, j, :] = w_tj silu(Wg_e x_t) * (Wu_e x_t) (or
+//                   another activation of the two, expert_act), then
 //                   y[t, :] += sum_j Wd_e act[t, j, :] + sum_(j: e is an identity expert) w_tj x_t.
 //                   Only the chosen experts' weights are read: the kernels for few tokens.
 //   expert_tiles    the same for many tokens: the picks are sorted by expert on the device
@@ -21,6 +22,20 @@
 #include "common.h"
 
 __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+
+// An expert's activation of its gate and up columns:
+//   EXPERT_SILU     silu(g) u
+//   EXPERT_CLAMPED  g' sigmoid(1.702 g') (u' + 1)  with g' = min(g, limit), u' = u clamped to [-limit, limit]
+enum { EXPERT_SILU = 0, EXPERT_CLAMPED = 1 };
+struct ExpertAct {
+  int kind;
+  float limit;
+};
+__device__ __forceinline__ float expert_act(const ExpertAct& a, float g, float u) {
+  if (a.kind == EXPERT_SILU) return silu_f(g) * u;
+  g = fminf(g, a.limit), u = fminf(fmaxf(u, -a.limit), a.limit);
+  return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
 
 // A wave a token, up to ROUTER_PER_LANE outputs a lane.  The k-th pick is the largest choice score
 // not picked yet, the lowest index on a tie.
@@ -155,7 +170,7 @@ __global__ __launch_bounds__(256) void expert_rows_up_kernel(const T* __restrict
                                                              const T* __restrict__ w_gate, const T* __restrict__ w_up,
                                                              const int* __restrict__ idx,
                                                              const float* __restrict__ weight, int n_experts, int top,
-                                                             int F, int width, T* __restrict__ act) {
+                                                             int F, int width, T* __restrict__ act, ExpertAct fn) {
   const int item = blockIdx.x, t = item / top;
   const int e = idx[item];
   if (e >= n_experts) return;  // an identity expert: nothing to compute
@@ -178,7 +193,7 @@ __global__ __launch_bounds__(256) void expert_rows_up_kernel(const T* __restrict
 #pragma unroll
     for (int r = 1; r < 4; ++r)
       if (lane == r) g = s[r], u = s[4 + r];
-    act[(size_t)item * F + f0 + lane] = from_f32<T>(wt * silu_f(g) * u);
+    act[(size_t)item * F + f0 + lane] = from_f32<T>(wt * expert_act(fn, g, u));
   }
 }
 
@@ -305,7 +320,7 @@ __global__ __launch_bounds__(256) void expert_tiles_up_kernel(const T* __restric
                                                               const T* __restrict__ w_up, const int* __restrict__ order,
                                                               const int* __restrict__ tiles, const int* __restrict__ n_tiles,
                                                               const float* __restrict__ weight, int top, int F, int width,
-                                                              T* __restrict__ act) {
+                                                              T* __restrict__ act, ExpertAct fn) {
   typedef Frag<T> Fr;
   if ((int)blockIdx.x >= *n_tiles) return;
   const int e = tiles[3 * blockIdx.x], first = tiles[3 * blockIdx.x + 1], count = tiles[3 * blockIdx.x + 2];
@@ -370,7 +385,7 @@ __global__ __launch_bounds__(256) void expert_tiles_up_kernel(const T* __restric
 #pragma unroll
       for (int c = 0; c < CF; ++c) {
         const int f = f0 + 16 * c + r;
-        if (f < F) act[(size_t)it * F + f] = from_f32<T>(wt * silu_f(ag[rg][c][i]) * au[rg][c][i]);
+        if (f < F) act[(size_t)it * F + f] = from_f32<T>(wt * expert_act(fn, ag[rg][c][i], au[rg][c][i]));
       }
     }
 }
@@ -552,12 +567,15 @@ extern "C" int act_mul(const void* gu, int ld, void* out, int ldo, int n_rows, i
 // act: [n_tokens * top, F] of the compute dtype; y: float rows.
 extern "C" int expert_rows(const void* x, int ldx, const void* w_gate, const void* w_up, const void* w_down,
                            const int* idx, const float* weight, int n_tokens, int n_experts, int top, int F, int width,
-                           void* act, float* y, int ldy, int accumulate, int dtype, hipStream_t stream) {
+                           void* act, float* y, int ldy, int accumulate, int dtype, int act_kind, float act_limit,
+                           hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (!x || !idx || !weight || !y || (n_experts > 0 && (!w_gate || !w_up || !w_down || !act)))
     FAIL("expert_rows: null pointer");
   if (top <= 0 || F <= 0 || width <= 0 || ldx < width || ldy < width) FAIL("expert_rows: sizes");
   if (dtype != DT_F32 && dtype != DT_BF16) FAIL("expert_rows: unknown dtype code %d", dtype);
+  if (act_kind != EXPERT_SILU && act_kind != EXPERT_CLAMPED) FAIL("expert_rows: unknown activation code %d", act_kind);
+  const ExpertAct fn = {act_kind, act_limit};
   const int feats = 16, cols = 16, per = dtype == DT_BF16 ? 8 : 4;
   const bool vec = F % per == 0 && width % per == 0 && ldx % per == 0 && !((uintptr_t)x & 15);
   dim3 block(256), up_grid(n_tokens * top, (F + feats - 1) / feats), down_grid(n_tokens, (width + cols - 1) / cols);
@@ -565,7 +583,7 @@ extern "C" int expert_rows(const void* x, int ldx, const void* w_gate, const voi
   do {                                                                                                                     \
     if (n_experts > 0)                                                                                                     \
       hipLaunchKernelGGL((expert_rows_up_kernel<T, VEC>), up_grid, block, 0, stream, (const T*)x, ldx, (const T*)w_gate,   \
-                         (const T*)w_up, idx, weight, n_experts, top, F, width, (T*)act);                           \
+                         (const T*)w_up, idx, weight, n_experts, top, F, width, (T*)act, fn);                       \
     hipLaunchKernelGGL((expert_rows_down_kernel<T, VEC>), down_grid, block, 0, stream, (const T*)act, (const T*)w_down,    \
                        idx, weight, (const T*)x, ldx, n_experts, top, F, width, y, ldy, accumulate);                 \
   } while (0)
@@ -593,7 +611,7 @@ extern "C" int expert_tiles_takes(int F, int width, int dtype) {
 extern "C" int expert_tiles(const void* x, int ldx, const void* w_gate, const void* w_up, const void* w_down, const int* idx,
                             const float* weight, int n_tokens, int n_experts, int top, int F, int width, int* order, int* tiles,
                             int* n_tiles, void* act, float* out, float* y, int ldy, int accumulate, int dtype,
-                            hipStream_t stream) {
+                            int act_kind, float act_limit, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (!x || !idx || !weight || !y || !w_gate || !w_up || !w_down || !order || !tiles || !n_tiles || !act || !out)
     FAIL("expert_tiles: null pointer");
@@ -602,6 +620,8 @@ extern "C" int expert_tiles(const void* x, int ldx, const void* w_gate, const vo
   if (!expert_tiles_takes(F, width, dtype)) FAIL("expert_tiles: inner size %d and width %d must be multiples of %d", F, width, dtype == DT_BF16 ? 8 : 4);
   if (n_experts > 8192) FAIL("expert_tiles: %d experts are more than the sorting block's LDS holds", n_experts);
   if (ldx % (dtype == DT_BF16 ? 8 : 4) || ((uintptr_t)x & 15)) FAIL("expert_tiles: the rows of x must be 16-byte aligned");
+  if (act_kind != EXPERT_SILU && act_kind != EXPERT_CLAMPED) FAIL("expert_tiles: unknown activation code %d", act_kind);
+  const ExpertAct fn = {act_kind, act_limit};
   const int n_items = n_tokens * top, most = expert_tiles_most(n_items, n_experts);
   hipLaunchKernelGGL(expert_sort_kernel, dim3(1), dim3(1024), 2 * n_experts * sizeof(int), stream, idx, n_items, n_experts,
                      order, tiles, n_tiles);
@@ -612,7 +632,7 @@ extern "C" int expert_tiles(const void* x, int ldx, const void* w_gate, const vo
 #define RUN(T, CF)                                                                                                       \
   do {                                                                                                                   \
     hipLaunchKernelGGL((expert_tiles_up_kernel<T, CF>), up_grid, block, 0, stream, (const T*)x, ldx, (const T*)w_gate,   \
-                       (const T*)w_up, order, tiles, n_tiles, weight, top, F, width, (T*)act);                           \
+                       (const T*)w_up, order, tiles, n_tiles, weight, top, F, width, (T*)act, fn);                       \
     hipLaunchKernelGGL((expert_tiles_down_kernel<T, CF>), down_grid, block, 0, stream, (const T*)act, (const T*)w_down,  \
                        order, tiles, n_tiles, F, width, out);                                                            \
     hipLaunchKernelGGL(expert_combine_kernel<T>, sum_grid, block, 0, stream, out, idx, weight, (const T*)x, ldx,         \

@@ -57,6 +57,11 @@ struct ScanArgs {
   int ldca, chan_logit;
   float chan_mult;
   const float* norm_w;  // [P] or null: with unit_rms, the normed output times this weight
+  int norm_stride;      // head h's weights start at norm_w + h * norm_stride (0: one weight for all heads)
+  // bonus [H * N] or null (with chan_a, the kernels that take chunks): the output reads the state ahead
+  // of the token's own decay and write, and the token itself through the bonus instead,
+  //   o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T q_t
+  const float* bonus;
 };
 
 __device__ __forceinline__ float channel_log_decay(const ScanArgs& a, size_t row, int h, int i) {
@@ -135,7 +140,7 @@ __global__ __launch_bounds__(256) void state_scan_kernel(ScanArgs a) {
     if (a.unit_rms) {
       const float ss = block_sum(tid < P ? o * o : 0.f, red);
       o *= 1.0f / sqrtf(ss / (float)P + a.eps);
-      if (a.norm_w && tid < P) o *= a.norm_w[tid];
+      if (a.norm_w && tid < P) o *= a.norm_w[(size_t)h * a.norm_stride + tid];
     }
     if (tid < P) {
       if (a.gate) o *= silu_f(a.gate[row * a.ldg + (size_t)h * P + tid]);
@@ -392,6 +397,9 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(ScanArgs a, int C, Sp
 // pair (t, j <= t) is summed as written, four lanes a pair, each a quarter of the channels, added
 // in a fixed order.  LT [Np][C + 4] holds L; afterwards QT becomes q exp(L_t) and KT becomes
 // k exp(L_C - L_j) in place, for the products with the state and into it.
+// With a bonus the queries read the state ahead of their own token: their side of every exponent is
+// L_(t-1) (zero at the chunk's first token), still <= 0 against L_j for j < t and against L_b, and
+// a pair (t, t) has the bonus in place of an exponential.
 template <typename T>
 __global__ __launch_bounds__(256) void channel_chunks_kernel(ScanArgs a, int C, SpanArgs sp) {
   extern __shared__ float lds[];
@@ -435,6 +443,9 @@ __global__ __launch_bounds__(256) void channel_chunks_kernel(ScanArgs a, int C, 
   }
   const bool outputs = sp.mode != SPAN_STATES;
   const int ct = C / 16, pt = Pp / 16, nt = Np / 16, lr = lane & 15, lg = lane >> 4;
+  const float* bonus = a.bonus ? a.bonus + (size_t)h * N : nullptr;
+  // the queries' side of an exponent: the sum up to the token, or with a bonus up to the one before
+  auto at_query = [&](const float* lrow, int t) { return !bonus ? lrow[t] : t > 0 ? lrow[t - 1] : 0.f; };
   for (int c0 = lo; c0 < n; c0 += C) {
     const int m = min(C, n - c0);
     const size_t row0 = (size_t)(start + c0);
@@ -506,7 +517,8 @@ __global__ __launch_bounds__(256) void channel_chunks_kernel(ScanArgs a, int C, 
         for (int i = part * quarter; i < (part + 1) * quarter; ++i) {
           const float* row = QT + (size_t)i * CP;
           const float* lrow = LT + (size_t)i * CP;
-          acc += row[t] * KT[(size_t)i * CP + j] * expf(lrow[t] - lrow[j]);
+          const float f = bonus && t == j ? bonus[min(i, N - 1)] : expf(at_query(lrow, t) - lrow[j]);
+          acc += row[t] * KT[(size_t)i * CP + j] * f;
         }
         acc += __shfl_xor(acc, 1);
         acc += __shfl_xor(acc, 2);
@@ -522,7 +534,7 @@ __global__ __launch_bounds__(256) void channel_chunks_kernel(ScanArgs a, int C, 
         for (int i = 0; i < Np; i += 4) {
           const size_t ro = (size_t)(i + lg) * CP;
           const float ref = LT[ro + t0 - 1];
-          const float qa = QT[ro + t0 + lr] * expf(LT[ro + t0 + lr] - ref);
+          const float qa = QT[ro + t0 + lr] * expf(at_query(LT + ro, t0 + lr) - ref);
           const float kb_ = KT[ro + j0 + lr] * expf(ref - LT[ro + j0 + lr]);
           acc = __builtin_amdgcn_mfma_f32_16x16x4f32(qa, kb_, acc, 0, 0, 0);
         }
@@ -536,7 +548,7 @@ __global__ __launch_bounds__(256) void channel_chunks_kernel(ScanArgs a, int C, 
       const int i = e / C, t = e - i * C;
       const size_t at = (size_t)i * CP + t;
       const float l = LT[at];
-      if (outputs) QT[at] *= expf(l);
+      if (outputs) QT[at] *= expf(at_query(LT + (size_t)i * CP, t));
       if (state_needed) KT[at] *= expf(LT[(size_t)i * CP + C - 1] - l);  // (from m on the sum stands still: L_C)
     }
     __syncthreads();
@@ -576,7 +588,7 @@ __global__ __launch_bounds__(256) void channel_chunks_kernel(ScanArgs a, int C, 
         if (lane == 0) Rs[t] = 1.0f / sqrtf(ss / (float)P + a.eps);
       }
     if (gates_ahead || (outputs && !a.gate && P <= 64)) {
-      const float nw = a.norm_w && a.unit_rms ? a.norm_w[min(lane, P - 1)] : 1.f;
+      const float nw = a.norm_w && a.unit_rms ? a.norm_w[(size_t)h * a.norm_stride + min(lane, P - 1)] : 1.f;
 #pragma unroll
       for (int u = 0; u < 16; ++u) {
         const int t = wave + 4 * u;
@@ -589,7 +601,7 @@ __global__ __launch_bounds__(256) void channel_chunks_kernel(ScanArgs a, int C, 
     } else {
       for (int pb = 0; outputs && pb < P; pb += 64) {
         const int pc = min(pb + lane, P - 1);
-        const float nw = a.norm_w && a.unit_rms ? a.norm_w[pc] : 1.f;
+        const float nw = a.norm_w && a.unit_rms ? a.norm_w[(size_t)h * a.norm_stride + pc] : 1.f;
         for (int tb = wave; tb < m; tb += 32) {
           float g8[8];
 #pragma unroll
@@ -747,6 +759,12 @@ static size_t channel_chunk_floats(int N, int P, int C) {
   return 3 * Np * CP + 2 * (size_t)C * Pp + (size_t)C * CP + Np * Pp + Np;
 }
 
+// 1 if chunks of tokens fit a block's LDS for a state of N x P (`by_channel`: a decay per key channel).
+extern "C" int state_chunks_takes(int N, int P, int by_channel) {
+  return N > 0 && P > 0 && P <= 256 &&
+         (by_channel ? channel_chunk_floats(N, P, 16) : chunk_floats(N, P, 16)) * sizeof(float) <= SCAN_MAX_LDS;
+}
+
 // `chunked`: the kernel that takes a chunk of tokens at a time (for steps in which some request
 // brings many tokens); otherwise, or where not even chunks of 16 fit the LDS, token by token.
 // `chunked`: 0 token by token; 1 chunks of tokens, a request a block; 2 chunks, the requests cut
@@ -764,6 +782,8 @@ extern "C" int state_scan(const ScanArgs* args, int chunked, int span, int n_spa
   if (a.Hk <= 0 || a.H % a.Hk) FAIL("state_scan: %d heads over %d key heads", a.H, a.Hk);
   if (!a.log_a && !a.decay && !a.chan_a) FAIL("state_scan: a decay per token, per head or per key channel is needed");
   if (a.chan_a && (a.ldca < a.H * a.N || a.Hk != a.H)) FAIL("state_scan: decays per key channel come in rows of heads x keys");
+  if (a.norm_stride != 0 && a.norm_stride < a.P) FAIL("state_scan: norm weights %d apart for heads of %d", a.norm_stride, a.P);
+  if (a.bonus && !a.chan_a) FAIL("state_scan: a bonus goes with decays per key channel");
   if (a.rot_dims && (a.rot_dims % 2 || a.rot_dims > a.N || !a.inv_freq || !a.positions))
     FAIL("state_scan: %d turning columns of %d", a.rot_dims, a.N);
   if (a.ldq < a.Hk * a.N || a.ldk < a.Hk * a.N || a.ldv < a.H * a.P || a.ldo < a.H * a.P || (a.gate && a.ldg < a.H * a.P))
@@ -832,6 +852,7 @@ extern "C" int state_scan(const ScanArgs* args, int chunked, int span, int n_spa
     CHECK_LAUNCH("state_scan");
     return 0;
   }
+  if (a.bonus) FAIL("state_scan: a bonus is for the kernels that take chunks; a state of %d x %d does not fit them", a.N, a.P);
   if (a.out_dtype == DT_F32)
     hipLaunchKernelGGL(state_scan_kernel<float>, grid, block, lds, stream, a);
   else

@@ -539,6 +539,55 @@ def linear(out, a, w, bias=None, gelu=False, accumulate=False, variant=0, scatte
     return out
 
 
+class GroupedWeight:
+    """Several weight matrices ``[n_i, K]`` that read different inputs of one shape (``planes``), for one
+    product: ``groups`` is a list of ``(weight, plane)``.  The matrices lie one after the other, each
+    padded with zero rows to whole blocks of ``BLOCK`` features, so that a block of a product kernel
+    reads one plane only; ``columns`` are each one's first column and width in the product's rows."""
+
+    BLOCK = 32
+
+    def __init__(self, groups):
+        K = groups[0][0].shape[1]
+        parts, self.columns, self.planes, at = [], [], [], 0
+        for w, plane in groups:
+            _need(w.dim() == 2 and w.shape[1] == K and w.dtype == groups[0][0].dtype, "GroupedWeight: matrices of one width and dtype")
+            n = w.shape[0]
+            pad = -n % self.BLOCK
+            parts += [w, w.new_zeros(pad, K)] if pad else [w]
+            self.columns.append((at, n))
+            self.planes.append(int(plane))
+            at += n + pad
+        whole = torch.cat(parts).contiguous()
+        self.N, self.K, self.dtype = at, K, whole.dtype
+        self.w = for_decode(whole)
+        # each group by itself, over the same memory: whole blocks of sixteen features of the packed order
+        self.parts = [self._slice(start, (n + 15) // 16 * 16 if isinstance(self.w, PackedWeight) else n, n) for start, n in self.columns]
+
+    def _slice(self, start, padded, n):
+        if not isinstance(self.w, PackedWeight):
+            return self.w[start : start + n]
+        part = PackedWeight.__new__(PackedWeight)
+        tile_row = (self.K + 63) // 64 * 1024  # elements of sixteen features
+        part.w, part.shape, part.dtype, part.device = None, (n, self.K), self.w.dtype, self.w.device
+        part.packed = self.w.packed[start // 16 * tile_row : (start + padded) // 16 * tile_row]
+        part.chunk_bytes, part.n_chunks = self.w.chunk_bytes, padded // 16
+        part.c = native.EngWeight(None, part.packed.data_ptr(), n, self.K, 0, DT[part.dtype], part.chunk_bytes, part.n_chunks, 0)
+        return part
+
+
+def linear_groups(alloc, planes, w):
+    """The products of a ``GroupedWeight``: for every group its float32 rows ``planes[plane] @ weight.T``.
+    ``planes`` is contiguous ``[n, rows, K]``; the rows lie in memory that ``alloc(shape, dtype)`` gives."""
+    T = planes.shape[1]
+    _need(planes.is_contiguous() and planes.shape[2] == w.K and planes.dtype == w.dtype, "linear_groups: shapes")
+    rows = alloc((T, w.N), torch.float32)
+    out = [rows[:, a : a + n] for a, n in w.columns]
+    for view, plane, part in zip(out, w.planes, w.parts):
+        linear(view, planes[plane], part, splits=splits_alone(T))
+    return out
+
+
 # ---------------------------------------------------------------------------
 
 
@@ -959,7 +1008,7 @@ class ScanArgs(ctypes.Structure):
                 ("state", _vp), ("state_stride", _c_size_t), ("state_offset", _c_size_t), ("seq_start", _vp),
                 ("seq_len", _vp), ("slot_ids", _vp), ("n_requests", _c_int), ("H", _c_int), ("Hk", _c_int),
                 ("N", _c_int), ("P", _c_int), ("n_tokens_hint", _c_int), ("chan_a", _vp), ("ldca", _c_int),
-                ("chan_logit", _c_int), ("chan_mult", _c_float), ("norm_w", _vp)]
+                ("chan_logit", _c_int), ("chan_mult", _c_float), ("norm_w", _vp), ("norm_stride", _c_int), ("bonus", _vp)]
 
 
 def _f32_rows(t, name, min_cols):
@@ -972,7 +1021,7 @@ def _f32_rows(t, name, min_cols):
 def state_scan(out, q, k, v, state, state_offset, seq_start, seq_len, slot_ids, n_requests, n_heads, n_key_heads,
                key_dim, value_dim, log_a=None, decay=None, k_scale=None, k_mult=1.0, skip=None, rot_dims=0,
                inv_freq=None, positions=None, unit_rms=False, eps=0.0, gate=None, chunked=False, spans=None,
-               channel_decay=None, channel_logit_mult=None, norm_weight=None):
+               channel_decay=None, channel_logit_mult=None, norm_weight=None, bonus=None):
     """``S = a S + k v^T; o = S^T q`` token by token for every (request, head), from and into the
     requests' rows of ``state`` (float32 ``[slots, floats a request]``, head ``h``'s matrix
     ``[key_dim, value_dim]`` at ``state_offset + h * key_dim * value_dim``).  ``q``, ``k``
@@ -988,7 +1037,9 @@ def state_scan(out, q, k, v, state, state_offset, seq_start, seq_len, slot_ids, 
     ``channel_decay`` (float32 ``[tokens, >= n_heads * key_dim]``): a decay for every key channel
     instead of one a head, given as its logarithm, or, with ``channel_logit_mult = m``, as a logit
     ``z`` with ``log a = m * log sigmoid(z)``.  ``norm_weight`` (float32 ``[value_dim]``): with
-    ``unit_rms``, the normed output times this weight, the same for every head.
+    ``unit_rms``, the normed output times this weight, the same for every head (``[n_heads *
+    value_dim]``: a weight of its own for every head).  ``bonus`` (float32 ``[n_heads * key_dim]``,
+    with ``channel_decay`` and ``chunked``): ``o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T q_t``.
     See csrc/linear_state.hip for the options."""
     lib = build.load("linear_state")
     a = ScanArgs()
@@ -1017,8 +1068,12 @@ def state_scan(out, q, k, v, state, state_offset, seq_start, seq_len, slot_ids, 
             a.chan_logit, a.chan_mult = 1, float(channel_logit_mult)
     if norm_weight is not None:
         _dev(norm_weight, "norm_weight", torch.float32)
-        _need(unit_rms and norm_weight.numel() == value_dim, "state_scan: norm_weight has value_dim values and goes with unit_rms")
-        a.norm_w = norm_weight.data_ptr()
+        _need(unit_rms and norm_weight.numel() in (value_dim, n_heads * value_dim), "state_scan: norm_weight has value_dim values (a head) and goes with unit_rms")
+        a.norm_w, a.norm_stride = norm_weight.data_ptr(), value_dim if norm_weight.numel() != value_dim else 0
+    if bonus is not None:
+        _dev(bonus, "bonus", torch.float32)
+        _need(channel_decay is not None and chunked and bonus.numel() == n_heads * key_dim, "state_scan: a bonus for every key channel")
+        a.bonus = bonus.data_ptr()
     a.k_mult = float(k_mult)
     if rot_dims:
         _dev(inv_freq, "inv_freq", torch.float32)
@@ -1361,11 +1416,20 @@ def silu_mul(out, gate_up, activation="silu"):
     return out
 
 
-def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=True):
+EXPERT_ACTIVATIONS = {"silu": 0, "clamped": 1}
+
+
+def _expert_activation(activation, limit):
+    _need(activation in EXPERT_ACTIVATIONS, f"experts: activation {activation!r} (known: {sorted(EXPERT_ACTIVATIONS)})")
+    return _c_int(EXPERT_ACTIVATIONS[activation]), _c_float(limit)
+
+
+def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=True, activation="silu", limit=0.0):
     """``y (+)= sum over a token's picks of weight * expert(x)``, reading only the picked experts'
     weights (``w_gate``, ``w_up``: ``[experts, F, width]``, ``w_down``: ``[experts, width, F]``); a
     pick at or beyond the number of experts gives ``weight * x``.  ``act``: room for ``[tokens *
-    top, F]`` of ``x``'s dtype."""
+    top, F]`` of ``x``'s dtype.  ``activation``: ``silu(g) * u``, or ``clamped``: ``g sigmoid(1.702 g) (u
+    + 1)`` with ``g`` at most ``limit`` and ``u`` within ``[-limit, limit]``."""
     lib = build.load("experts")
     ldx, ldy = _rows2d(x, "x"), _rows2d(y, "y")
     T, width = x.shape
@@ -1384,7 +1448,8 @@ def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=Tr
     _need(idx.numel() >= T * top and weight.numel() >= T * top, "expert_rows: idx / weight too short")
     rc = lib.expert_rows(_ptr(x), _c_int(ldx), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _ptr(idx), _ptr(weight),
                          _c_int(T), _c_int(n_experts), _c_int(top), _c_int(F), _c_int(width), _ptr(act), _ptr(y),
-                         _c_int(ldy), _c_int(int(bool(accumulate))), _c_int(DT[x.dtype]), _stream())
+                         _c_int(ldy), _c_int(int(bool(accumulate))), _c_int(DT[x.dtype]),
+                         *_expert_activation(activation, limit), _stream())
     build.check(lib, rc, "expert_rows")
     return y
 
@@ -1394,7 +1459,7 @@ def expert_tiles_takes(inner, width, dtype):
     return bool(build.load("experts").expert_tiles_takes(_c_int(inner), _c_int(width), _c_int(DT[dtype])))
 
 
-def expert_tiles(y, x, w_gate, w_up, w_down, idx, weight, top, alloc, accumulate=True):
+def expert_tiles(y, x, w_gate, w_up, w_down, idx, weight, top, alloc, accumulate=True, activation="silu", limit=0.0):
     """What ``expert_rows`` computes, for many tokens: the picks are sorted by expert on the device
     and every tile of up to 64 picks of one expert is a small product on the matrix cores.
     ``alloc(shape, dtype)`` gives the work memory (the sorted list, the tiles, the activations
@@ -1417,7 +1482,7 @@ def expert_tiles(y, x, w_gate, w_up, w_down, idx, weight, top, alloc, accumulate
     rc = lib.expert_tiles(_ptr(x), _c_int(ldx), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _ptr(idx), _ptr(weight), _c_int(T),
                           _c_int(n_experts), _c_int(top), _c_int(F), _c_int(width), _ptr(order), _ptr(tiles), _ptr(n_tiles),
                           _ptr(act), _ptr(out), _ptr(y), _c_int(ldy), _c_int(int(bool(accumulate))), _c_int(DT[x.dtype]),
-                          _stream())
+                          *_expert_activation(activation, limit), _stream())
     build.check(lib, rc, "expert_tiles")
     return y
 
@@ -1548,4 +1613,316 @@ def normed_gate(out, y, gate, weight, eps):
     rc = lib.normed_gate(_ptr(y), _c_int(ldy), _ptr(gate), _c_int(ldg), _ptr(weight), _c_float(eps), _c_int(n), _c_int(width),
                          _ptr(out), _c_int(ldo), _c_int(DT[out.dtype]), _stream())
     build.check(lib, rc, "normed_gate")
+    return out
+
+
+# ---------------------------------------------------------------------------
+# a norm without statistics, and the token shift behind it (csrc/dynamic_tanh.hip)
+
+
+class TokenMixArgs(ctypes.Structure):
+    """Mirror of ``TokenMixArgs`` in csrc/dynamic_tanh.hip."""
+
+    _fields_ = [("x", _vp), ("ldx", _c_int), ("n_rows", _c_int), ("width", _c_int), ("alpha", _vp), ("w", _vp), ("b", _vp),
+                ("mu", _vp), ("n_mix", _c_int), ("out", _vp), ("state", _vp), ("state_stride", _c_size_t),
+                ("state_offset", _c_size_t), ("token_req", _vp), ("seq_start", _vp), ("seq_len", _vp), ("slot_ids", _vp)]
+
+
+def _tanh_norm(norm, width):
+    """The device pointers of a norm given as ``(alpha, weight, shift)``, float32."""
+    for name, t, n in zip(("alpha", "weight", "shift"), norm, (1, width, width)):
+        _dev(t, name, torch.float32)
+        t.numel() == n or _fail(f"dynamic_tanh: {name} has {t.numel()} values, want {n}")
+    return [_ptr(t) for t in norm]
+
+
+def dynamic_tanh(out, x, norm):
+    """``out = tanh(alpha * x) * weight + shift`` over float32 rows; ``norm = (alpha, weight, shift)``;
+    ``out`` float32 or bfloat16, contiguous."""
+    lib = build.load("dynamic_tanh")
+    n, width = out.shape
+    ldx = _f32_rows(x, "x", width)
+    _need(out.is_contiguous() and out.dtype in DT and x.shape[0] >= n, "dynamic_tanh: shapes")
+    rc = lib.dynamic_tanh(_ptr(out), _ptr(x), _c_int(ldx), None, *_tanh_norm(norm, width), _c_int(n), _c_int(width),
+                          _c_int(DT[out.dtype]), _stream())
+    build.check(lib, rc, "dynamic_tanh")
+    return out
+
+
+def embed_dynamic_tanh(out, table, ids, scale, norm):
+    """``out[t] = tanh(alpha * scale * table[ids[t]]) * weight + shift`` into float32 ``out``."""
+    lib = build.load("dynamic_tanh")
+    n, width = out.shape
+    _dev(out, "out", torch.float32)
+    _dev(table, "table")
+    _dev(ids, "ids", torch.int32)
+    _need(table.dtype in DT and table.shape[1] == width and ids.numel() >= n, "embed_dynamic_tanh: shapes")
+    rc = lib.embed_dynamic_tanh(_ptr(out), _ptr(table), _c_int(DT[table.dtype]), _ptr(ids), _c_float(scale),
+                                *_tanh_norm(norm, width), _c_int(n), _c_int(width), _stream())
+    build.check(lib, rc, "embed_dynamic_tanh")
+    return out
+
+
+def token_mix(out, x, norm, mu, state, state_offset, token_req, seq_start, seq_len, slot_ids):
+    """The rows ``h`` of a dynamic-tanh norm over the float32 stream ``x`` into ``out[0]`` and ``h + (h' -
+    h) * mu[m]`` into ``out[1 + m]``, where ``h'`` is the row before in the same sequence (zeros ahead
+    of the first; from the request's row of ``state`` at ``state_offset`` where it came in an earlier
+    step).  ``out`` contiguous ``[1 + n_mix, rows, width]``, float32 or bfloat16; ``mu`` float32
+    ``[n_mix, width]``.  The requests' last normed rows are left in ``state``."""
+    lib = build.load("dynamic_tanh")
+    planes, n, width = out.shape
+    a = TokenMixArgs()
+    a.ldx, a.x = _f32_rows(x, "x", width), x.data_ptr()
+    _need(out.is_contiguous() and out.dtype in DT and x.shape[0] >= n and token_req.numel() >= n, "token_mix: shapes")
+    a.n_rows, a.width, a.n_mix, a.out = n, width, planes - 1, out.data_ptr()
+    _dev(mu, "mu", torch.float32)
+    _need(tuple(mu.shape) == (planes - 1, width), "token_mix: a row of mu a mix")
+    a.mu = mu.data_ptr()
+    a.alpha, a.w, a.b = (p.value for p in _tanh_norm(norm, width))
+    _dev(state, "state", torch.float32)
+    _need(state.dim() == 2 and state_offset + width <= state.shape[1], "token_mix: the state rows are too short")
+    a.state, a.state_stride, a.state_offset = state.data_ptr(), state.stride(0), int(state_offset)
+    for name, t in (("token_req", token_req), ("seq_start", seq_start), ("seq_len", seq_len), ("slot_ids", slot_ids)):
+        _dev(t, name, torch.int32)
+        setattr(a, name, t.data_ptr())
+    rc = lib.token_mix(ctypes.byref(a), _c_int(DT[out.dtype]), _stream())
+    build.check(lib, rc, "token_mix")
+    return out
+
+
+# ---------------------------------------------------------------------------
+# recurrences over a matrix state for steps of few tokens (csrc/state_step.hip)
+
+
+class StepArgs(ctypes.Structure):
+    """Mirror of ``StepArgs`` in csrc/state_step.hip."""
+
+    _fields_ = [("q", _vp), ("k", _vp), ("v", _vp), ("ldq", _c_int), ("ldk", _c_int), ("ldv", _c_int), ("qk_stride", _c_int),
+                ("v_stride", _c_int), ("gate", _vp), ("ldg", _c_int), ("norm_w", _vp), ("norm_stride", _c_int), ("eps", _c_float),
+                ("out", _vp), ("ldo", _c_int), ("out_dtype", _c_int), ("state", _vp), ("state_stride", _c_size_t),
+                ("state_offset", _c_size_t), ("seq_start", _vp), ("seq_len", _vp), ("slot_ids", _vp), ("n_requests", _c_int),
+                ("H", _c_int), ("Hk", _c_int), ("N", _c_int), ("P", _c_int), ("mode", _c_int), ("log_g", _vp), ("beta", _vp),
+                ("ld_gb", _c_int), ("A_log", _vp), ("dt_bias", _vp), ("conv_w", _vp), ("taps", _c_int), ("ring_offset", _c_size_t),
+                ("positions", _vp), ("q_scale", _c_float), ("z", _vp), ("ldz", _c_int), ("rank", _c_int), ("w2_dtype", _c_int),
+                ("w2t", _vp), ("w0", _vp), ("bonus", _vp)]
+
+
+STEP_DELTA, STEP_DELTA_RAW, STEP_BONUS = 0, 1, 2
+
+
+class DeltaRaw:
+    """What ``state_step`` needs to make the delta rule's operands from the projection's own columns:
+    the convolution's weights (float32 ``[channels, taps]``, channels of queries, keys and values in
+    this order), where its ring of inputs starts in a request's state row (``[taps, channels]``,
+    position ``p`` in row ``p % taps``), ``A_log`` and ``dt_bias`` a head, the queries' factor."""
+
+    def __init__(self, conv_w, ring_offset, a_log, dt_bias, q_scale):
+        for name, t in (("conv_w", conv_w), ("a_log", a_log), ("dt_bias", dt_bias)):
+            _dev(t, name, torch.float32)
+        self.conv_w, self.ring_offset, self.a_log, self.dt_bias, self.q_scale = conv_w, int(ring_offset), a_log, dt_bias, float(q_scale)
+
+
+class LowRankDecay:
+    """A decay per key channel through a narrow middle, ``log w = -exp(w0 + W2 tanh(z))``: ``w2t`` is
+    ``W2`` transposed, ``[rank, channels]`` (float32 or bfloat16), ``w0`` float32 a channel."""
+
+    def __init__(self, w2t, w0):
+        _dev(w2t, "w2t")
+        _dev(w0, "w0", torch.float32)
+        _need(w2t.dtype in DT and w2t.dim() == 2 and w0.numel() == w2t.shape[1], "LowRankDecay: a row a middle column")
+        self.w2t, self.w0, self.rank, self.width = w2t, w0, w2t.shape[0], w2t.shape[1]
+
+
+def lowrank_decay(log_w, z, decay):
+    """``log_w[t] = -exp(w0 + W2 tanh(z[t]))`` (float32 ``[rows, channels]``)."""
+    lib = build.load("state_step")
+    ldz = _f32_rows(z, "z", decay.rank)
+    _dev(log_w, "log_w", torch.float32)
+    _need(log_w.shape[1] == decay.width and z.shape[0] >= log_w.shape[0], "lowrank_decay: shapes")
+    rc = lib.lowrank_decay(_ptr(z), _c_int(ldz), _c_int(decay.rank), _ptr(decay.w2t), _c_int(DT[decay.w2t.dtype]), _ptr(decay.w0),
+                           _c_int(decay.width), _ptr(log_w), _c_int(log_w.shape[0]), _stream())
+    build.check(lib, rc, "lowrank_decay")
+    return log_w
+
+
+def state_step_takes(key_dim, value_dim):
+    """Whether ``state_step`` holds a head's state of these sizes in a block's registers."""
+    return bool(build.load("state_step").state_step_takes(_c_int(key_dim), _c_int(value_dim)))
+
+
+def state_step(out, q, k, v, state, state_offset, seq_start, seq_len, slot_ids, n_requests, n_heads, n_key_heads, key_dim,
+               value_dim, norm_weight, eps, gate=None, qk_stride=None, v_stride=None, log_g=None, beta=None, raw=None,
+               positions=None, z=None, decay=None, bonus=None):
+    """A recurrence over a matrix state token by token, a block a (head, request), the state in
+    registers; the heads' output divided by its root mean square, times ``norm_weight`` (``value_dim``
+    values, or that many a head) and ``silu(gate)``.
+
+    * the gated delta rule ``S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q`` on prepared
+      rows: ``log_g``, ``beta`` float32 ``[rows, n_heads]``;
+    * with ``raw`` (a ``DeltaRaw``; every request brings one token) the same from the projection's
+      columns, ``beta`` and ``log_g`` the columns that become them (convolution, silu, unit vectors,
+      ``beta = sigmoid(.)``, ``g = exp(-exp(A_log) softplus(. + dt_bias))``);
+    * with ``decay`` (a ``LowRankDecay`` over ``z``, float32 ``[rows, >= rank]``) and ``bonus``: ``o =
+      (S + diag(bonus) k v^T)^T q; S <- diag(w) S + k v^T``.
+
+    Key head ``h`` at column ``h * qk_stride``, value head at ``h * v_stride`` (default: side by side)."""
+    lib = build.load("state_step")
+    a = StepArgs()
+    T = out.shape[0]
+    qs, vstr = key_dim if qk_stride is None else qk_stride, value_dim if v_stride is None else v_stride
+    a.ldq, a.ldk = (_f32_rows(t, n, (n_key_heads - 1) * qs + key_dim) for t, n in ((q, "q"), (k, "k")))
+    a.ldv = _f32_rows(v, "v", (n_heads - 1) * vstr + value_dim)
+    _need(q.shape[0] >= T and k.shape[0] >= T and v.shape[0] >= T, "state_step: fewer operand rows than output rows")
+    a.q, a.k, a.v, a.qk_stride, a.v_stride = q.data_ptr(), k.data_ptr(), v.data_ptr(), int(qs), int(vstr)
+    if gate is not None:
+        a.ldg, a.gate = _f32_rows(gate, "gate", n_heads * value_dim), gate.data_ptr()
+    _dev(norm_weight, "norm_weight", torch.float32)
+    _need(norm_weight.numel() in (value_dim, n_heads * value_dim), "state_step: norm_weight has value_dim values (a head)")
+    a.norm_w, a.norm_stride, a.eps = norm_weight.data_ptr(), value_dim if norm_weight.numel() != value_dim else 0, float(eps)
+    a.ldo = _rows2d(out, "out")
+    _need(out.dtype in DT and out.shape[1] == n_heads * value_dim, "state_step: out is [tokens, heads * value_dim]")
+    a.out, a.out_dtype = out.data_ptr(), DT[out.dtype]
+    _dev(state, "state", torch.float32)
+    _need(state.dim() == 2 and state_offset + n_heads * key_dim * value_dim <= state.shape[1], "state_step: the state rows are too short")
+    a.state, a.state_stride, a.state_offset = state.data_ptr(), state.stride(0), int(state_offset)
+    for name, t in (("seq_start", seq_start), ("seq_len", seq_len), ("slot_ids", slot_ids)):
+        _dev(t, name, torch.int32)
+        _need(t.numel() >= n_requests, f"state_step: {name} is shorter than the requests")
+        setattr(a, name, t.data_ptr())
+    a.n_requests, a.H, a.Hk, a.N, a.P = int(n_requests), int(n_heads), int(n_key_heads), int(key_dim), int(value_dim)
+    if decay is not None:
+        a.mode = STEP_BONUS
+        _need(decay.width == n_heads * key_dim and n_key_heads == n_heads, "state_step: a decay for every key channel")
+        a.ldz, a.z = _f32_rows(z, "z", decay.rank), z.data_ptr()
+        a.rank, a.w2_dtype, a.w2t, a.w0 = decay.rank, DT[decay.w2t.dtype], decay.w2t.data_ptr(), decay.w0.data_ptr()
+        _dev(bonus, "bonus", torch.float32)
+        _need(bonus.numel() == n_heads * key_dim and z.shape[0] >= T, "state_step: a bonus for every key channel")
+        a.bonus = bonus.data_ptr()
+    else:
+        ld = _f32_rows(log_g, "log_g", n_heads)
+        _need(_f32_rows(beta, "beta", n_heads) == ld and log_g.shape[0] >= T and beta.shape[0] >= T, "state_step: log_g and beta are rows of one stride")
+        a.log_g, a.beta, a.ld_gb, a.mode = log_g.data_ptr(), beta.data_ptr(), ld, STEP_DELTA
+        if raw is not None:
+            channels, taps = raw.conv_w.shape
+            _dev(positions, "positions", torch.int32)
+            _need(channels == 2 * n_key_heads * key_dim + n_heads * value_dim and raw.a_log.numel() == n_heads
+                  and raw.dt_bias.numel() == n_heads and positions.numel() >= T, "state_step: the convolution's channels, gates a head")
+            _need(taps == 1 or raw.ring_offset + taps * channels <= state.shape[1], "state_step: the state rows are too short")
+            a.mode, a.conv_w, a.taps, a.ring_offset = STEP_DELTA_RAW, raw.conv_w.data_ptr(), taps, raw.ring_offset
+            a.A_log, a.dt_bias, a.positions, a.q_scale = raw.a_log.data_ptr(), raw.dt_bias.data_ptr(), positions.data_ptr(), raw.q_scale
+    rc = lib.state_step(ctypes.byref(a), _stream())
+    build.check(lib, rc, "state_step")
+    return out
+
+
+def state_chunks_takes(key_dim, value_dim, by_channel=True):
+    """Whether ``state_scan``'s kernels that take chunks of tokens hold a state of these sizes."""
+    return bool(build.load("linear_state").state_chunks_takes(_c_int(key_dim), _c_int(value_dim), _c_int(int(by_channel))))
+
+
+# ---------------------------------------------------------------------------
+# the gated delta rule for portions of many tokens (csrc/delta_chunks.hip)
+
+
+class DeltaPrepareArgs(ctypes.Structure):
+    """Mirror of ``DeltaPrepareArgs`` in csrc/delta_chunks.hip."""
+
+    _fields_ = [("u", _vp), ("ldu", _c_int), ("b_col", _c_int), ("a_col", _c_int), ("n_rows", _c_int), ("H", _c_int), ("Hk", _c_int),
+                ("N", _c_int), ("P", _c_int), ("conv_w", _vp), ("taps", _c_int), ("A_log", _vp), ("dt_bias", _vp), ("q_scale", _c_float),
+                ("state", _vp), ("state_stride", _c_size_t), ("ring_offset", _c_size_t), ("token_req", _vp), ("positions", _vp),
+                ("seq_start", _vp), ("seq_len", _vp), ("slot_ids", _vp), ("q", _vp), ("k", _vp), ("v", _vp), ("log_g", _vp), ("beta", _vp)]
+
+
+class DeltaChunkArgs(ctypes.Structure):
+    """Mirror of ``DeltaChunkArgs`` in csrc/delta_chunks.hip."""
+
+    _fields_ = [("q", _vp), ("k", _vp), ("v", _vp), ("log_g", _vp), ("beta", _vp), ("cum", _vp), ("w", _vp), ("u", _vp), ("states", _vp),
+                ("state", _vp), ("state_stride", _c_size_t), ("state_offset", _c_size_t), ("span_req", _vp), ("span_start", _vp),
+                ("span_first", _vp), ("seq_start", _vp), ("seq_len", _vp), ("slot_ids", _vp), ("n_chunks", _c_int), ("n_requests", _c_int),
+                ("H", _c_int), ("Hk", _c_int), ("N", _c_int), ("P", _c_int), ("norm_w", _vp), ("norm_stride", _c_int), ("eps", _c_float),
+                ("gate", _vp), ("ldg", _c_int), ("out", _vp), ("ldo", _c_int), ("out_dtype", _c_int)]
+
+
+DELTA_CHUNK = 64  # tokens a chunk
+
+
+def _sixteens(n):
+    return (n + 15) // 16 * 16
+
+
+def delta_prepare(alloc, u, b_col, a_col, n_heads, n_key_heads, key_dim, value_dim, raw, state, token_req, positions, seq_start,
+                  seq_len, slot_ids):
+    """The delta rule's operands from the projection's float32 rows ``u`` (queries, keys and values from
+    column 0 on, the columns that become ``beta`` and ``g`` from ``b_col`` and ``a_col``): ``(q, k, v,
+    log_g, beta)`` in memory that ``alloc(shape, dtype)`` gives, heads padded by zeros to multiples of
+    sixteen columns.  ``raw``: a ``DeltaRaw``.  The requests' last inputs go to their rings."""
+    lib = build.load("delta_chunks")
+    T = u.shape[0]
+    channels, taps = raw.conv_w.shape
+    a = DeltaPrepareArgs()
+    a.ldu, a.u = _f32_rows(u, "u", max(channels, b_col + n_heads, a_col + n_heads)), u.data_ptr()
+    _need(channels == 2 * n_key_heads * key_dim + n_heads * value_dim and raw.a_log.numel() == n_heads
+          and raw.dt_bias.numel() == n_heads, "delta_prepare: the convolution's channels, gates a head")
+    _dev(state, "state", torch.float32)
+    _need(state.dim() == 2 and (taps == 1 or raw.ring_offset + taps * channels <= state.shape[1]), "delta_prepare: the state rows are too short")
+    a.b_col, a.a_col, a.n_rows, a.H, a.Hk, a.N, a.P = int(b_col), int(a_col), T, int(n_heads), int(n_key_heads), int(key_dim), int(value_dim)
+    a.conv_w, a.taps, a.A_log, a.dt_bias, a.q_scale = raw.conv_w.data_ptr(), taps, raw.a_log.data_ptr(), raw.dt_bias.data_ptr(), raw.q_scale
+    a.state, a.state_stride, a.ring_offset = state.data_ptr(), state.stride(0), raw.ring_offset
+    for name, t, n in (("token_req", token_req, T), ("positions", positions, T), ("seq_start", seq_start, 1), ("seq_len", seq_len, 1),
+                       ("slot_ids", slot_ids, 1)):
+        _dev(t, name, torch.int32)
+        _need(t.numel() >= n, f"delta_prepare: {name} too short")
+        setattr(a, name, t.data_ptr())
+    q, k = (alloc((T, n_key_heads * _sixteens(key_dim)), torch.float32) for _ in range(2))
+    v = alloc((T, n_heads * _sixteens(value_dim)), torch.float32)
+    log_g, beta = alloc((T, n_heads), torch.float32), alloc((T, n_heads), torch.float32)
+    a.q, a.k, a.v, a.log_g, a.beta = (t.data_ptr() for t in (q, k, v, log_g, beta))
+    rc = lib.delta_prepare(ctypes.byref(a), _stream())
+    build.check(lib, rc, "delta_prepare")
+    return q, k, v, log_g, beta
+
+
+def delta_chunks_takes(key_dim, value_dim):
+    return bool(build.load("delta_chunks").delta_chunks_takes(_c_int(key_dim), _c_int(value_dim)))
+
+
+def delta_chunks(out, operands, state, state_offset, spans, seq_start, seq_len, slot_ids, n_requests, n_heads, n_key_heads, key_dim,
+                 value_dim, norm_weight, eps, gate, alloc):
+    """The gated delta rule over ``operands`` (what ``delta_prepare`` returned) in chunks of 64 tokens;
+    the rest as in ``state_step``.  ``spans``: ``(number of chunks, request of each, its first token
+    counted from the request's first of this step, every request's first chunk)``, int32 on the device."""
+    lib = build.load("delta_chunks")
+    q, k, v, log_g, beta = operands
+    n_chunks, span_req, span_start, span_first = spans
+    T, Np, Pp = out.shape[0], _sixteens(key_dim), _sixteens(value_dim)
+    a = DeltaChunkArgs()
+    for name, t, shape in (("q", q, (T, n_key_heads * Np)), ("k", k, (T, n_key_heads * Np)), ("v", v, (T, n_heads * Pp)),
+                           ("log_g", log_g, (T, n_heads)), ("beta", beta, (T, n_heads))):
+        _dev(t, name, torch.float32)
+        _need(tuple(t.shape) == shape, f"delta_chunks: {name} is {tuple(t.shape)}, want {shape}")
+        setattr(a, name, t.data_ptr())
+    work = {"cum": alloc((T, n_heads), torch.float32), "w": alloc((T, n_heads * Np), torch.float32),
+            "u": alloc((T, n_heads * Pp), torch.float32), "states": alloc((n_chunks, n_heads, Np, Pp), torch.float32)}
+    for name, t in work.items():
+        setattr(a, name, t.data_ptr())
+    _dev(state, "state", torch.float32)
+    _need(state.dim() == 2 and state_offset + n_heads * key_dim * value_dim <= state.shape[1], "delta_chunks: the state rows are too short")
+    a.state, a.state_stride, a.state_offset = state.data_ptr(), state.stride(0), int(state_offset)
+    for name, t, n in (("span_req", span_req, n_chunks), ("span_start", span_start, n_chunks), ("span_first", span_first, n_requests),
+                       ("seq_start", seq_start, n_requests), ("seq_len", seq_len, n_requests), ("slot_ids", slot_ids, n_requests)):
+        _dev(t, name, torch.int32)
+        _need(t.numel() >= n, f"delta_chunks: {name} too short")
+        setattr(a, name, t.data_ptr())
+    a.n_chunks, a.n_requests, a.H, a.Hk, a.N, a.P = int(n_chunks), int(n_requests), int(n_heads), int(n_key_heads), int(key_dim), int(value_dim)
+    _dev(norm_weight, "norm_weight", torch.float32)
+    _need(norm_weight.numel() in (value_dim, n_heads * value_dim), "delta_chunks: norm_weight has value_dim values (a head)")
+    a.norm_w, a.norm_stride, a.eps = norm_weight.data_ptr(), value_dim if norm_weight.numel() != value_dim else 0, float(eps)
+    if gate is not None:
+        a.ldg, a.gate = _f32_rows(gate, "gate", n_heads * value_dim), gate.data_ptr()
+        _need(gate.shape[0] >= T, "delta_chunks: fewer gate rows than output rows")
+    a.ldo = _rows2d(out, "out")
+    _need(out.dtype in DT and out.shape[1] == n_heads * value_dim, "delta_chunks: out is [tokens, heads * value_dim]")
+    a.out, a.out_dtype = out.data_ptr(), DT[out.dtype]
+    rc = lib.delta_chunks(ctypes.byref(a), _stream())
+    build.check(lib, rc, "delta_chunks")
     return out

@@ -137,6 +137,47 @@ class Mixer(Part):
         raise NotImplementedError
 
 
+class ProjectsFirst:
+    """What a mixer adds to start with one product of the layer's norm into float32 rows that an
+    arrangement may hand to others too.  ``input_names()`` are the tensors whose rows, in this order,
+    are the mixer's own columns; ``more_names`` (set by the arrangement before the weights are loaded)
+    those of another part that reads the same norm, a feed-forward's router, whose product then costs
+    no launch of its own.  ``project`` gives ``(normed rows, the mixer's columns, the other part's
+    columns or None)``; the mixer's ``forward`` takes its columns as ``rows``."""
+
+    more_names = ()
+
+    def load_projection(self, tensors):
+        import torch
+
+        from ..ops import kernels
+
+        own, more = [tensors[n] for n in self.input_names()], [tensors[n] for n in self.more_names]
+        self.in_cols = sum(t.shape[0] for t in own)
+        self.in_w = kernels.for_decode(torch.cat(own + more).contiguous())
+        self.first_weight = self.in_w
+
+    def project(self, ctx, h, norm, cache):
+        import torch
+
+        from ..ops import kernels
+
+        x = norm.forward(ctx, h)
+        rows = ctx.scratch((x.shape[0], self.in_w.shape[0]), torch.float32)
+        kernels.linear(rows, x, self.in_w, splits=kernels.splits_alone(x.shape[0]))
+        return x, rows[:, : self.in_cols], rows[:, self.in_cols :] if self.more_names else None
+
+    def own_rows(self, ctx, x):
+        """The mixer's columns where nobody has made them yet."""
+        import torch
+
+        from ..ops import kernels
+
+        rows = ctx.scratch((x.shape[0], self.in_w.shape[0]), torch.float32)
+        kernels.linear(rows, x, self.in_w, splits=kernels.splits_alone(x.shape[0]))
+        return rows[:, : self.in_cols]
+
+
 class FeedForward(Part):
     native_kind = native.FFN
 

@@ -246,8 +246,11 @@ class SharedNormBlock(Block):
       values).  The layers of a step share the ``Y`` through ``ctx.shared`` (``depth_total``
       layers: the one with ``depth = 0`` takes the memory, the sublayers add straight into ``Y``).
 
-    The norm is an RMS norm (an ``rmsnorm`` part gives weight and eps).  Norm, convolution, the
-    sums and the weighted sum are 32-bit (csrc/parallel_block.hip).  The
+    The norm is an RMS norm (an ``rmsnorm`` part gives weight and eps); without the two options it may be
+    any norm.  Norm, convolution, the
+    sums and the weighted sum are 32-bit (csrc/parallel_block.hip).  A mixer that starts with a
+    product of the norm (``ProjectsFirst``) makes norm and product itself, and where the feed-forward
+    starts with one too (``input_names``, ``projection_given``) its rows come out of the same product.  The
     run's state slot holds the convolution's inputs and, behind them, what a mixer that keeps
     state beside its pages (``wants_state``) asks for.  No counterpart in mlx_lm/models/gpt2.py,
     whose blocks have a norm for each sublayer and run them in turn (:98-108).
@@ -261,10 +264,14 @@ class SharedNormBlock(Block):
         from .convolution import ShortConvolution
 
         super().__init__(prefix)
-        if not (hasattr(norm, "weight") and hasattr(norm, "eps")) or hasattr(norm, "bias"):
-            raise ValueError(f"this arrangement fuses an RMS norm, not a {type(norm).__name__}")
+        rms = hasattr(norm, "weight") and hasattr(norm, "eps") and not hasattr(norm, "bias")
+        self.plain = not rms or hasattr(mixer, "project")  # no options: norm, sublayers, two sums
+        if self.plain and (input_taps or depth is not None):
+            raise ValueError(f"this arrangement's options go with an RMS norm and a mixer that takes it, not with a {type(norm).__name__} ahead of a {type(mixer).__name__}")
         self.norm, self.mixer, self.ffn = norm, mixer, ffn
-        self.width, self.eps = norm.width, norm.eps
+        self.width, self.eps = norm.width, getattr(norm, "eps", None)
+        if hasattr(mixer, "project") and hasattr(ffn, "input_names") and hasattr(ffn, "projection_given"):
+            mixer.more_names, ffn.projection_given = tuple(ffn.input_names()), True
         if self.width % 8:
             raise ValueError(f"width {self.width} must be a multiple of 8")
         # (the part holds the weights and knows the state's layout; the kernels are this arrangement's own)
@@ -319,6 +326,8 @@ class SharedNormBlock(Block):
         from ..engine.context import CacheView
         from ..ops import kernels
 
+        if self.plain:
+            return self._forward_plain(ctx, h, cache, writes_cache)
         T, W = h.shape
         kept = target = None
         if self.depth is not None:
@@ -357,6 +366,23 @@ class SharedNormBlock(Block):
         ctx.scratch_release(mark)
         if kept is not None:
             kernels.depth_average(h, kept, self.depth_w, self.depth + 2)
+        return h
+
+
+    def _forward_plain(self, ctx, h, cache, writes_cache):
+        mark = ctx.scratch_mark()
+        if hasattr(self.mixer, "project"):
+            u, rows, more = self.mixer.project(ctx, h, self.norm, cache)
+            self.mixer.forward(ctx, u, h, cache, writes_cache, rows=rows)
+        else:
+            u, more = self.norm.forward(ctx, h), None
+            self.mixer.forward(ctx, u, h, cache, writes_cache)
+        if self.ffn is not None:
+            if more is not None:
+                self.ffn.forward(ctx, u, h, rows=more)
+            else:
+                self.ffn.forward(ctx, u, h)
+        ctx.scratch_release(mark)
         return h
 
 

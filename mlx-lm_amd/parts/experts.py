@@ -17,7 +17,11 @@ class GatedExperts(FeedForward):
       ``renormalize`` divided by the chosen ones' sum (+ 1e-20); times ``weight_scale``;
     * the last ``n_identity`` router outputs stand for experts that give their input back;
     * ``shared_inner > 0``: one more expert of that inner size (``shared.gate`` ...) that every
-      token uses with weight one.
+      token uses with weight one;
+    * ``activation = "clamped"``: an expert is ``Wdown (g sigmoid(1.702 g) (u + 1))`` with ``g = min(Wgate
+      x, limit)`` and ``u = Wup x`` clamped to ``[-limit, limit]`` (not the shared expert).
+
+    (``renormalize`` without a correction is the softmax over the chosen outputs alone.)
 
     The choice runs on the device (csrc/experts.hip), so a step launches kernels only.  For few
     tokens the chosen experts' weights are read straight from the stacked tensors, a wave a
@@ -33,8 +37,14 @@ class GatedExperts(FeedForward):
     TILES_FROM = 64  # from this many tokens in a step the picks are sorted and go to the matrix cores in tiles
 
     def __init__(self, width, n_experts, inner, top, n_identity=0, shared_inner=0, correction=True, renormalize=False,
-                 weight_scale=1.0, prefix=""):
+                 weight_scale=1.0, activation="silu", limit=0.0, prefix=""):
         super().__init__(prefix)
+        if activation not in kernels.EXPERT_ACTIVATIONS:
+            raise ValueError(f"experts' activation {activation!r} (known: {sorted(kernels.EXPERT_ACTIVATIONS)})")
+        if activation == "clamped" and limit <= 0:
+            raise ValueError(f"clamped activations need a positive limit, got {limit}")
+        self.activation, self.limit = activation, float(limit)
+        self.projection_given = False  # the router's outputs come out of a product that another part makes
         self.renormalize, self.weight_scale = bool(renormalize), float(weight_scale)
         if n_experts < 0 or n_identity < 0 or n_experts + n_identity <= 0:
             raise ValueError(f"{n_experts} experts and {n_identity} identity experts")
@@ -65,6 +75,10 @@ class GatedExperts(FeedForward):
             t[n("shared.down")] = TensorSpec((self.width, self.shared_inner), "matrix")
         return t
 
+    def input_names(self):
+        """The tensor whose rows are the projection that ``forward`` starts with."""
+        return [self._name("router")]
+
     def load(self, tensors):
         n = self._name
         self.w_gate = self.w_up = self.w_down = None
@@ -72,8 +86,9 @@ class GatedExperts(FeedForward):
             self.w_gate = torch.stack([tensors[n(f"e{e}.gate")] for e in range(self.n_experts)]).contiguous()
             self.w_up = torch.stack([tensors[n(f"e{e}.up")] for e in range(self.n_experts)]).contiguous()
             self.w_down = torch.stack([tensors[n(f"e{e}.down")] for e in range(self.n_experts)]).contiguous()
-        self.router_w = kernels.for_decode(tensors[n("router")].contiguous())
-        self.first_weight = self.router_w
+        if not self.projection_given:
+            self.router_w = kernels.for_decode(tensors[n("router")].contiguous())
+            self.first_weight = self.router_w
         self.correction = tensors[n("correction")] if self.has_correction else None
         self.shared_in = self.shared_out = None
         if self.shared_inner:
@@ -86,15 +101,18 @@ class GatedExperts(FeedForward):
             self.shared_in = kernels.for_decode(torch.cat([g, u]).contiguous())
             self.shared_out = kernels.for_decode(d.contiguous())
             # for steps of few tokens: router, gate and up in one product (float32 rows)
-            self.merged_in = kernels.for_decode(torch.cat([tensors[n("router")], g, u]).contiguous())
+            if not self.projection_given:
+                self.merged_in = kernels.for_decode(torch.cat([tensors[n("router")], g, u]).contiguous())
 
-    def forward(self, ctx, x, residual):
+    def forward(self, ctx, x, residual, rows=None):
+        """``rows``: the router's float32 outputs, where the caller has made them already."""
         T = x.shape[0]
+        merged = self.shared_inner and T <= self.MERGED_UP_TO and rows is None
         mark = ctx.scratch_mark()
         idx = ctx.scratch((T, self.top), torch.int32)
         weight = ctx.scratch((T, self.top), torch.float32)
         accumulate = not self.overwrite
-        if self.shared_inner and T <= self.MERGED_UP_TO:
+        if merged:
             # few tokens: what a launch costs counts for more than what it computes
             zu = ctx.scratch((T, self.n_out + 2 * self.shared_padded), torch.float32)
             kernels.linear(zu, x, self.merged_in)
@@ -103,10 +121,12 @@ class GatedExperts(FeedForward):
             kernels.linear(residual, act, self.shared_out, accumulate=accumulate)
             accumulate = True
         else:
-            z = ctx.scratch((T, self.n_out), torch.float32)
-            kernels.linear(z, x, self.router_w, splits=kernels.splits_alone(T))
+            z = rows
+            if z is None:
+                z = ctx.scratch((T, self.n_out), torch.float32)
+                kernels.linear(z, x, self.router_w, splits=kernels.splits_alone(T))
             kernels.router_choice(idx, weight, z, self.correction, self.top, self.renormalize, self.weight_scale)
-        if self.shared_inner and T > self.MERGED_UP_TO:
+        if self.shared_inner and not merged:
             gu = ctx.scratch((T, 2 * self.shared_padded), ctx.dtype)
             kernels.linear(gu, x, self.shared_in, splits=kernels.splits_alone(T))
             act = ctx.scratch((T, self.shared_padded), ctx.dtype)
@@ -115,11 +135,11 @@ class GatedExperts(FeedForward):
             accumulate = True
         if self.n_experts and T >= self.TILES_FROM and kernels.expert_tiles_takes(self.inner, self.width, x.dtype):
             kernels.expert_tiles(residual, x, self.w_gate, self.w_up, self.w_down, idx, weight, self.top, ctx.scratch,
-                                 accumulate=accumulate)
+                                 accumulate=accumulate, activation=self.activation, limit=self.limit)
         else:
             act = ctx.scratch((T * self.top, self.inner), ctx.dtype) if self.n_experts else None
             kernels.expert_rows(residual, x, self.w_gate, self.w_up, self.w_down, idx, weight, self.top, act,
-                                accumulate=accumulate)
+                                accumulate=accumulate, activation=self.activation, limit=self.limit)
         ctx.scratch_release(mark)
 
 

@@ -5,20 +5,24 @@ import torch
 from ..config.plan import CacheNeed
 from ..ops import kernels
 from .attention import CausalSelfAttention
-from .base import Mixer, TensorSpec, register_mixer
+from .base import Mixer, ProjectsFirst, TensorSpec, register_mixer
 from .linear_state import _matrix, _padded_columns
 from .rotary import rotary_table
 
 
-class LatentAttention(Mixer):
+class LatentAttention(ProjectsFirst, Mixer):
     """Queries through a latent: ``cq = N(Wdq x; dq.norm)``, ``q = Wuq cq``, head by head ``[key_dim
     plain | rot_dim rotated]``.  ``Wdkv x`` gives ``kv_rank + rot_dim`` columns: the first
     ``kv_rank``, RMS-normed, are the latent ``c``; the rest, rotated, one key part shared by all
     heads.  Head ``h`` has keys ``[Wuk_h c | rotated part]`` and values ``Wuv_h c``; causal softmax
-    of ``(q . k) * scale``; the head's output times ``sigmoid((Wg x)_h)``; ``Wo`` on the heads.
-    Rotation: pairs ``(2i, 2i + 1)`` of the ``rot_dim`` columns by ``position * base^(-2i / rot_dim)``.
+    of ``(q . k) * scale`` over every earlier key, or the last ``window``; with ``gate`` the head's
+    output times ``sigmoid((Wg x)_h)``; ``Wo`` on the heads.
+    Rotation: pairs ``(2i, 2i + 1)`` of the ``rot_dim`` columns (``interleaved``), or ``(i, i + rot_dim / 2)``,
+    by ``position * base^(-2i / rot_dim)``.
     A layer with ``own_latent=False`` has no ``Wdkv``: it reads the cache slot that another such
-    layer writes (the plan points its run there), with its own ``Wuk`` and ``Wuv``.
+    layer writes (the plan points its run there), with its own ``Wuk``, ``Wuv`` and window:
+    ``cache_window`` is the longest window among a slot's readers (0: some reader sees everything),
+    which says what its pages keep.
 
     What a page holds is the token's ``[c | rotated part]`` once, as the key and the value of a
     single key head: since ``q_h . (Wuk_h c) = (Wuk_h^T q_h) . c`` and ``Wo_h (Wuv_h sum_j p_j c_j)``
@@ -39,7 +43,7 @@ class LatentAttention(Mixer):
     length_class = staticmethod(CausalSelfAttention.length_class)
 
     def __init__(self, width, n_heads, key_dim, rot_dim, value_dim, q_rank, kv_rank, scale, eps, rot_base=10000.0,
-                 rot_scaling=None, own_latent=True, prefix=""):
+                 rot_scaling=None, own_latent=True, window=0, cache_window=None, gate=True, interleaved=True, prefix=""):
         super().__init__(prefix)
         if min(n_heads, key_dim, value_dim, q_rank, kv_rank) <= 0 or rot_dim < 0 or rot_dim % 2:
             raise ValueError(f"{n_heads} heads of {key_dim} + {rot_dim} key and {value_dim} value columns, ranks {q_rank} and {kv_rank}")
@@ -52,9 +56,14 @@ class LatentAttention(Mixer):
         self.q_rank, self.kv_rank, self.scale, self.eps = q_rank, kv_rank, float(scale), float(eps)
         self.rot_base, self.rot_scaling, self.own_latent = float(rot_base), rot_scaling, bool(own_latent)
         self.latent_cols = kv_rank + rot_dim
+        self.window, self.cache_window = int(window), int(window if cache_window is None else cache_window)
+        if self.window < 0 or (self.cache_window and not 0 < self.window <= self.cache_window):
+            raise ValueError(f"a window of {window} keys over pages that keep {cache_window}")
+        self.gate, self.interleaved = bool(gate), bool(interleaved)
+        self.lead_cols = q_rank + (n_heads if self.gate else 0)  # the projection's columns ahead of the latent
 
     def cache_need(self):
-        return CacheNeed(1, self.head_dim, 0)
+        return CacheNeed(1, self.head_dim, self.cache_window)
 
     def tensors(self):
         n, H = self._name, self.n_heads
@@ -62,20 +71,23 @@ class LatentAttention(Mixer):
              n("uq"): TensorSpec((H * (self.key_dim + self.rot_dim), self.q_rank), "matrix"),
              n("uk"): TensorSpec((H * self.key_dim, self.kv_rank), "matrix"),
              n("uv"): TensorSpec((H * self.value_dim, self.kv_rank), "matrix"),
-             n("g"): TensorSpec((H, self.width), "matrix"),
              n("o"): TensorSpec((self.width, H * self.value_dim), "matrix")}
+        if self.gate:
+            t[n("g")] = TensorSpec((H, self.width), "matrix")
         if self.own_latent:
             t[n("dkv")] = TensorSpec((self.latent_cols, self.width), "matrix")
             t[n("dkv.norm")] = TensorSpec((self.kv_rank,), "vector")
         return t
 
+    def input_names(self):
+        """The tensors whose rows, in this order, are the projection that ``forward`` starts with."""
+        return [self._name(x) for x in ("dq",) + (("g",) if self.gate else ()) + (("dkv",) if self.own_latent else ())]
+
     def load(self, tensors):
         n, H, d, dr, dv, r, hd = self._name, self.n_heads, self.key_dim, self.rot_dim, self.value_dim, self.kv_rank, self.head_dim
         dq = tensors[n("dq")]
         dev, dtype = dq.device, dq.dtype
-        first = [dq, tensors[n("g")]] + ([tensors[n("dkv")]] if self.own_latent else [])
-        self.in_w = _matrix(torch.cat(first))
-        self.first_weight = self.in_w
+        self.load_projection(tensors)
         self.q_norm = tensors[n("dq.norm")]
         self.c_norm = tensors[n("dkv.norm")] if self.own_latent else None
         uq = tensors[n("uq")].double().view(H, d + dr, self.q_rank)
@@ -92,11 +104,11 @@ class LatentAttention(Mixer):
         if dr:
             self.inv_freq, self.rot_mult = rotary_table(dr, self.rot_base, self.rot_scaling, dev)
 
-    def forward(self, ctx, x, residual, cache, writes_cache=True):
+    def forward(self, ctx, x, residual, cache, writes_cache=True, rows=None):
+        """``rows``: the projection's float32 rows, where the caller has made them already."""
         T, H, r, dr, hd, Q = x.shape[0], self.n_heads, self.kv_rank, self.rot_dim, self.head_dim, self.q_rank
         mark = ctx.scratch_mark()
-        u = ctx.scratch((T, Q + H + (self.latent_cols if self.own_latent else 0)), torch.float32)
-        kernels.linear(u, x, self.in_w, splits=kernels.splits_alone(T))
+        u = rows if rows is not None else self.own_rows(ctx, x)
         Qp = -(-Q // 8) * 8
         cq = ctx.scratch((T, Qp), ctx.dtype)
         if Qp == Q:
@@ -105,7 +117,8 @@ class LatentAttention(Mixer):
             kernels.head_prepare(cq, u, 0, 1, Q, dst_stride=Qp, dst_fill=Qp, norm_dim=Q, norm_weight=self.q_norm, eps=self.eps)
         qf = ctx.scratch((T, H * (r + dr)), torch.float32)
         kernels.linear(qf, cq, self.q_w, splits=kernels.splits_alone(T))
-        rot = dict(rot_off=r, rot_dims=dr, inv_freq=self.inv_freq, rot_mult=self.rot_mult, positions=ctx.positions)
+        rot = dict(rot_off=r, rot_dims=dr, inv_freq=self.inv_freq, rot_mult=self.rot_mult, interleaved=self.interleaved,
+                   positions=ctx.positions)
         q = ctx.scratch((T, H * hd), ctx.dtype)
         calls = [(q, qf, 0, H, r + dr, dict(dst_stride=hd, dst_fill=hd, **rot))]
         if writes_cache:
@@ -114,12 +127,13 @@ class LatentAttention(Mixer):
             # the latent goes straight to its pages, as the one key head's key and as its value
             for values in (False, True):
                 pages = kernels.PagesOut(cache.kv, values, cache.block_table, ctx.token_req, ctx.positions)
-                calls.append((pages, u, Q + H, 1, r + dr, dict(dst_stride=hd, dst_fill=hd, norm_dim=r, norm_weight=self.c_norm,
+                calls.append((pages, u, self.lead_cols, 1, r + dr, dict(dst_stride=hd, dst_fill=hd, norm_dim=r, norm_weight=self.c_norm,
                                                                eps=self.eps, **rot)))
         kernels.head_prepare_many(*calls)  # (queries and the latent in one launch)
         att = ctx.scratch((T, H * hd), ctx.dtype)
-        kernels.attend(ctx, att, q, cache, H, 1, hd, self.scale)
-        kernels.head_gate(att, hd, H, u[:, Q:Q + H])
+        kernels.attend(ctx, att, q, cache, H, 1, hd, self.scale, self.window)
+        if self.gate:
+            kernels.head_gate(att, hd, H, u[:, Q:Q + H])
         kernels.linear(residual, att, self.out_w, accumulate=True, splits=kernels.splits_alone(T))
         ctx.scratch_release(mark)
 

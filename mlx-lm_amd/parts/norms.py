@@ -98,5 +98,48 @@ class RMSNorm(Norm):
         return ctx.tensor(out.m)
 
 
+class DynamicTanh(Norm):
+    """``scale * (tanh(alpha * x) * weight + shift)``: no mean and no variance, an element needs nothing
+    but itself.  Tensors ``<name>`` and ``<name>.b`` (a value a column) and ``<name>.alpha`` (one number).
+    ``scale``: a constant that the consumer's output would be multiplied by; it rides on weight and shift.
+
+    Reads the float32 residual stream, computes in float32, writes the compute dtype
+    (csrc/dynamic_tanh.hip).  ``operands`` is what kernels that fuse the norm take.  No counterpart
+    in mlx_lm/models/gpt2.py, whose norms are LayerNorms.
+    """
+
+    graph_safe = True  # launches kernels only: a step of such parts can be recorded
+
+    def __init__(self, width, weight_name="weight", scale=1.0, prefix=""):
+        super().__init__(prefix)
+        if width <= 0 or width % 4:
+            raise ValueError(f"rows of {width} columns: a positive multiple of 4")
+        self.width, self.scale, self.name = width, float(scale), self._name(weight_name)
+        self.operands = None
+
+    def tensors(self):
+        return {self.name: TensorSpec((self.width,), "vector"), self.name + ".b": TensorSpec((self.width,), "vector"),
+                self.name + ".alpha": TensorSpec((), "vector")}
+
+    def load(self, tensors):
+        w, b = (tensors[self.name + x] * self.scale if self.scale != 1.0 else tensors[self.name + x] for x in ("", ".b"))
+        self.operands = (tensors[self.name + ".alpha"].reshape(1).contiguous(), w.contiguous(), b.contiguous())
+
+    def make_native(self):
+        P = ctypes.c_void_p
+        L = native.part_library("dynamic_tanh", {"make_dynamic_tanh": [ctypes.c_int, P, P, P]})
+        return native.made(L.make_dynamic_tanh(native.host(), self.width, *(native.ptr(t) for t in self.operands)), "dynamic tanh")
+
+    def forward(self, ctx, x, rows=None, n_rows=None, lazy=False):
+        out = native.EngValue()
+        xm = native.mat(x)
+        with ctx.enter():
+            rc = native.lib().eng_norm_forward(self.native(), ctypes.byref(ctx.c), ctypes.byref(xm), native.ptr(rows),
+                                               int(n_rows or 0), 0, None, ctypes.byref(out))
+        native.check(rc, "dynamic tanh")
+        return ctx.tensor(out.m)
+
+
 register_norm("layernorm", LayerNorm)
+register_norm("dynamic_tanh", DynamicTanh)
 register_norm("rmsnorm", RMSNorm)
