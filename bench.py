@@ -35,8 +35,9 @@ Pafutar model runs once without a window (like for like with GPT-2's attention) 
 window of 512 that keeps the first 64 tokens.  Ruzolorn runs at the same layer sizes too
 (``ruzolorn_config``), without a window and with one of 512, and Zatinex (``zatinex_config``:
 differential attention, gated linear attention and latent attention by turns, a dense gated
-feed-forward), and Sazilorn (``sazilorn_config``: its parallel, HGRN2 and attention mixers by turns,
-dense and expert feed-forwards).  It prints one JSON line of its own.
+feed-forward), Sazilorn (``sazilorn_config``: its parallel, HGRN2 and attention mixers by turns,
+dense and expert feed-forwards) and Gilidra (``gilidra_config``: its time-mixing, latent-attention and
+delta-rule mixers by turns, clamped experts).  It prints one JSON line of its own.
 """
 
 import argparse
@@ -78,6 +79,8 @@ def design_config(design, size, window=None):
         return zatinex_config(s)
     if design == "sazilorn":
         return sazilorn_config(s)
+    if design == "gilidra":
+        return gilidra_config(s)
     mixer = {"heads": s["heads"], "kv_heads": s["heads"], "dim": s["dim"], "vdim": s["dim"], "scale": s["dim"] ** -0.5}
     if window:
         mixer["mask"] = {"size": window[0], "keep_first": window[1]}
@@ -169,6 +172,29 @@ def sazilorn_config(s):
             "norm": {"eps": 1e-5}, "canon": {"taps": 4}, "layers": layers}
 
 
+def gilidra_config(s):
+    """Gilidra at GPT-2's layer sizes, its three mixers by turns.  Time mixing: as many heads of the same
+    size (Zatinex's gated linear attention is its like).  Latent attention: Zatinex's sizes, a window of
+    1,024, every second such layer reading the first one's latents with a window of half of it.  Delta
+    rule: as many value heads of the same size over half as many key heads, four taps.  Feed-forward:
+    sixteen experts of three sixteenths of GPT-2's inner size, four a token: a token multiplies with 3 x
+    4 x 3/16 = 2.25 inner sizes of weights, as Ruzolorn's and (its mixtures) Sazilorn's do."""
+    H, d, D = s["heads"], s["dim"], s["width"]
+    latent = {"heads": H, "dim": d, "rot_dim": d // 2, "vdim": d, "q_rank": D // 2, "kv_rank": 192, "mask": {"size": 1024},
+              "scale": (d + d // 2) ** -0.5, "rot": {"dims": d // 2, "base": 10000.0}}
+    mixers = [("wkv", {"heads": H, "dim": d, "decay_rank": 64}), ("latent_attention", latent),
+              ("delta", {"heads": H, "kv_heads": H // 2, "dim": d, "vdim": d, "conv": 4})]
+    mlp = {"kind": "moe", "expert": {"ff": s["ff"] * 3 // 16, "limit": 7.0}, "router": {"experts": 16, "top": 4}}
+    layers = []
+    for i in range(s["layers"]):
+        kind, mixer = mixers[i % 3]
+        if kind == "latent_attention" and (i // 3) % 2 == 1:
+            mixer = dict(mixer, kv_from=1, mask={"size": 512})
+        layers.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Gilidra", "vocab": DESIGN_VOCAB, "width": D, "max_positions": DESIGN_POSITIONS, "norm": {"eps": 1e-6},
+            "logit_scale": 0.5, "layers": layers}
+
+
 def bench_design(config, dtype, batches, steps, warmup):
     """Prefill of 2 x 1,024 tokens (three warm-up trials, the mean of five) and decode from
     context 512 at each of ``batches``, for the model that ``config`` describes."""
@@ -216,9 +242,10 @@ def compare_designs(a):
     for size in sizes:
         entry = {"layer_sizes": DESIGN_SIZES[size]}
         runs = {"gpt2": ("gpt2", None), "pafutar": ("pafutar", None), "pafutar_window_512_keep_64": ("pafutar", (512, 64)),
-                "ruzolorn": ("ruzolorn", None), "ruzolorn_window_512": ("ruzolorn", (512, 0)), "zatinex": ("zatinex", None), "sazilorn": ("sazilorn", None)}
+                "ruzolorn": ("ruzolorn", None), "ruzolorn_window_512": ("ruzolorn", (512, 0)), "zatinex": ("zatinex", None), "sazilorn": ("sazilorn", None),
+                "gilidra": ("gilidra", None)}
         for name, (design, window) in runs.items():
-            if a.design_only and name != a.design_only:
+            if a.design_only and name not in a.design_only.split(","):
                 continue
             entry[name] = bench_design(design_config(design, size, window), a.dtype, batches, a.steps, a.warmup)
         line["sizes"][size] = entry
@@ -325,7 +352,7 @@ def main():
     ap.add_argument("--designs", action="store_true",
                     help="a mode of its own: Pafutar beside GPT-2 at equal layer sizes (prefill and decode)")
     ap.add_argument("--design-size", choices=sorted(DESIGN_SIZES), default=None, help="with --designs: one size only")
-    ap.add_argument("--design-only", default=None, help="with --designs: one of gpt2, pafutar, pafutar_window_512_keep_64, ruzolorn, ruzolorn_window_512, zatinex, sazilorn")
+    ap.add_argument("--design-only", default=None, help="with --designs: one of gpt2, pafutar, pafutar_window_512_keep_64, ruzolorn, ruzolorn_window_512, zatinex, sazilorn, gilidra (or several, separated by commas)")
     a = ap.parse_args()
     if a.designs:
         if a.gpus != 1:

@@ -17,7 +17,8 @@
 // Kernels:
 //  * kv_write: scatter this step's keys and values into their pages.
 //  * attn_tile: 16 consecutive queries of one request per block, key tiles
-//    of 64 staged in LDS; any head_dim that is a multiple of 16 up to 256.
+//    of 64 staged in LDS; any head_dim that is a multiple of 16 up to 256 (wider heads, up to 1024:
+//    attn_tile_wide, which stages keys and values 256 columns at a time).
 //    Float caches with head_dim 64 or 128 in pages of whole 16 keys take
 //    attn_tile_mfma instead: a wave a tile, v_mfma_f32_16x16x4_f32, no LDS.
 //  * attn_row: one query per block, its keys split over the block's four
@@ -335,6 +336,120 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(AttnArgs p) {
   }
 }
 
+// attn_tile_wide: the same for heads of more than 256 columns (a latent that all heads share): keys and
+// values are staged WIDE_COLS columns at a time, a score growing over the pieces of its key.  A lane
+// holds NJ columns of the output (lane, lane + 64, ...).
+#define WIDE_COLS 256
+#define WIDE_MAX_HEAD_DIM 1024
+
+template <typename T, int NJ>
+__global__ __launch_bounds__(256) void attn_tile_wide_kernel(AttnArgs p) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int hd = p.head_dim;
+  constexpr int stride = WIDE_COLS + 1;
+  float* Qs = lds;                // [QT][hd], scaled
+  float* KVs = Qs + QT * hd;      // [KT][WIDE_COLS + 1]
+  float* Ps = KVs + KT * stride;  // [QT][KT]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int row0 = p.items[2 * blockIdx.x], nq = p.items[2 * blockIdx.x + 1];
+  const int h = blockIdx.y, kv_head = h / (p.n_heads / p.n_kv_heads);
+  const int pos0 = p.positions[row0];
+  const int* table = p.block_table + (size_t)p.token_req[row0] * p.max_blocks;
+  const T* q = (const T*)p.q;
+  const float q_scale = p.head_scale ? p.head_scale[h] : p.scale;
+  const float slope = p.slopes ? p.slopes[h] : 0.f;
+  for (int c = tid; c < QT * hd; c += 256) {
+    const int qi = c / hd, d = c - qi * hd;
+    Qs[c] = qi < nq ? to_f32(q[(size_t)(row0 + qi) * p.ldq + h * hd + d]) * q_scale : 0.f;
+  }
+  const KeyRuns runs = key_runs(p, pos0, pos0 + nq);
+  const int n_sink_tiles = (runs.sink_hi + KT - 1) / KT, kt0 = (runs.k_lo / KT) * KT;
+  const int n_tiles_all = n_sink_tiles + (runs.k_hi - kt0 + KT - 1) / KT;
+  float m[4], l[4], o[4][NJ];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    m[i] = -INFINITY, l[i] = 0.f;
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) o[i][j] = 0.f;
+  }
+  for (int t = 0; t < n_tiles_all; ++t) {
+    const bool sink = t < n_sink_tiles;
+    const int kt = sink ? t * KT : kt0 + (t - n_sink_tiles) * KT;
+    const int k_lo = sink ? 0 : runs.k_lo, k_hi = sink ? runs.sink_hi : runs.k_hi;
+    // columns c0 .. of this tile's keys (values), rows outside [k_lo, k_hi) zero
+    auto stage = [&](const T* pages, int c0) {
+      const int cols = min(WIDE_COLS, hd - c0);
+      __syncthreads();  // what was staged before is no longer read
+      for (int e = tid; e < KT * cols; e += 256) {
+        const int key = e / cols, c = e - key * cols, pos = kt + key;
+        float v = 0.f;
+        if (pos >= k_lo && pos < k_hi)
+          v = to_f32(pages[(size_t)table[pos / p.page_size] * p.page_stride +
+                           ((size_t)kv_head * p.page_size + pos % p.page_size) * hd + c0 + c]);
+        KVs[key * stride + c] = v;
+      }
+      __syncthreads();
+      return cols;
+    };
+    const int kpos = kt + lane;
+    float s[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int c0 = 0; c0 < hd; c0 += WIDE_COLS) {
+      const int cols = stage((const T*)p.k_pages, c0);
+      const float* krow = KVs + lane * stride;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float* qrow = Qs + (wave * 4 + i) * hd + c0;
+        for (int d = 0; d < cols; ++d) s[i] += qrow[d] * krow[d];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int qi = wave * 4 + i, qpos = pos0 + qi;
+      const bool ok = qi < nq && kpos >= k_lo && kpos < k_hi && sees(p, qpos, kpos);
+      const float sc = ok ? shaped_score(p, s[i], slope, h, qpos - kpos) : -INFINITY;
+      const float m_new = fmaxf(m[i], wave_max(sc));
+      float pr = 0.f, alpha = 1.f;
+      if (m_new != -INFINITY) {
+        pr = ok ? expf(sc - m_new) : 0.f;
+        alpha = expf(m[i] - m_new);
+      }
+      l[i] = l[i] * alpha + wave_sum(pr);
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) o[i][j] *= alpha;
+      m[i] = m_new;
+      Ps[qi * KT + lane] = pr;
+    }
+#pragma unroll
+    for (int cb = 0; cb < NJ / 4; ++cb) {  // (four of a lane's columns lie in each staged piece)
+      if (cb * WIDE_COLS >= hd) continue;  // (the same for the whole block)
+      const int cols = stage((const T*)p.v_pages, cb * WIDE_COLS);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float* prow = Ps + (wave * 4 + i) * KT;
+        for (int key = 0; key < KT; ++key) {
+          const float pv = prow[key];
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            if (lane + 64 * j < cols) o[i][4 * cb + j] += pv * KVs[key * stride + lane + 64 * j];
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int qi = wave * 4 + i;
+    if (qi >= nq) continue;
+    const float inv = 1.0f / l[i];
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+      const int d = lane + 64 * j;
+      if (d < hd)
+        ((T*)p.out)[(size_t)(row0 + qi) * p.ldo + h * hd + d] =
+            from_f32<T>(o[i][j] * inv * gate_of(p, row0 + qi, h * hd + d, sizeof(T) == 2));
+    }
+  }
+}
+
 // ---------------------------------------------------------------------------
 // attn_tile_mfma: float storage, head_dim = 64 * NV, page_size a multiple of 16.  Grid
 // (ceil(n_tiles / 4), n_heads), 256 threads; every wave takes a tile of its own and walks its
@@ -634,12 +749,12 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(AttnArgs p) {
 DEFINE_LAST_ERROR(mlxlm_last_error)
 
 static int check_geometry(const char* who, int n_heads, int n_kv_heads, int head_dim,
-                          int page_size, int dtype) {
+                          int page_size, int dtype, int widest = 256) {
   if (dtype != DT_F32 && dtype != DT_BF16) FAIL("%s: unknown dtype code %d", who, dtype);
   if (n_heads <= 0 || n_kv_heads <= 0 || n_heads % n_kv_heads != 0)
     FAIL("%s: %d query heads cannot be grouped over %d key heads", who, n_heads, n_kv_heads);
-  if (head_dim < 4 || head_dim > 256 || head_dim % 4 != 0)
-    FAIL("%s: head_dim %d must be a multiple of 4 between 4 and 256", who, head_dim);
+  if (head_dim < 4 || head_dim > widest || head_dim % 4 != 0)
+    FAIL("%s: head_dim %d must be a multiple of 4 between 4 and %d", who, head_dim, widest);
   if (page_size <= 0) FAIL("%s: page_size %d must be positive", who, page_size);
   return 0;
 }
@@ -690,7 +805,7 @@ static int fill_args(AttnArgs& p, const char* who, void* out, const void* q, int
                      const int* block_table, int max_blocks, const int* token_req,
                      const int* positions, const int* items, int n_heads, int n_kv_heads,
                      int head_dim, int page_size, int window, float scale, int dtype) {
-  if (check_geometry(who, n_heads, n_kv_heads, head_dim, page_size, dtype)) return 1;
+  if (check_geometry(who, n_heads, n_kv_heads, head_dim, page_size, dtype, WIDE_MAX_HEAD_DIM)) return 1;
   if (!out || !q || !k_pages || !v_pages || !block_table || !token_req || !positions || !items)
     FAIL("%s: null pointer", who);
   const int vec = dtype == DT_F32 ? 4 : 8;
@@ -775,8 +890,24 @@ static int tile_launch(void* out, const void* q, int ldq, int ldo, const void* k
     CHECK_LAUNCH("attn_tile");
     return 0;
   }
-  const size_t lds = sizeof(float) * ((size_t)QT * head_dim + (size_t)KT * (head_dim + 1) + QT * KT);
   dim3 grid(n_tiles, n_heads), block(256);
+  if (head_dim > 256) {
+    const size_t wide = sizeof(float) * ((size_t)QT * head_dim + (size_t)KT * (WIDE_COLS + 1) + QT * KT);
+#define WIDE(T, NJ)                                                                          \
+  do {                                                                                       \
+    if (allow_lds("attn_tile", (const void*)attn_tile_wide_kernel<T, NJ>, wide)) return 1;   \
+    hipLaunchKernelGGL((attn_tile_wide_kernel<T, NJ>), grid, block, wide, stream, p);        \
+  } while (0)
+    if (dtype == DT_F32) {
+      if (head_dim <= 512) WIDE(float, 8); else WIDE(float, 16);
+    } else {
+      if (head_dim <= 512) WIDE(bf16, 8); else WIDE(bf16, 16);
+    }
+#undef WIDE
+    CHECK_LAUNCH("attn_tile");
+    return 0;
+  }
+  const size_t lds = sizeof(float) * ((size_t)QT * head_dim + (size_t)KT * (head_dim + 1) + QT * KT);
   if (dtype == DT_F32) {
     if (allow_lds("attn_tile", (const void*)attn_tile_kernel<float>, lds)) return 1;
     hipLaunchKernelGGL(attn_tile_kernel<float>, grid, block, lds, stream, p);

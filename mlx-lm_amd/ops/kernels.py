@@ -1264,6 +1264,7 @@ def head_gate(x, head_stride, n_heads, gate):
 
 
 FAST_HEAD_DIMS = (16, 32, 64, 128, 256)
+WIDE_HEAD_DIM = 1024  # the widest head that the general tile kernel takes (it stages 256 columns at a time)
 
 
 def attention_head_dim(columns):
