@@ -9,7 +9,9 @@
 //                   wave four features at once: act[t, j, :] = w_tj silu(Wg_e x_t) * (Wu_e x_t) (or
 //                   another activation of the two, expert_act), then
 //                   y[t, :] += sum_j Wd_e act[t, j, :] + sum_(j: e is an identity expert) w_tj x_t.
-//                   Only the chosen experts' weights are read: the kernels for few tokens.
+//                   Only the chosen experts' weights are read: the kernels for few tokens.  The first
+//                   may make the choice itself from the router's outputs, the second may leave the
+//                   next layer's norm of the rows it completes.
 //   expert_tiles    the same for many tokens: the picks are sorted by expert on the device
 //                   (expert_sort: counts, offsets, tiles of up to 64 picks of one expert), and
 //                   every tile is a small matrix product on the matrix cores with the rows
@@ -163,20 +165,45 @@ __device__ __forceinline__ void lane_dots(const T* const* __restrict__ a, const 
   }
 }
 
+// The router's outputs of every token, for a kernel that chooses the experts itself.
+struct RouteArgs {
+  const float* z;  // [tokens, ldz], or null: idx and weight hold the choice already
+  int ldz;
+  const float* correction;
+  int n_out, renorm;
+  float mult;
+};
+#define ROUTED_MOST 64  // picks a token that a block chooses itself
+
 // Block (token x pick, 16 features): a wave four features at once (eight rows of weights in
-// flight), lanes along the width.
-template <typename T, bool VEC>
+// flight), lanes along the width.  ROUTED: the block's first wave chooses the token's experts from the
+// router's outputs; the block of the first pick and features leaves the choice for the kernel behind.
+template <typename T, bool VEC, bool ROUTED>
 __global__ __launch_bounds__(256) void expert_rows_up_kernel(const T* __restrict__ x, int ldx,
                                                              const T* __restrict__ w_gate, const T* __restrict__ w_up,
-                                                             const int* __restrict__ idx,
-                                                             const float* __restrict__ weight, int n_experts, int top,
-                                                             int F, int width, T* __restrict__ act, ExpertAct fn) {
+                                                             int* __restrict__ idx, float* __restrict__ weight, int n_experts,
+                                                             int top, int F, int width, T* __restrict__ act, ExpertAct fn,
+                                                             RouteArgs route) {
+  __shared__ int s_idx[ROUTED ? ROUTED_MOST : 1];
+  __shared__ float s_weight[ROUTED ? ROUTED_MOST : 1];
   const int item = blockIdx.x, t = item / top;
-  const int e = idx[item];
-  if (e >= n_experts) return;  // an identity expert: nothing to compute
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  int e;
+  float wt;
+  if constexpr (ROUTED) {
+    if (wave == 0)
+      route_token(route.z + (size_t)t * route.ldz, route.correction, route.n_out, top, s_idx, s_weight, lane, route.renorm, route.mult);
+    __syncthreads();
+    const int j = item - t * top;
+    if (j == 0 && blockIdx.y == 0 && (int)threadIdx.x < top)
+      idx[(size_t)t * top + threadIdx.x] = s_idx[threadIdx.x], weight[(size_t)t * top + threadIdx.x] = s_weight[threadIdx.x];
+    e = s_idx[j], wt = s_weight[j];
+  } else {
+    e = idx[item], wt = weight[item];
+  }
+  if (e >= n_experts) return;  // an identity expert: nothing to compute
   const int f0 = blockIdx.y * 16 + wave * 4;
-  if (f0 >= F) return;  // (no barrier in this kernel)
+  if (f0 >= F) return;  // (no barrier from here on)
   const T* rows[8];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
@@ -187,7 +214,6 @@ __global__ __launch_bounds__(256) void expert_rows_up_kernel(const T* __restrict
   lane_dots<T, VEC, 8>(rows, x + (size_t)t * ldx, width, lane, s);
 #pragma unroll
   for (int r = 0; r < 8; ++r) s[r] = wave_sum(s[r]);
-  const float wt = weight[item];
   if (lane < 4 && f0 + lane < F) {
     float g = s[0], u = s[4];
 #pragma unroll
@@ -197,20 +223,30 @@ __global__ __launch_bounds__(256) void expert_rows_up_kernel(const T* __restrict
   }
 }
 
-// Block (token, 16 columns): a wave four output columns at once, lanes along the features.
-template <typename T, bool VEC>
+// The layer behind's norm of the rows that the experts' sum completes, where that norm needs nothing but
+// the element: out = tanh(alpha y) w + b (out null: none).
+struct NextNorm {
+  const float* alpha;
+  const float* w;
+  const float* b;
+  void* out;  // [tokens, width] of the compute dtype
+};
+
+// Block (token, 16 / PW columns): a wave four output columns at once, lanes along the features; PW waves
+// share the token's picks (every PW-th each) and are summed in their order.
+template <typename T, bool VEC, int PW>
 __global__ __launch_bounds__(256) void expert_rows_down_kernel(const T* __restrict__ act, const T* __restrict__ w_down,
                                                                const int* __restrict__ idx,
                                                                const float* __restrict__ weight,
                                                                const T* __restrict__ x, int ldx, int n_experts, int top,
                                                                int F, int width, float* __restrict__ y, int ldy,
-                                                               int accumulate) {
+                                                               int accumulate, NextNorm next) {
+  __shared__ float part[4][8];
   const int t = blockIdx.x;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int n0 = blockIdx.y * 16 + wave * 4;
-  if (n0 >= width) return;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, pw = wave % PW;
+  const int n0 = blockIdx.y * (16 / PW) + wave / PW * 4;
   float tot[4] = {0.f, 0.f, 0.f, 0.f}, same = 0.f;
-  for (int j = 0; j < top; ++j) {
+  for (int j = pw; j < top; j += PW) {
     const int e = idx[(size_t)t * top + j];
     if (e >= n_experts) {
       same += weight[(size_t)t * top + j];
@@ -226,15 +262,22 @@ __global__ __launch_bounds__(256) void expert_rows_down_kernel(const T* __restri
   }
 #pragma unroll
   for (int r = 0; r < 4; ++r) tot[r] = wave_sum(tot[r]);
-  if (lane < 4 && n0 + lane < width) {
-    float v = tot[0];
-#pragma unroll
-    for (int r = 1; r < 4; ++r)
-      if (lane == r) v = tot[r];
-    v += same * to_f32(x[(size_t)t * ldx + n0 + lane]);
-    float* o = y + (size_t)t * ldy + n0 + lane;
-    *o = accumulate ? *o + v : v;
+  if (PW > 1) {
+    if (lane == 0) part[wave][0] = tot[0], part[wave][1] = tot[1], part[wave][2] = tot[2], part[wave][3] = tot[3], part[wave][4] = same;
+    __syncthreads();
   }
+  if (pw != 0 || lane >= 4 || n0 + lane >= width) return;
+  float v = tot[0];
+#pragma unroll
+  for (int r = 1; r < 4; ++r)
+    if (lane == r) v = tot[r];
+#pragma unroll
+  for (int i = 1; i < PW; ++i) v += part[wave + i][lane], same += part[wave + i][4];
+  v += same * to_f32(x[(size_t)t * ldx + n0 + lane]);
+  float* o = y + (size_t)t * ldy + n0 + lane;
+  if (accumulate) v = *o + v;
+  *o = v;
+  if (next.out) ((T*)next.out)[(size_t)t * width + n0 + lane] = from_f32<T>(tanhf(*next.alpha * v) * next.w[n0 + lane] + next.b[n0 + lane]);
 }
 
 // ---------------------------------------------------------------------------
@@ -564,11 +607,12 @@ extern "C" int act_mul(const void* gu, int ld, void* out, int ldo, int n_rows, i
   return act_mul_launch(gu, ld, out, ldo, n_rows, F, dtype, activation, stream);
 }
 
-// act: [n_tokens * top, F] of the compute dtype; y: float rows.
+// act: [n_tokens * top, F] of the compute dtype; y: float rows.  `route` (or null): the choice is made
+// here, from the router's outputs, into idx and weight.  `next` (or null): the norm of the new rows.
 extern "C" int expert_rows(const void* x, int ldx, const void* w_gate, const void* w_up, const void* w_down,
-                           const int* idx, const float* weight, int n_tokens, int n_experts, int top, int F, int width,
+                           int* idx, float* weight, int n_tokens, int n_experts, int top, int F, int width,
                            void* act, float* y, int ldy, int accumulate, int dtype, int act_kind, float act_limit,
-                           hipStream_t stream) {
+                           const RouteArgs* route, const NextNorm* next, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (!x || !idx || !weight || !y || (n_experts > 0 && (!w_gate || !w_up || !w_down || !act)))
     FAIL("expert_rows: null pointer");
@@ -576,16 +620,32 @@ extern "C" int expert_rows(const void* x, int ldx, const void* w_gate, const voi
   if (dtype != DT_F32 && dtype != DT_BF16) FAIL("expert_rows: unknown dtype code %d", dtype);
   if (act_kind != EXPERT_SILU && act_kind != EXPERT_CLAMPED) FAIL("expert_rows: unknown activation code %d", act_kind);
   const ExpertAct fn = {act_kind, act_limit};
-  const int feats = 16, cols = 16, per = dtype == DT_BF16 ? 8 : 4;
+  if (route) {
+    if (n_experts <= 0 || top > ROUTED_MOST) FAIL("expert_rows: %d picks of %d experts are not chosen here", top, n_experts);
+    if (!route->z || route->n_out <= 0 || top > route->n_out || route->ldz < route->n_out || route->n_out > 64 * ROUTER_PER_LANE)
+      FAIL("expert_rows: %d of %d outputs, rows of %d", top, route->n_out, route->ldz);
+  }
+  const NextNorm nn = next ? *next : NextNorm{};
+  if (next && (!nn.out || !nn.alpha || !nn.w || !nn.b || !accumulate)) FAIL("expert_rows: the next norm's pointers, or rows that are not complete here");
+  const RouteArgs rt = route ? *route : RouteArgs{};
+  const int feats = 16, per = dtype == DT_BF16 ? 8 : 4, pw = top >= 4 ? 4 : top >= 2 ? 2 : 1, cols = 16 / pw;
   const bool vec = F % per == 0 && width % per == 0 && ldx % per == 0 && !((uintptr_t)x & 15);
   dim3 block(256), up_grid(n_tokens * top, (F + feats - 1) / feats), down_grid(n_tokens, (width + cols - 1) / cols);
-#define RUN(T, VEC)                                                                                                        \
-  do {                                                                                                                     \
-    if (n_experts > 0)                                                                                                     \
-      hipLaunchKernelGGL((expert_rows_up_kernel<T, VEC>), up_grid, block, 0, stream, (const T*)x, ldx, (const T*)w_gate,   \
-                         (const T*)w_up, idx, weight, n_experts, top, F, width, (T*)act, fn);                       \
-    hipLaunchKernelGGL((expert_rows_down_kernel<T, VEC>), down_grid, block, 0, stream, (const T*)act, (const T*)w_down,    \
-                       idx, weight, (const T*)x, ldx, n_experts, top, F, width, y, ldy, accumulate);                 \
+#define UP(T, VEC, ROUTED)                                                                                                  \
+  hipLaunchKernelGGL((expert_rows_up_kernel<T, VEC, ROUTED>), up_grid, block, 0, stream, (const T*)x, ldx, (const T*)w_gate, \
+                     (const T*)w_up, idx, weight, n_experts, top, F, width, (T*)act, fn, rt)
+#define DOWN(T, VEC, PW)                                                                                                   \
+  hipLaunchKernelGGL((expert_rows_down_kernel<T, VEC, PW>), down_grid, block, 0, stream, (const T*)act, (const T*)w_down,  \
+                     idx, weight, (const T*)x, ldx, n_experts, top, F, width, y, ldy, accumulate, nn)
+#define RUN(T, VEC)                         \
+  do {                                      \
+    if (n_experts > 0) {                    \
+      if (route) UP(T, VEC, true);          \
+      else UP(T, VEC, false);               \
+    }                                       \
+    if (pw == 4) DOWN(T, VEC, 4);           \
+    else if (pw == 2) DOWN(T, VEC, 2);      \
+    else DOWN(T, VEC, 1);                   \
   } while (0)
   if (dtype == DT_F32) {
     if (vec) RUN(float, true); else RUN(float, false);
@@ -593,6 +653,8 @@ extern "C" int expert_rows(const void* x, int ldx, const void* w_gate, const voi
     if (vec) RUN(bf16, true); else RUN(bf16, false);
   }
 #undef RUN
+#undef UP
+#undef DOWN
   CHECK_LAUNCH("expert_rows");
   return 0;
 }

@@ -57,6 +57,15 @@
 #define LN_MAX_V 8  // float4 per lane a normed row may take (K <= 2048)
 #define ZERO4 make_uint4(0u, 0u, 0u, 0u)  // a constant, not a variable: see load_pass
 
+// Matrices that lie one after the other in W and read inputs of their own (a mixer whose projections
+// each read another mix of the rows): the features from end[g - 1] up to end[g] (multiples of 32) read
+// plane[g] of A, planes `stride` elements apart.  n == 0: one input for all.
+#define A_GROUPS_MOST 8
+struct AGroups {
+  int n;
+  int end[A_GROUPS_MOST], plane[A_GROUPS_MOST];
+  size_t stride;
+};
 struct DecodeGemmArgs {
   const uint16_t* W;
   const float* bias;
@@ -84,7 +93,17 @@ struct DecodeGemmArgs {
   int a_packed;        // rows kernel: A lies in tiles of 16 rows x 64 k in the weights' packed order (packed_at)
   int row_groups;      // rows kernel: the rows go in this many groups of R_TILES tiles, a block each
   int out_kblocks;     // FLAG_OUT_PACKED: tiles a tile row of out, (N + 63) / 64
+  AGroups groups;
 };
+
+// The input that the block with features from n0 on reads.
+__device__ __forceinline__ const uint16_t* input_of(const DecodeGemmArgs& p, int n0) {
+  int plane = 0;
+#pragma unroll
+  for (int g = A_GROUPS_MOST - 1; g >= 0; --g)
+    if (g < p.groups.n && n0 < p.groups.end[g]) plane = p.groups.plane[g];
+  return p.A + (size_t)plane * p.groups.stride;
+}
 
 __device__ __forceinline__ uint32_t pack2(float a, float b) { return pack_bf16x2(a, b); }
 
@@ -290,6 +309,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_bf16_decode_kernel(DecodeGemmArg
     }
   } else {
     load_pass(w0, 0);  // in flight while the activations are copied
+    const uint16_t* in = input_of(p, n0);
     // four independent loads a thread and round: one trip to L2 instead of four in a row
     const int per_row = (min(p.K, kb + n_chunks * 64) - kb) / 8;
     const int total = p.M * per_row;
@@ -299,7 +319,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_bf16_decode_kernel(DecodeGemmArg
       for (int j = 0; j < 4; ++j) {
         const int c = min(c0 + j * NW * 64, total - 1);
         const int r = c / per_row, k = (c - r * per_row) * 8;
-        t[j] = *(const uint4*)(p.A + (size_t)r * p.lda + kb + k);
+        t[j] = *(const uint4*)(in + (size_t)r * p.lda + kb + k);
       }
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
@@ -449,7 +469,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_rows_kernel(DecodeGemmAr
   // (l / 16) * 16 on (rows beyond M repeat the last; what they give is not stored)
   const uint16_t* arow[R_TILES];
 #pragma unroll
-  for (int rt = 0; rt < R_TILES; ++rt) arow[rt] = p.A + (size_t)min((t0 + rt) * 16 + (lane & 15), p.M - 1) * p.lda;
+  for (int rt = 0; rt < R_TILES; ++rt) arow[rt] = input_of(p, n0) + (size_t)min((t0 + rt) * 16 + (lane & 15), p.M - 1) * p.lda;
   const int m_tiles = (p.M + 15) / 16;
   auto load_a = [&](Frag (&a)[R_TILES][2], int i) {
     const int c = c_begin + min(wave + WAVES * i, n_chunks - 1);
@@ -806,12 +826,12 @@ static int fill_epilogue(DecodeGemmArgs& p, const char* who, void* out, const fl
 
 // With n_splits > 1 the epilogue does not run: the partial sums go to `ws`
 // ([n_splits][M][N] floats) and sum_partials or sum_partials_norm finishes.
-extern "C" int gemm_bf16_decode(
+static int decode_launch(
     void* out, const void* A, int lda, const float* X, int ldx, const float* gamma,
     const float* beta, float eps, const void* W, const float* bias, int M, int N, int K, int ldw,
     int ldo, int flags, void* k_pages, void* v_pages, size_t page_stride, const int* block_table,
     int max_blocks, const int* token_req, const int* positions, int q_width, int kv_width,
-    int head_dim, int page_size, int n_splits, float* ws, size_t ws_floats, hipStream_t stream) {
+    int head_dim, int page_size, int n_splits, float* ws, size_t ws_floats, const AGroups* groups, hipStream_t stream) {
   if (M == 0) return 0;
   const bool ln = X != nullptr;
   if (!gemm_bf16_decode_takes(M, K, ln, n_splits))
@@ -828,6 +848,7 @@ extern "C" int gemm_bf16_decode(
   if (X && (!gamma || !aligned16(gamma) || !aligned16(beta)))
     FAIL("gemm_bf16_decode: the norm needs a scale (and a shift, or none), 16-byte aligned");
   DecodeGemmArgs p;
+  p.groups = groups ? *groups : AGroups{};
   if (fill_epilogue(p, "gemm_bf16_decode", out, bias, M, N, ldo, flags, k_pages, v_pages, page_stride,
                     block_table, max_blocks, token_req, positions, q_width, kv_width, head_dim, page_size))
     return -1;
@@ -869,6 +890,17 @@ extern "C" int gemm_bf16_decode(
   return 0;
 }
 
+extern "C" int gemm_bf16_decode(
+    void* out, const void* A, int lda, const float* X, int ldx, const float* gamma,
+    const float* beta, float eps, const void* W, const float* bias, int M, int N, int K, int ldw,
+    int ldo, int flags, void* k_pages, void* v_pages, size_t page_stride, const int* block_table,
+    int max_blocks, const int* token_req, const int* positions, int q_width, int kv_width,
+    int head_dim, int page_size, int n_splits, float* ws, size_t ws_floats, hipStream_t stream) {
+  return decode_launch(out, A, lda, X, ldx, gamma, beta, eps, W, bias, M, N, K, ldw, ldo, flags, k_pages, v_pages, page_stride,
+                       block_table, max_blocks, token_req, positions, q_width, kv_width, head_dim, page_size, n_splits, ws,
+                       ws_floats, nullptr, stream);
+}
+
 // 1 if gemm_bf16_rows takes these sizes
 extern "C" int gemm_bf16_rows_takes(int M, int K, int n_splits) {
   if (M < 17 || M > ROWS_MAX_M || K < 8 || K % 8 != 0 || n_splits < 1 || n_splits > (K + 63) / 64) return 0;
@@ -899,12 +931,12 @@ extern "C" int gemm_bf16_rows_splits(int M, int N, int K, int force) {
 // (with a bfloat16 out, no accumulate, no scatter) writes out in that order too, for the product
 // that reads it next; ldo is not used then.  With n_splits > 1 the partial sums go to `ws` and
 // sum_partials or sum_partials_norm finishes.
-extern "C" int gemm_bf16_rows(void* out, const void* A, int lda, const void* W, const float* bias, int M,
+static int rows_launch(void* out, const void* A, int lda, const void* W, const float* bias, int M,
                               int N, int K, int ldo, int flags, void* k_pages, void* v_pages,
                               size_t page_stride, const int* block_table, int max_blocks,
                               const int* token_req, const int* positions, int q_width, int kv_width,
                               int head_dim, int page_size, int n_splits, float* ws, size_t ws_floats,
-                              hipStream_t stream) {
+                              const AGroups* groups, hipStream_t stream) {
   if (M == 0) return 0;
   if (!gemm_bf16_rows_takes(M, K, n_splits))
     FAIL("gemm_bf16_rows: M=%d K=%d in %d splits is outside what this kernel takes", M, K, n_splits);
@@ -913,6 +945,7 @@ extern "C" int gemm_bf16_rows(void* out, const void* A, int lda, const void* W, 
   if (lda != 0 && (lda % 8 != 0 || lda < K)) FAIL("gemm_bf16_rows: A rows must be 16-byte aligned");
   if (!aligned16(A)) FAIL("gemm_bf16_rows: A must be 16-byte aligned");
   DecodeGemmArgs p = {};
+  if (groups) p.groups = *groups;
   if (fill_epilogue(p, "gemm_bf16_rows", out, bias, M, N, ldo, flags, k_pages, v_pages, page_stride,
                     block_table, max_blocks, token_req, positions, q_width, kv_width, head_dim, page_size))
     return -1;
@@ -942,6 +975,51 @@ extern "C" int gemm_bf16_rows(void* out, const void* A, int lda, const void* W, 
     hipLaunchKernelGGL((gemm_bf16_rows_kernel<3, 2, 2 * RW, 4>), grid, dim3(2 * RW * 64), 0, stream, p);
   CHECK_LAUNCH("gemm_bf16_rows");
   return 0;
+}
+
+extern "C" int gemm_bf16_rows(void* out, const void* A, int lda, const void* W, const float* bias, int M,
+                              int N, int K, int ldo, int flags, void* k_pages, void* v_pages,
+                              size_t page_stride, const int* block_table, int max_blocks,
+                              const int* token_req, const int* positions, int q_width, int kv_width,
+                              int head_dim, int page_size, int n_splits, float* ws, size_t ws_floats,
+                              hipStream_t stream) {
+  return rows_launch(out, A, lda, W, bias, M, N, K, ldo, flags, k_pages, v_pages, page_stride, block_table, max_blocks, token_req,
+                     positions, q_width, kv_width, head_dim, page_size, n_splits, ws, ws_floats, nullptr, stream);
+}
+
+// Several products in one launch: float rows out [M, N] (row stride ldo), M up to 64, W in the packed
+// order; the features from end[g - 1] up to end[g] read plane[g] of A (see AGroups).  Returns 0, or 2
+// where the sizes are not for these kernels (nothing is launched then).
+extern "C" int sum_partials(void* out, const float* ws, int n_splits, const float* bias, int M, int N,
+                            int ldo, int flags, void* k_pages, void* v_pages, size_t page_stride,
+                            const int* block_table, int max_blocks, const int* token_req,
+                            const int* positions, int q_width, int kv_width, int head_dim,
+                            int page_size, hipStream_t stream);
+extern "C" int gemm_bf16_groups(float* out, const void* A, int lda, size_t plane_stride, const int* ends, const int* planes,
+                                int n_groups, const void* W, int M, int N, int K, int ldo, float* ws, size_t ws_floats,
+                                hipStream_t stream) {
+  if (M == 0) return 0;
+  if (n_groups < 1 || n_groups > A_GROUPS_MOST || M > ROWS_MAX_M) return 2;
+  if (!ends || !planes || plane_stride % 8 != 0) FAIL("gemm_bf16_groups: null pointer, or planes that are not 16-byte aligned");
+  AGroups g = {};
+  g.n = n_groups, g.stride = plane_stride;
+  for (int i = 0; i < n_groups; ++i) {
+    if (ends[i] % 32 != 0 || ends[i] <= (i ? ends[i - 1] : 0) || planes[i] < 0)
+      FAIL("gemm_bf16_groups: group %d ends at feature %d (multiples of 32, ascending)", i, ends[i]);
+    g.end[i] = ends[i], g.plane[i] = planes[i];
+  }
+  if (g.end[n_groups - 1] != N) FAIL("gemm_bf16_groups: the groups end at feature %d of %d", g.end[n_groups - 1], N);
+  if (M <= 16) {
+    if (!gemm_bf16_decode_takes(M, K, 0, 1)) return 2;
+    return decode_launch(out, A, lda, nullptr, 0, nullptr, nullptr, 0.f, W, nullptr, M, N, K, 0, ldo, FLAG_OUT_F32, nullptr, nullptr, 0,
+                         nullptr, 0, nullptr, nullptr, 0, 0, 0, 0, 1, nullptr, 0, &g, stream);
+  }
+  const int least = ((K + 63) / 64 + RW * R_HELD - 1) / (RW * R_HELD);  // as few parts as the kernel takes
+  if (!gemm_bf16_rows_takes(M, K, least) || (least > 1 && ws_floats < (size_t)least * M * N)) return 2;
+  int rc = rows_launch(out, A, lda, W, nullptr, M, N, K, ldo, FLAG_OUT_F32, nullptr, nullptr, 0, nullptr, 0, nullptr, nullptr, 0, 0, 0,
+                       0, least, ws, ws_floats, &g, stream);
+  if (rc || least == 1) return rc;
+  return sum_partials(out, ws, least, nullptr, M, N, ldo, FLAG_OUT_F32, nullptr, nullptr, 0, nullptr, 0, nullptr, nullptr, 0, 0, 0, 0, stream);
 }
 
 // out = epilogue(sum of the n_splits partial products in ws): what gemm_bf16_decode left out.

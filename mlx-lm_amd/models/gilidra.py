@@ -171,7 +171,9 @@ class Model:
                 parts["ffn"] = PartSpec("gated_experts", {
                     "width": D, "n_experts": mlp["router"]["experts"], "inner": mlp["expert"]["ff"], "top": mlp["router"]["top"],
                     "correction": False, "renormalize": True, "activation": "clamped", "limit": float(mlp["expert"]["limit"])}, p + "mlp.")
-            layers.append(LayerSpec("shared_norm", parts))
+            # (the layer behind starts with its norm, unless a token shift makes that itself)
+            follows = i + 1 < len(args.layers) and args.layers[i + 1]["type"] != "wkv" and mlp is not None
+            layers.append(LayerSpec("shared_norm", parts, {"next_norm": norm(f"l{i + 1}.norm1")} if follows else {}))
             if source != i:
                 schedule.append(RunEntry(layer=i, cache=slot_of[source], writes_cache=False))
                 continue

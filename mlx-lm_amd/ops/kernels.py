@@ -561,6 +561,8 @@ class GroupedWeight:
         whole = torch.cat(parts).contiguous()
         self.N, self.K, self.dtype = at, K, whole.dtype
         self.w = for_decode(whole)
+        ends = [a + (n + self.BLOCK - 1) // self.BLOCK * self.BLOCK for a, n in self.columns]
+        self.c_ends, self.c_planes = (_c_int * len(ends))(*ends), (_c_int * len(ends))(*self.planes)
         # each group by itself, over the same memory: whole blocks of sixteen features of the packed order
         self.parts = [self._slice(start, (n + 15) // 16 * 16 if isinstance(self.w, PackedWeight) else n, n) for start, n in self.columns]
 
@@ -583,6 +585,15 @@ def linear_groups(alloc, planes, w):
     _need(planes.is_contiguous() and planes.shape[2] == w.K and planes.dtype == w.dtype, "linear_groups: shapes")
     rows = alloc((T, w.N), torch.float32)
     out = [rows[:, a : a + n] for a, n in w.columns]
+    if isinstance(w.w, PackedWeight) and 0 < T <= 64:  # few rows: one launch for all
+        lib = build.load("gemm_bf16_decode")
+        ws = split_workspace(planes.device)
+        rc = lib.gemm_bf16_groups(_ptr(rows), _ptr(planes), _c_int(w.K), _c_size_t(T * w.K), w.c_ends, w.c_planes, _c_int(len(w.planes)),
+                                  _ptr(w.w.packed), _c_int(T), _c_int(w.N), _c_int(w.K), _c_int(w.N), _ptr(ws), _c_size_t(ws.numel()),
+                                  _stream())
+        if rc != 2:
+            build.check(lib, rc, "linear_groups")
+            return out
     for view, plane, part in zip(out, w.planes, w.parts):
         linear(view, planes[plane], part, splits=splits_alone(T))
     return out
@@ -1425,12 +1436,30 @@ def _expert_activation(activation, limit):
     return _c_int(EXPERT_ACTIVATIONS[activation]), _c_float(limit)
 
 
-def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=True, activation="silu", limit=0.0):
+class RouteArgs(ctypes.Structure):
+    """Mirror of ``RouteArgs`` in csrc/experts.hip."""
+
+    _fields_ = [("z", _vp), ("ldz", _c_int), ("correction", _vp), ("n_out", _c_int), ("renorm", _c_int), ("mult", _c_float)]
+
+
+class NextNorm(ctypes.Structure):
+    """Mirror of ``NextNorm`` in csrc/experts.hip."""
+
+    _fields_ = [("alpha", _vp), ("w", _vp), ("b", _vp), ("out", _vp)]
+
+
+ROUTED_MOST = 64  # up to this many picks a token, ``expert_rows`` makes the choice itself
+
+
+def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=True, activation="silu", limit=0.0, route=None, after=None):
     """``y (+)= sum over a token's picks of weight * expert(x)``, reading only the picked experts'
     weights (``w_gate``, ``w_up``: ``[experts, F, width]``, ``w_down``: ``[experts, width, F]``); a
     pick at or beyond the number of experts gives ``weight * x``.  ``act``: room for ``[tokens *
     top, F]`` of ``x``'s dtype.  ``activation``: ``silu(g) * u``, or ``clamped``: ``g sigmoid(1.702 g) (u
-    + 1)`` with ``g`` at most ``limit`` and ``u`` within ``[-limit, limit]``."""
+    + 1)`` with ``g`` at most ``limit`` and ``u`` within ``[-limit, limit]``.  ``route = (z, correction,
+    renormalize, weight_scale)``: the choice is made here (``router_choice``), into ``idx`` and ``weight``.
+    ``after = (out, norm)``: the rows that this completes (``accumulate``) pass ``dynamic_tanh`` with
+    ``norm`` into ``out`` (``x``'s dtype) too."""
     lib = build.load("experts")
     ldx, ldy = _rows2d(x, "x"), _rows2d(y, "y")
     T, width = x.shape
@@ -1447,10 +1476,28 @@ def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=Tr
     _dev(idx, "idx", torch.int32)
     _dev(weight, "weight", torch.float32)
     _need(idx.numel() >= T * top and weight.numel() >= T * top, "expert_rows: idx / weight too short")
+    rt = nn = None
+    if route is not None:
+        z, correction, renormalize, weight_scale = route
+        rt = RouteArgs()
+        rt.ldz, rt.z, rt.n_out = _f32_rows(z, "z", 1), z.data_ptr(), z.shape[1]
+        _need(z.shape[0] >= T, "expert_rows: fewer rows of router outputs than tokens")
+        if correction is not None:
+            _dev(correction, "correction", torch.float32)
+            _need(correction.numel() == z.shape[1], "expert_rows: correction length")
+            rt.correction = correction.data_ptr()
+        rt.renorm, rt.mult = int(bool(renormalize)), float(weight_scale)
+    if after is not None:
+        out, norm = after
+        _need(out.is_contiguous() and out.dtype == x.dtype and tuple(out.shape) == (T, width) and accumulate, "expert_rows: after")
+        nn = NextNorm()
+        nn.alpha, nn.w, nn.b = (p.value for p in _tanh_norm(norm, width))
+        nn.out = out.data_ptr()
     rc = lib.expert_rows(_ptr(x), _c_int(ldx), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _ptr(idx), _ptr(weight),
                          _c_int(T), _c_int(n_experts), _c_int(top), _c_int(F), _c_int(width), _ptr(act), _ptr(y),
                          _c_int(ldy), _c_int(int(bool(accumulate))), _c_int(DT[x.dtype]),
-                         *_expert_activation(activation, limit), _stream())
+                         *_expert_activation(activation, limit), ctypes.byref(rt) if rt is not None else None,
+                         ctypes.byref(nn) if nn is not None else None, _stream())
     build.check(lib, rc, "expert_rows")
     return y
 

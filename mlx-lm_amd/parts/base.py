@@ -162,7 +162,9 @@ class ProjectsFirst:
 
         from ..ops import kernels
 
-        x = norm.forward(ctx, h)
+        x = ctx.shared.pop("normed_rows", None)  # (the layer before may have left them)
+        if x is None:
+            x = norm.forward(ctx, h)
         rows = ctx.scratch((x.shape[0], self.in_w.shape[0]), torch.float32)
         kernels.linear(rows, x, self.in_w, splits=kernels.splits_alone(x.shape[0]))
         return x, rows[:, : self.in_cols], rows[:, self.in_cols :] if self.more_names else None

@@ -250,7 +250,10 @@ class SharedNormBlock(Block):
     any norm.  Norm, convolution, the
     sums and the weighted sum are 32-bit (csrc/parallel_block.hip).  A mixer that starts with a
     product of the norm (``ProjectsFirst``) makes norm and product itself, and where the feed-forward
-    starts with one too (``input_names``, ``projection_given``) its rows come out of the same product.  The
+    starts with one too (``input_names``, ``projection_given``) its rows come out of the same product.
+    ``next_norm``: the norm (a ``PartSpec``) that the following layer starts with, if it is one without
+    statistics: in steps of few tokens the feed-forward, which completes the rows, leaves it for that
+    layer (``ctx.shared["normed_rows"]``).  The
     run's state slot holds the convolution's inputs and, behind them, what a mixer that keeps
     state beside its pages (``wants_state``) asks for.  No counterpart in mlx_lm/models/gpt2.py,
     whose blocks have a norm for each sublayer and run them in turn (:98-108).
@@ -260,7 +263,8 @@ class SharedNormBlock(Block):
     OPTIONAL = ("ffn",)
 
     def __init__(self, norm, mixer, ffn=None, input_taps=0, input_conv_name="canon1", depth=None, depth_total=0,
-                 depth_name="dwa", prefix=""):
+                 depth_name="dwa", next_norm=None, prefix=""):
+        from .base import NORMS, build_part
         from .convolution import ShortConvolution
 
         super().__init__(prefix)
@@ -272,6 +276,9 @@ class SharedNormBlock(Block):
         self.width, self.eps = norm.width, getattr(norm, "eps", None)
         if hasattr(mixer, "project") and hasattr(ffn, "input_names") and hasattr(ffn, "projection_given"):
             mixer.more_names, ffn.projection_given = tuple(ffn.input_names()), True
+        self.next_norm = build_part(NORMS, "norm", next_norm) if next_norm is not None else None
+        if self.next_norm is not None and not (self.plain and hasattr(self.next_norm, "operands") and hasattr(ffn, "projection_given")):
+            raise ValueError("the next layer's norm rides on a feed-forward of experts and needs no statistics")
         if self.width % 8:
             raise ValueError(f"width {self.width} must be a multiple of 8")
         # (the part holds the weights and knows the state's layout; the kernels are this arrangement's own)
@@ -293,7 +300,7 @@ class SharedNormBlock(Block):
             for sub in getattr(part, "sub_parts", lambda: ())():
                 walk(sub)
 
-        for p in (self.norm, self.input_conv, self.mixer, self.ffn):
+        for p in (self.norm, self.input_conv, self.mixer, self.ffn, self.next_norm):
             walk(p)
         return tuple(out) + (self,)  # (the arrangement owns a tensor itself, so it is one of its own parts)
 
@@ -370,6 +377,9 @@ class SharedNormBlock(Block):
 
 
     def _forward_plain(self, ctx, h, cache, writes_cache):
+        after = None
+        if self.next_norm is not None and h.shape[0] < self.ffn.TILES_FROM:
+            after = (ctx.scratch(tuple(h.shape), ctx.dtype), self.next_norm.operands)  # (kept beyond this layer)
         mark = ctx.scratch_mark()
         if hasattr(self.mixer, "project"):
             u, rows, more = self.mixer.project(ctx, h, self.norm, cache)
@@ -378,10 +388,11 @@ class SharedNormBlock(Block):
             u, more = self.norm.forward(ctx, h), None
             self.mixer.forward(ctx, u, h, cache, writes_cache)
         if self.ffn is not None:
-            if more is not None:
-                self.ffn.forward(ctx, u, h, rows=more)
-            else:
-                self.ffn.forward(ctx, u, h)
+            options = {} if more is None else {"rows": more}
+            if after is not None:
+                options["after"] = after
+            if self.ffn.forward(ctx, u, h, **options) and after is not None:
+                ctx.shared["normed_rows"] = after[0]
         ctx.scratch_release(mark)
         return h
 

@@ -104,11 +104,15 @@ class GatedExperts(FeedForward):
             if not self.projection_given:
                 self.merged_in = kernels.for_decode(torch.cat([tensors[n("router")], g, u]).contiguous())
 
-    def forward(self, ctx, x, residual, rows=None):
-        """``rows``: the router's float32 outputs, where the caller has made them already."""
+    def forward(self, ctx, x, residual, rows=None, after=None):
+        """``rows``: the router's float32 outputs, where the caller has made them already.  ``after``:
+        ``(out, norm operands)`` of a dynamic tanh over the rows that this completes, for the layer
+        behind; returns whether it was made (steps of few tokens only)."""
         T = x.shape[0]
         merged = self.shared_inner and T <= self.MERGED_UP_TO and rows is None
         mark = ctx.scratch_mark()
+        tiles = self.n_experts and T >= self.TILES_FROM and kernels.expert_tiles_takes(self.inner, self.width, x.dtype)
+        route = None
         idx = ctx.scratch((T, self.top), torch.int32)
         weight = ctx.scratch((T, self.top), torch.float32)
         accumulate = not self.overwrite
@@ -125,7 +129,10 @@ class GatedExperts(FeedForward):
             if z is None:
                 z = ctx.scratch((T, self.n_out), torch.float32)
                 kernels.linear(z, x, self.router_w, splits=kernels.splits_alone(T))
-            kernels.router_choice(idx, weight, z, self.correction, self.top, self.renormalize, self.weight_scale)
+            if not tiles and self.n_experts and self.top <= kernels.ROUTED_MOST:
+                route = (z, self.correction, self.renormalize, self.weight_scale)  # (chosen by the kernel that reads the experts)
+            else:
+                kernels.router_choice(idx, weight, z, self.correction, self.top, self.renormalize, self.weight_scale)
         if self.shared_inner and not merged:
             gu = ctx.scratch((T, 2 * self.shared_padded), ctx.dtype)
             kernels.linear(gu, x, self.shared_in, splits=kernels.splits_alone(T))
@@ -133,14 +140,15 @@ class GatedExperts(FeedForward):
             kernels.silu_mul(act, gu)
             kernels.linear(residual, act, self.shared_out, accumulate=accumulate, splits=kernels.splits_alone(T))
             accumulate = True
-        if self.n_experts and T >= self.TILES_FROM and kernels.expert_tiles_takes(self.inner, self.width, x.dtype):
+        if tiles:
             kernels.expert_tiles(residual, x, self.w_gate, self.w_up, self.w_down, idx, weight, self.top, ctx.scratch,
                                  accumulate=accumulate, activation=self.activation, limit=self.limit)
         else:
             act = ctx.scratch((T * self.top, self.inner), ctx.dtype) if self.n_experts else None
             kernels.expert_rows(residual, x, self.w_gate, self.w_up, self.w_down, idx, weight, self.top, act,
-                                accumulate=accumulate, activation=self.activation, limit=self.limit)
+                                accumulate=accumulate, activation=self.activation, limit=self.limit, route=route, after=after)
         ctx.scratch_release(mark)
+        return after is not None and not tiles
 
 
 register_feed_forward("gated_experts", GatedExperts)

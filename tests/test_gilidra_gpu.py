@@ -390,6 +390,35 @@ def test_clamped_experts_with_weights_over_the_chosen_alone(dtype, T, F, top):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("F,width,top,E", [(24, 48, 1, 5), (9, 44, 2, 70), (64, 96, 5, 5), (40, 24, 4, 130), (16, 8, 11, 12)])
+def test_the_choice_and_the_next_norm_inside_the_experts_kernels(dtype, F, width, top, E):
+    """The experts chosen by the kernel that reads them, and the next layer's norm left by the one that
+    completes the rows, against the separate kernels: the same picks and weights, sums to rounding."""
+    from mlx_lm_amd.ops import kernels
+
+    g = torch.Generator().manual_seed(F + top)
+    T = 7
+    x = torch.randn(T, width, generator=g).to(dtype).cuda()
+    gate, up, down = (torch.randn(*s, generator=g).to(dtype).cuda() * s[-1] ** -0.5 for s in ((E, F, width), (E, F, width), (E, width, F)))
+    zs = torch.randn(T, E + 3, generator=g).cuda()
+    z, correction = zs[:, :E], torch.randn(E, generator=g).cuda() * 0.1
+    norm = tuple(t.cuda() for t in (torch.tensor([0.6]), torch.randn(width, generator=g), torch.randn(width, generator=g)))
+    idx, weight = torch.empty(T, top, dtype=torch.int32, device="cuda"), torch.empty(T, top, device="cuda")
+    kernels.router_choice(idx, weight, z, correction, top, renormalize=True, weight_scale=1.5)
+    start = torch.randn(T, width, generator=g).cuda()
+    act = torch.empty(T * top, F, dtype=dtype, device="cuda")
+    y, y2, out = start.clone(), start.clone(), torch.empty(T, width, dtype=dtype, device="cuda")
+    kernels.expert_rows(y, x, gate, up, down, idx, weight, top, act, activation="clamped", limit=0.8)
+    idx2, weight2 = torch.full_like(idx, -1), torch.zeros_like(weight)
+    kernels.expert_rows(y2, x, gate, up, down, idx2, weight2, top, act, activation="clamped", limit=0.8, route=(z, correction, True, 1.5),
+                        after=(out, norm))
+    assert torch.equal(idx, idx2) and torch.equal(weight, weight2) and torch.equal(y, y2)
+    want = torch.empty_like(out)
+    kernels.dynamic_tanh(want, y, norm)
+    assert torch.equal(out, want)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("T", [1, 5, 16, 17, 33, 64, 65, 200])
 def test_products_that_read_planes_of_their_own(dtype, T):
     """Matrices of widths that are no multiples of a block, each over an input of its own, for one
