@@ -10,13 +10,14 @@
 //                   another activation of the two, expert_act), then
 //                   y[t, :] += sum_j Wd_e act[t, j, :] + sum_(j: e is an identity expert) w_tj x_t.
 //                   Only the chosen experts' weights are read: the kernels for few tokens.  The first
-//                   may make the choice itself from the router's outputs, the second may leave the
-//                   next layer's norm of the rows it completes.
+//                   may make the choice itself from the router's outputs, the second (as expert_combine)
+//                   may leave the next layer's norm of the rows it completes.
 //   expert_tiles    the same for many tokens: the picks are sorted by expert on the device
-//                   (expert_sort: counts, offsets, tiles of up to 64 picks of one expert), and
+//                   (expert_sort: counts, offsets, tiles of picks of one expert), and
 //                   every tile is a small matrix product on the matrix cores with the rows
-//                   gathered through the sorted list: [gate | up] with the activation and the
-//                   pick's weight in the epilogue, then down into a row of its own for every
+//                   gathered through the sorted list (bfloat16: through LDS, tiles of 32, 64 or 128
+//                   picks; 32-bit: operands straight from memory): [gate | up] with the activation and
+//                   the pick's weight in the epilogue, then down into a row of its own for every
 //                   pick; expert_combine adds a token's picks in their order, and the identity
 //                   experts' share.  The grid is as large as the tiles could be at most; blocks
 //                   beyond the tiles that there are leave at once, so nothing comes to the host.
@@ -283,15 +284,17 @@ __global__ __launch_bounds__(256) void expert_rows_down_kernel(const T* __restri
 // ---------------------------------------------------------------------------
 // many tokens: picks sorted by expert, a tile of picks a block
 
-#define TILE_PICKS 64
+#define TILE_PICKS 64        // picks a tile of the 32-bit kernels
+#define TILE_PICKS_LEAST 32  // the smallest tile of the bfloat16 kernels
 
-// One block.  tiles: (expert, first place in `order`, picks) each.
+// One block.  tiles: (expert, first place in `order`, picks) each, up to `tile_picks` picks a tile.
 __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict__ idx, int n_items, int n_experts,
-                                                           int* __restrict__ order, int* __restrict__ tiles,
+                                                           int tile_picks, int* __restrict__ order, int* __restrict__ tiles,
                                                            int* __restrict__ n_tiles) {
   extern __shared__ int lds_i[];
   int* counts = lds_i;
   int* cursor = lds_i + n_experts;
+  int* first_tile = cursor + n_experts;
   for (int e = threadIdx.x; e < n_experts; e += 1024) counts[e] = 0;
   __syncthreads();
   for (int i = threadIdx.x; i < n_items; i += 1024) {
@@ -302,16 +305,18 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict
   if (threadIdx.x == 0) {
     int at = 0, nt = 0;
     for (int e = 0; e < n_experts; ++e) {
-      cursor[e] = at;
-      for (int r0 = 0; r0 < counts[e]; r0 += TILE_PICKS) {
-        tiles[3 * nt] = e, tiles[3 * nt + 1] = at + r0, tiles[3 * nt + 2] = min(TILE_PICKS, counts[e] - r0);
-        ++nt;
-      }
-      at += counts[e];
+      cursor[e] = at, first_tile[e] = nt;
+      at += counts[e], nt += (counts[e] + tile_picks - 1) / tile_picks;
     }
     *n_tiles = nt;
   }
   __syncthreads();
+  for (int e = threadIdx.x; e < n_experts; e += 1024) {
+    int* tile = tiles + 3 * first_tile[e];
+    for (int r0 = 0; r0 < counts[e]; r0 += tile_picks, tile += 3)
+      tile[0] = e, tile[1] = cursor[e] + r0, tile[2] = min(tile_picks, counts[e] - r0);
+  }
+  __syncthreads();  // (the cursors move from here on)
   for (int i = threadIdx.x; i < n_items; i += 1024) {
     const int e = idx[i];
     if (e < n_experts) order[atomicAdd(&cursor[e], 1)] = i;  // (any order within an expert: a pick's row is computed by itself)
@@ -498,12 +503,154 @@ __global__ __launch_bounds__(256) void expert_tiles_down_kernel(const T* __restr
     }
 }
 
+// The bfloat16 kernels for many tokens: both products as tiles through LDS.  A block takes one tile of
+// picks (BM = 32 WM TM of one expert, gathered through the sorted list) and BN = 64 WN rows of that
+// expert's weights; WM x WN waves, each 32 TM picks x 64 weight rows on v_mfma_f32_32x32x16_bf16, the
+// weights as the instruction's rows, so that a lane ends up with four neighbouring outputs of a pick.
+// UP: a wave's 64 weight rows are the gate's and the up projection's rows of the same 32 features, so
+// the activation is the wave's own; down: 64 output columns.  Two k-blocks of 64 columns lie in LDS, two
+// more are on their way in registers.  Blocks go to the eight dies in turn; the (tile, weight rows)
+// pairs are put in panels of PANEL tiles, weight rows after weight rows inside a panel, and that
+// sequence is cut into eight runs, one a die: the tiles of an expert meet its weights in one L2.
+// The grid is as large as the tiles could be at most; blocks beyond those that there are leave at once.
+#define XK 64              // columns a k-block
+#define X_ZERO make_uint4(0u, 0u, 0u, 0u)  // a constant: a select against a variable would go through scratch memory
+#define X_STRIDE (XK + 8)  // LDS row stride: 16-byte reads of neighbouring rows on distinct banks
+template <int WM, int WN, int TM, bool UP>
+__global__ __launch_bounds__(64 * WM * WN, 2) void expert_gemm_kernel(const uint16_t* __restrict__ x, int ldx,
+                                                                   const uint16_t* __restrict__ w_a,
+                                                                   const uint16_t* __restrict__ w_b,
+                                                                   const int* __restrict__ order, const int* __restrict__ tiles,
+                                                                   const int* __restrict__ n_tiles,
+                                                                   const float* __restrict__ weight, int top, int N, int K,
+                                                                   void* __restrict__ out, ExpertAct fn) {
+  constexpr int BM = WM * TM * 32, BN = WN * 64, THREADS = 64 * WM * WN, ROW_STEP = THREADS / 8;
+  constexpr int PA = BM / ROW_STEP, PB = BN / ROW_STEP, PANEL = BM >= 128 ? 4 : 8;
+  __shared__ __attribute__((aligned(16))) uint16_t smem[2 * (BM + BN) * X_STRIDE];
+  const int nt = *n_tiles, columns = UP ? BN / 2 : BN, nb = (N + columns - 1) / columns;
+  const int total = nt * nb, run = (total + N_DIES - 1) / N_DIES, local = blockIdx.x / N_DIES;
+  const int at = (int)(blockIdx.x % N_DIES) * run + local;
+  if (local >= run || at >= total) return;
+  const int panel = at / (PANEL * nb), rem = at - panel * PANEL * nb, tall = min(PANEL, nt - panel * PANEL);
+  const int tile = panel * PANEL + rem % tall, fb = rem / tall;
+  const int e = tiles[3 * tile], first = tiles[3 * tile + 1], count = tiles[3 * tile + 2];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave / WN, wn = wave % WN;
+
+  // a thread moves PA pieces of 16 bytes of the picks' rows and PB of the weights' per k-block: piece i
+  // is row tid / 8 + ROW_STEP i, columns 8 (tid % 8) ..; rows beyond the tile repeat rows inside it
+  const int kc = (tid & 7) * 8;
+  int pa[PA], pb[PB];  // (element offsets of 32 bits: registers are scarce here)
+  const uint16_t* wa = w_a + (size_t)e * N * K;
+  const uint16_t* wb = UP ? w_b + (size_t)e * N * K : wa;
+#pragma unroll
+  for (int i = 0; i < PA; ++i) {
+    const int r = (tid >> 3) + ROW_STEP * i, item = order[first + (r < count ? r : r % count)];
+    pa[i] = (UP ? item / top : item) * ldx + kc;
+  }
+#pragma unroll
+  for (int i = 0; i < PB; ++i) {
+    const int c = (tid >> 3) + ROW_STEP * i;
+    const int f = UP ? fb * columns + (c >> 6) * 32 + (c & 31) : fb * columns + c;
+    pb[i] = (f < N ? f : f % N) * K + kc;
+  }
+  uint4 ra[2][PA], rb[2][PB];
+  auto load = [&](uint4 (&xa)[PA], uint4 (&xb)[PB], int k0) {
+    const int kk = k0 + kc < K ? k0 : -kc;  // (a piece beyond K: the row's first columns, zeroed on their way to LDS)
+#pragma unroll
+    for (int i = 0; i < PA; ++i) xa[i] = *(const uint4*)(x + (pa[i] + kk));
+    // (32 rows of the gate, 32 of the up projection by turns: which of the two a piece belongs to is known)
+#pragma unroll
+    for (int i = 0; i < PB; ++i) xb[i] = *(const uint4*)(((ROW_STEP * i) & 32 ? wb : wa) + (pb[i] + kk));
+  };
+  static_assert(!UP || ROW_STEP == 32 || ROW_STEP == 16, "a thread's pieces lie in one of the two matrices each");
+  const int lds_at = (tid >> 3) * X_STRIDE + kc;
+  auto store = [&](int stage, const uint4 (&xa)[PA], const uint4 (&xb)[PB], int k0) {
+    const bool in = k0 + kc < K;
+    uint16_t* a = smem + stage * (BM + BN) * X_STRIDE + lds_at;
+    uint16_t* b = a + BM * X_STRIDE;
+#pragma unroll
+    for (int i = 0; i < PA; ++i) *(uint4*)(a + i * ROW_STEP * X_STRIDE) = in ? xa[i] : X_ZERO;
+#pragma unroll
+    for (int i = 0; i < PB; ++i) *(uint4*)(b + i * ROW_STEP * X_STRIDE) = in ? xb[i] : X_ZERO;
+  };
+  f32x16_t acc[TM][2];
+#pragma unroll
+  for (int i = 0; i < TM; ++i)
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) acc[i][j][r] = 0.f;
+  auto multiply = [&](int stage) {
+    const uint16_t* a = smem + stage * (BM + BN) * X_STRIDE + (wm * TM * 32 + (lane & 31)) * X_STRIDE + (lane >> 5) * 8;
+    const uint16_t* b = smem + (stage * (BM + BN) + BM) * X_STRIDE + (wn * 64 + (lane & 31)) * X_STRIDE + (lane >> 5) * 8;
+#pragma unroll
+    for (int ks = 0; ks < XK; ks += 16) {
+      bf16x8_t av[TM], bv[2];
+#pragma unroll
+      for (int i = 0; i < TM; ++i) av[i] = *(const bf16x8_t*)(a + i * 32 * X_STRIDE + ks);
+#pragma unroll
+      for (int j = 0; j < 2; ++j) bv[j] = *(const bf16x8_t*)(b + j * 32 * X_STRIDE + ks);
+#pragma unroll
+      for (int i = 0; i < TM; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bv[j], av[i], acc[i][j], 0, 0, 0);
+    }
+  };
+  const int blocks = (K + XK - 1) / XK, last = (blocks - 1) * XK;
+  load(ra[0], rb[0], 0);
+  load(ra[1], rb[1], min(XK, last));
+  store(0, ra[0], rb[0], 0);
+  __syncthreads();
+  for (int kb = 0; kb < blocks; kb += 2) {
+    load(ra[0], rb[0], min((kb + 2) * XK, last));
+    __builtin_amdgcn_sched_barrier(0);  // (the loads go out ahead of the arithmetic)
+    multiply(0);
+    store(1, ra[1], rb[1], min((kb + 1) * XK, last));
+    __syncthreads();
+    if (kb + 1 >= blocks) break;
+    load(ra[1], rb[1], min((kb + 3) * XK, last));
+    __builtin_amdgcn_sched_barrier(0);
+    multiply(1);
+    store(0, ra[0], rb[0], min((kb + 2) * XK, last));
+    __syncthreads();
+  }
+  // register r of a 32 x 32 tile: weight row 8 (r / 4) + 4 (lane / 32) + r % 4, pick lane % 32
+#pragma unroll
+  for (int i = 0; i < TM; ++i) {
+    const int r = (wm * TM + i) * 32 + (lane & 31);
+    if (r >= count) continue;
+    const int item = order[first + r];
+    if constexpr (UP) {
+      const float wt = weight[item];
+#pragma unroll
+      for (int g = 0; g < 4; ++g) {
+        const int f = fb * columns + wn * 32 + 8 * g + 4 * (lane >> 5);
+        if (f >= N) continue;  // (N is a multiple of eight: a piece of four is inside or outside)
+        float v[4];
+#pragma unroll
+        for (int c = 0; c < 4; ++c) v[c] = wt * expert_act(fn, acc[i][0][4 * g + c], acc[i][1][4 * g + c]);
+        *(uint2*)((uint16_t*)out + (size_t)item * N + f) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < 2; ++j)
+#pragma unroll
+        for (int g = 0; g < 4; ++g) {
+          const int n = fb * columns + wn * 64 + 32 * j + 8 * g + 4 * (lane >> 5);
+          if (n >= N) continue;
+          *(float4*)((float*)out + (size_t)item * N + n) =
+              make_float4(acc[i][j][4 * g], acc[i][j][4 * g + 1], acc[i][j][4 * g + 2], acc[i][j][4 * g + 3]);
+        }
+    }
+  }
+}
+
 // Thread (token, column): a token's picks in their order, identity experts give weight * x.
 template <typename T>
 __global__ __launch_bounds__(256) void expert_combine_kernel(const float* __restrict__ out, const int* __restrict__ idx,
                                                              const float* __restrict__ weight, const T* __restrict__ x, int ldx,
                                                              int n_experts, int top, int width, float* __restrict__ y, int ldy,
-                                                             int accumulate) {
+                                                             int accumulate, NextNorm next) {
   const int n = blockIdx.y * 256 + threadIdx.x, t = blockIdx.x;
   if (n >= width) return;
   float s = 0.f, same = 0.f;
@@ -514,9 +661,11 @@ __global__ __launch_bounds__(256) void expert_combine_kernel(const float* __rest
     else
       s += out[it * width + n];
   }
-  const float v = s + same * to_f32(x[(size_t)t * ldx + n]);
+  float v = s + same * to_f32(x[(size_t)t * ldx + n]);
   float* o = y + (size_t)t * ldy + n;
-  *o = accumulate ? *o + v : v;
+  if (accumulate) v = *o + v;
+  *o = v;
+  if (next.out) ((T*)next.out)[(size_t)t * width + n] = from_f32<T>(tanhf(*next.alpha * v) * next.w[n] + next.b[n]);
 }
 
 DEFINE_LAST_ERROR(mlxlm_last_error)
@@ -660,7 +809,9 @@ extern "C" int expert_rows(const void* x, int ldx, const void* w_gate, const voi
 }
 
 // The most tiles that n_items picks over n_experts experts can make.
-extern "C" int expert_tiles_most(int n_items, int n_experts) { return (n_items + TILE_PICKS - 1) / TILE_PICKS + n_experts; }
+extern "C" int expert_tiles_most(int n_items, int n_experts) {
+  return (n_items + TILE_PICKS_LEAST - 1) / TILE_PICKS_LEAST + n_experts;
+}
 
 // 1 if expert_tiles takes these sizes (the operands are read 16 bytes a lane).
 extern "C" int expert_tiles_takes(int F, int width, int dtype) {
@@ -669,43 +820,67 @@ extern "C" int expert_tiles_takes(int F, int width, int dtype) {
 }
 
 // order: [n_tokens * top] ints, tiles: [3 * expert_tiles_most] ints, n_tiles: one int, act: [n_tokens * top, F]
-// of the compute dtype, out: [n_tokens * top, width] floats.
+// of the compute dtype, out: [n_tokens * top, width] floats.  `next` (or null): the norm of the new rows.
 extern "C" int expert_tiles(const void* x, int ldx, const void* w_gate, const void* w_up, const void* w_down, const int* idx,
                             const float* weight, int n_tokens, int n_experts, int top, int F, int width, int* order, int* tiles,
                             int* n_tiles, void* act, float* out, float* y, int ldy, int accumulate, int dtype,
-                            int act_kind, float act_limit, hipStream_t stream) {
+                            int act_kind, float act_limit, const NextNorm* next, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
+  const NextNorm nn = next ? *next : NextNorm{};
+  if (next && (!nn.out || !nn.alpha || !nn.w || !nn.b || !accumulate)) FAIL("expert_tiles: the next norm's pointers, or rows that are not complete here");
   if (!x || !idx || !weight || !y || !w_gate || !w_up || !w_down || !order || !tiles || !n_tiles || !act || !out)
     FAIL("expert_tiles: null pointer");
   if (n_experts <= 0 || top <= 0 || ldx < width || ldy < width) FAIL("expert_tiles: sizes");
   if (dtype != DT_F32 && dtype != DT_BF16) FAIL("expert_tiles: unknown dtype code %d", dtype);
   if (!expert_tiles_takes(F, width, dtype)) FAIL("expert_tiles: inner size %d and width %d must be multiples of %d", F, width, dtype == DT_BF16 ? 8 : 4);
   if (n_experts > 8192) FAIL("expert_tiles: %d experts are more than the sorting block's LDS holds", n_experts);
+  if ((size_t)n_tokens * ldx >= (1u << 31) || (size_t)n_tokens * top * F >= (1u << 31) || (size_t)F * width >= (1u << 31))
+    FAIL("expert_tiles: operands of 2^31 elements or more are not supported");
   if (ldx % (dtype == DT_BF16 ? 8 : 4) || ((uintptr_t)x & 15)) FAIL("expert_tiles: the rows of x must be 16-byte aligned");
   if (act_kind != EXPERT_SILU && act_kind != EXPERT_CLAMPED) FAIL("expert_tiles: unknown activation code %d", act_kind);
   const ExpertAct fn = {act_kind, act_limit};
-  const int n_items = n_tokens * top, most = expert_tiles_most(n_items, n_experts);
-  hipLaunchKernelGGL(expert_sort_kernel, dim3(1), dim3(1024), 2 * n_experts * sizeof(int), stream, idx, n_items, n_experts,
-                     order, tiles, n_tiles);
-  // (wide blocks where the tiles alone fill the GPU, narrow ones where they are few)
-  const bool wide = (long)most * ((F + 255) / 256) >= 256;
-  const int per = wide ? 256 : 64;
-  dim3 block(256), up_grid(most, (F + per - 1) / per), down_grid(most, (width + per - 1) / per), sum_grid(n_tokens, (width + 255) / 256);
-#define RUN(T, CF)                                                                                                       \
-  do {                                                                                                                   \
-    hipLaunchKernelGGL((expert_tiles_up_kernel<T, CF>), up_grid, block, 0, stream, (const T*)x, ldx, (const T*)w_gate,   \
-                       (const T*)w_up, order, tiles, n_tiles, weight, top, F, width, (T*)act, fn);                       \
-    hipLaunchKernelGGL((expert_tiles_down_kernel<T, CF>), down_grid, block, 0, stream, (const T*)act, (const T*)w_down,  \
-                       order, tiles, n_tiles, F, width, out);                                                            \
-    hipLaunchKernelGGL(expert_combine_kernel<T>, sum_grid, block, 0, stream, out, idx, weight, (const T*)x, ldx,         \
-                       n_experts, top, width, y, ldy, accumulate);                                                       \
-  } while (0)
+  const int n_items = n_tokens * top;
+  const dim3 block(256), sum_grid(n_tokens, (width + 255) / 256);
+  // tiles of as many picks as an expert has on average: an expert's weights are then read about once
+  const int each = n_items / n_experts;
+  const int picks = dtype == DT_F32 ? TILE_PICKS : each >= 96 ? 128 : each >= 40 ? 64 : TILE_PICKS_LEAST;
+  const int most = (n_items + picks - 1) / picks + n_experts;
+  hipLaunchKernelGGL(expert_sort_kernel, dim3(1), dim3(1024), 3 * n_experts * sizeof(int), stream, idx, n_items, n_experts,
+                     picks, order, tiles, n_tiles);
   if (dtype == DT_F32) {
-    if (wide) RUN(float, 4); else RUN(float, 1);
-  } else {
-    if (wide) RUN(bf16, 4); else RUN(bf16, 1);
-  }
+    // (wide blocks where the tiles alone fill the GPU, narrow ones where they are few)
+    const bool wide = (long)most * ((F + 255) / 256) >= 256;
+    const int per = wide ? 256 : 64;
+    const dim3 up_grid(most, (F + per - 1) / per), down_grid(most, (width + per - 1) / per);
+#define RUN(CF)                                                                                                             \
+  do {                                                                                                                      \
+    hipLaunchKernelGGL((expert_tiles_up_kernel<float, CF>), up_grid, block, 0, stream, (const float*)x, ldx,                 \
+                       (const float*)w_gate, (const float*)w_up, order, tiles, n_tiles, weight, top, F, width, (float*)act, fn); \
+    hipLaunchKernelGGL((expert_tiles_down_kernel<float, CF>), down_grid, block, 0, stream, (const float*)act,                \
+                       (const float*)w_down, order, tiles, n_tiles, F, width, out);                                         \
+  } while (0)
+    if (wide) RUN(4); else RUN(1);
 #undef RUN
+    hipLaunchKernelGGL(expert_combine_kernel<float>, sum_grid, block, 0, stream, out, idx, weight, (const float*)x, ldx, n_experts,
+                       top, width, y, ldy, accumulate, nn);
+  } else {
+#define RUN(WM, WN, TM)                                                                                                     \
+  do {                                                                                                                      \
+    const long up_blocks = (long)most * ((F + 32 * WN - 1) / (32 * WN)), down_blocks = (long)most * ((width + 64 * WN - 1) / (64 * WN)); \
+    hipLaunchKernelGGL((expert_gemm_kernel<WM, WN, TM, true>), dim3((unsigned)((up_blocks + 7) / 8 * 8)), dim3(64 * WM * WN), 0,  \
+                       stream, (const uint16_t*)x, ldx, (const uint16_t*)w_gate, (const uint16_t*)w_up, order, tiles,         \
+                       n_tiles, weight, top, F, width, act, fn);                                                            \
+    hipLaunchKernelGGL((expert_gemm_kernel<WM, WN, TM, false>), dim3((unsigned)((down_blocks + 7) / 8 * 8)), dim3(64 * WM * WN), 0, \
+                       stream, (const uint16_t*)act, F, (const uint16_t*)w_down, (const uint16_t*)nullptr, order, tiles,     \
+                       n_tiles, weight, top, width, F, out, fn);                                                            \
+  } while (0)
+    if (picks == 128) RUN(2, 2, 2);
+    else if (picks == 64) RUN(2, 2, 1);
+    else RUN(1, 2, 1);
+#undef RUN
+    hipLaunchKernelGGL(expert_combine_kernel<bf16>, sum_grid, block, 0, stream, out, idx, weight, (const bf16*)x, ldx, n_experts,
+                       top, width, y, ldy, accumulate, nn);
+  }
   CHECK_LAUNCH("expert_tiles");
   return 0;
 }

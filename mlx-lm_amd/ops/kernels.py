@@ -1448,6 +1448,15 @@ class NextNorm(ctypes.Structure):
     _fields_ = [("alpha", _vp), ("w", _vp), ("b", _vp), ("out", _vp)]
 
 
+def _next_norm(after, x, accumulate):
+    out, norm = after
+    _need(out.is_contiguous() and out.dtype == x.dtype and out.shape == x.shape and accumulate, "experts: after goes with rows that are complete here")
+    nn = NextNorm()
+    nn.alpha, nn.w, nn.b = (p.value for p in _tanh_norm(norm, x.shape[1]))
+    nn.out = out.data_ptr()
+    return nn
+
+
 ROUTED_MOST = 64  # up to this many picks a token, ``expert_rows`` makes the choice itself
 
 
@@ -1476,7 +1485,7 @@ def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=Tr
     _dev(idx, "idx", torch.int32)
     _dev(weight, "weight", torch.float32)
     _need(idx.numel() >= T * top and weight.numel() >= T * top, "expert_rows: idx / weight too short")
-    rt = nn = None
+    rt, nn = None, None
     if route is not None:
         z, correction, renormalize, weight_scale = route
         rt = RouteArgs()
@@ -1488,11 +1497,7 @@ def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=Tr
             rt.correction = correction.data_ptr()
         rt.renorm, rt.mult = int(bool(renormalize)), float(weight_scale)
     if after is not None:
-        out, norm = after
-        _need(out.is_contiguous() and out.dtype == x.dtype and tuple(out.shape) == (T, width) and accumulate, "expert_rows: after")
-        nn = NextNorm()
-        nn.alpha, nn.w, nn.b = (p.value for p in _tanh_norm(norm, width))
-        nn.out = out.data_ptr()
+        nn = _next_norm(after, x, accumulate)
     rc = lib.expert_rows(_ptr(x), _c_int(ldx), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _ptr(idx), _ptr(weight),
                          _c_int(T), _c_int(n_experts), _c_int(top), _c_int(F), _c_int(width), _ptr(act), _ptr(y),
                          _c_int(ldy), _c_int(int(bool(accumulate))), _c_int(DT[x.dtype]),
@@ -1507,9 +1512,9 @@ def expert_tiles_takes(inner, width, dtype):
     return bool(build.load("experts").expert_tiles_takes(_c_int(inner), _c_int(width), _c_int(DT[dtype])))
 
 
-def expert_tiles(y, x, w_gate, w_up, w_down, idx, weight, top, alloc, accumulate=True, activation="silu", limit=0.0):
+def expert_tiles(y, x, w_gate, w_up, w_down, idx, weight, top, alloc, accumulate=True, activation="silu", limit=0.0, after=None):
     """What ``expert_rows`` computes, for many tokens: the picks are sorted by expert on the device
-    and every tile of up to 64 picks of one expert is a small product on the matrix cores.
+    and every tile of 32 to 128 picks of one expert is a small product on the matrix cores.
     ``alloc(shape, dtype)`` gives the work memory (the sorted list, the tiles, the activations
     and a float32 row for every pick)."""
     lib = build.load("experts")
@@ -1530,7 +1535,8 @@ def expert_tiles(y, x, w_gate, w_up, w_down, idx, weight, top, alloc, accumulate
     rc = lib.expert_tiles(_ptr(x), _c_int(ldx), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _ptr(idx), _ptr(weight), _c_int(T),
                           _c_int(n_experts), _c_int(top), _c_int(F), _c_int(width), _ptr(order), _ptr(tiles), _ptr(n_tiles),
                           _ptr(act), _ptr(out), _ptr(y), _c_int(ldy), _c_int(int(bool(accumulate))), _c_int(DT[x.dtype]),
-                          *_expert_activation(activation, limit), _stream())
+                          *_expert_activation(activation, limit),
+                          ctypes.byref(_next_norm(after, x, accumulate)) if after is not None else None, _stream())
     build.check(lib, rc, "expert_tiles")
     return y
 

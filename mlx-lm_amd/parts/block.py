@@ -252,7 +252,7 @@ class SharedNormBlock(Block):
     product of the norm (``ProjectsFirst``) makes norm and product itself, and where the feed-forward
     starts with one too (``input_names``, ``projection_given``) its rows come out of the same product.
     ``next_norm``: the norm (a ``PartSpec``) that the following layer starts with, if it is one without
-    statistics: in steps of few tokens the feed-forward, which completes the rows, leaves it for that
+    statistics: the feed-forward, which completes the rows, leaves it for that
     layer (``ctx.shared["normed_rows"]``).  The
     run's state slot holds the convolution's inputs and, behind them, what a mixer that keeps
     state beside its pages (``wants_state``) asks for.  No counterpart in mlx_lm/models/gpt2.py,
@@ -378,8 +378,14 @@ class SharedNormBlock(Block):
 
     def _forward_plain(self, ctx, h, cache, writes_cache):
         after = None
-        if self.next_norm is not None and h.shape[0] < self.ffn.TILES_FROM:
-            after = (ctx.scratch(tuple(h.shape), ctx.dtype), self.next_norm.operands)  # (kept beyond this layer)
+        if self.next_norm is not None:
+            # two buffers by turns, kept beyond this layer: the norm that this layer reads, the one it leaves
+            buffers = ctx.shared.setdefault("norm_buffers", [])
+            if len(buffers) < 2:
+                buffers.append(ctx.scratch(tuple(h.shape), ctx.dtype))
+            else:
+                buffers.reverse()
+            after = (buffers[-1], self.next_norm.operands)
         mark = ctx.scratch_mark()
         if hasattr(self.mixer, "project"):
             u, rows, more = self.mixer.project(ctx, h, self.norm, cache)
@@ -391,7 +397,8 @@ class SharedNormBlock(Block):
             options = {} if more is None else {"rows": more}
             if after is not None:
                 options["after"] = after
-            if self.ffn.forward(ctx, u, h, **options) and after is not None:
+            self.ffn.forward(ctx, u, h, **options)
+            if after is not None:
                 ctx.shared["normed_rows"] = after[0]
         ctx.scratch_release(mark)
         return h

@@ -24,9 +24,9 @@ class GatedExperts(FeedForward):
     (``renormalize`` without a correction is the softmax over the chosen outputs alone.)
 
     The choice runs on the device (csrc/experts.hip), so a step launches kernels only.  For few
-    tokens the chosen experts' weights are read straight from the stacked tensors, a wave a
-    feature, by kernels that touch nothing else; for many tokens the picks are sorted by expert on
-    the device and go to the matrix cores in tiles of up to 64 picks of one expert.  The shared
+    tokens the chosen experts' weights are read straight from the stacked tensors, a wave four
+    features, by kernels that touch nothing else; for many tokens the picks are sorted by expert on
+    the device and go to the matrix cores in tiles of 32 to 128 picks of one expert.  The shared
     expert goes through the framework's products.  No counterpart in
     mlx_lm/models/gpt2.py, whose feed-forward (:71-84) is dense.
     """
@@ -34,7 +34,9 @@ class GatedExperts(FeedForward):
     graph_safe = True  # launches kernels only: a step of such parts can be recorded
     can_overwrite = True
     MERGED_UP_TO = 16  # up to this many tokens the router's and the shared expert's first products are one
-    TILES_FROM = 64  # from this many tokens in a step the picks are sorted and go to the matrix cores in tiles
+    # From TILES_FROM tokens in a step, or in bfloat16 from TILES_MIN tokens if every expert has TILES_EACH
+    # picks on average, the picks are sorted and go to the matrix cores in tiles.
+    TILES_FROM, TILES_MIN, TILES_EACH = 64, 8, 3
 
     def __init__(self, width, n_experts, inner, top, n_identity=0, shared_inner=0, correction=True, renormalize=False,
                  weight_scale=1.0, activation="silu", limit=0.0, prefix=""):
@@ -107,11 +109,12 @@ class GatedExperts(FeedForward):
     def forward(self, ctx, x, residual, rows=None, after=None):
         """``rows``: the router's float32 outputs, where the caller has made them already.  ``after``:
         ``(out, norm operands)`` of a dynamic tanh over the rows that this completes, for the layer
-        behind; returns whether it was made (steps of few tokens only)."""
+        behind (made by the last kernel here)."""
         T = x.shape[0]
         merged = self.shared_inner and T <= self.MERGED_UP_TO and rows is None
         mark = ctx.scratch_mark()
-        tiles = self.n_experts and T >= self.TILES_FROM and kernels.expert_tiles_takes(self.inner, self.width, x.dtype)
+        many = T >= self.TILES_FROM or (x.dtype == torch.bfloat16 and T >= self.TILES_MIN and T * self.top >= self.TILES_EACH * self.n_experts)
+        tiles = self.n_experts and many and kernels.expert_tiles_takes(self.inner, self.width, x.dtype)
         route = None
         idx = ctx.scratch((T, self.top), torch.int32)
         weight = ctx.scratch((T, self.top), torch.float32)
@@ -142,13 +145,12 @@ class GatedExperts(FeedForward):
             accumulate = True
         if tiles:
             kernels.expert_tiles(residual, x, self.w_gate, self.w_up, self.w_down, idx, weight, self.top, ctx.scratch,
-                                 accumulate=accumulate, activation=self.activation, limit=self.limit)
+                                 accumulate=accumulate, activation=self.activation, limit=self.limit, after=after)
         else:
             act = ctx.scratch((T * self.top, self.inner), ctx.dtype) if self.n_experts else None
             kernels.expert_rows(residual, x, self.w_gate, self.w_up, self.w_down, idx, weight, self.top, act,
                                 accumulate=accumulate, activation=self.activation, limit=self.limit, route=route, after=after)
         ctx.scratch_release(mark)
-        return after is not None and not tiles
 
 
 register_feed_forward("gated_experts", GatedExperts)

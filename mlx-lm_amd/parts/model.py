@@ -169,6 +169,7 @@ class DecoderModel:
         One call into the native host, which walks the parts: embedding (+ position term),
         the scheduled blocks, the final norm on the wanted rows only, the head."""
         logits = None
+        ctx.shared.clear()  # (a step that is recorded walks the model twice over the same scratch memory)
         if ctx.n_wanted:
             logits = ctx.logits_out(ctx.n_wanted, self.vocab_size)
             ctx.c.logits, ctx.c.logits_rows = logits.data_ptr(), logits.shape[0]

@@ -359,16 +359,18 @@ def test_the_bonus_recurrence_in_portions_of_two_requests(H, N, rank, wide):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("T", [3, 80])
-@pytest.mark.parametrize("F,top", [(24, 2), (9, 1), (64, 5)])
-def test_clamped_experts_with_weights_over_the_chosen_alone(dtype, T, F, top):
+@pytest.mark.parametrize("T", [3, 80, 300])
+@pytest.mark.parametrize("F,top,W", [(24, 2, 48), (9, 1, 48), (64, 5, 48), (136, 3, 200)])
+def test_clamped_experts_with_weights_over_the_chosen_alone(dtype, T, F, top, W):
+    """A few tokens, and tiles of 32, 64 and 128 picks of an expert (one expert gets few picks)."""
     from mlx_lm_amd.ops import kernels
 
     g = torch.Generator().manual_seed(F + top)
-    E, W, limit = 5, 48, 0.6
+    E, limit = 5, 0.6
     x = torch.randn(T, W, generator=g).to(dtype)
     gate, up, down = ((torch.randn(*s, generator=g) * s[-1] ** -0.5 * f).to(dtype) for s, f in (((E, F, W), 2.0), ((E, F, W), 2.0), ((E, W, F), 1.0)))
     z = torch.randn(T, E, generator=g) * 3
+    z[:, 2] -= 4.0
     idx, weight = torch.empty(T, top, dtype=torch.int32, device="cuda"), torch.empty(T, top, device="cuda")
     kernels.router_choice(idx, weight, z.cuda(), None, top, renormalize=True)
     y = torch.full((T, W), 0.5, device="cuda")
@@ -416,6 +418,11 @@ def test_the_choice_and_the_next_norm_inside_the_experts_kernels(dtype, F, width
     want = torch.empty_like(out)
     kernels.dynamic_tanh(want, y, norm)
     assert torch.equal(out, want)
+    if kernels.expert_tiles_takes(F, width, dtype):
+        y3 = start.clone()
+        kernels.expert_tiles(y3, x, gate, up, down, idx, weight, top, _alloc, activation="clamped", limit=0.8, after=(out, norm))
+        kernels.dynamic_tanh(want, y3, norm)
+        assert torch.equal(out, want)
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
