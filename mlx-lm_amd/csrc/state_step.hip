@@ -2,7 +2,7 @@
 // between a mixer's projection and its output projection in one launch:
 //
 //   STEP_DELTA      the gated delta rule on prepared rows (queries scaled, keys of unit length)
-//                     S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+//                     u = beta (v - g S^T k);  S <- g S + k u^T;  o = S^T q  (the new S)
 //   STEP_DELTA_RAW  the same from the projection's own columns, one token a request: a causal
 //                   convolution per channel with silu, queries and keys made unit vectors, beta =
 //                   sigmoid(.), g = exp(-exp(A_log) softplus(. + dt_bias)).  The convolution's last
@@ -10,7 +10,7 @@
 //                   that is written is none of those that are read, so the heads that share a key
 //                   head read it side by side.
 //   STEP_BONUS      a decay per key channel and a bonus for the current token
-//                     o = (S + diag(u) k v^T)^T r;  S <- diag(w) S + k v^T
+//                     o = S^T r + (r . (u * k)) v;  S <- diag(w) S + k v^T
 //                   with w = exp(-exp(w0 + W2 tanh(z))) made here from the low-rank middle z.
 //
 // A block a (head, request); S [N][P] lies in the threads' registers, asked for at once and written

@@ -1811,7 +1811,7 @@ def state_step(out, q, k, v, state, state_offset, seq_start, seq_len, slot_ids, 
     registers; the heads' output divided by its root mean square, times ``norm_weight`` (``value_dim``
     values, or that many a head) and ``silu(gate)``.
 
-    * the gated delta rule ``S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q`` on prepared
+    * the gated delta rule ``u = beta (v - g S^T k); S <- g S + k u^T; o = S^T q`` on prepared
       rows: ``log_g``, ``beta`` float32 ``[rows, n_heads]``;
     * with ``raw`` (a ``DeltaRaw``; every request brings one token) the same from the projection's
       columns, ``beta`` and ``log_g`` the columns that become them (convolution, silu, unit vectors,

@@ -11,7 +11,7 @@ from .linear_state import _SequenceArrays, _matrix, _padded_columns, _rows_for
 class GatedDeltaRule(ProjectsFirst, _SequenceArrays, Mixer):
     """The gated delta rule, per head with a matrix state ``S`` (``key_dim x value_dim``):
 
-        ``S <- g S``,   ``u = beta (v - S^T k)``,   ``S <- S + k u^T``,   ``o = S^T q``
+        ``d_t = beta_t (v_t - g_t S_(t-1)^T k_t)``,   ``S_t = g_t S_(t-1) + k_t d_t^T``,   ``o_t = S_t^T q_t``
 
     ``q = Wq x``, ``k = Wk x`` (``n_key_heads x key_dim``; head ``h`` reads key head ``h // (n_heads /
     n_key_heads)``) and ``v = Wv x`` (``n_heads x value_dim``) each pass a short causal convolution per

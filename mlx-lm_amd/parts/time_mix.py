@@ -9,12 +9,12 @@ from .linear_state import _SequenceArrays, _matrix, _padded_columns, _rows_for
 
 
 class TimeMix(_SequenceArrays, Mixer):
-    """Time mixing in the manner of RWKV.  With ``h'`` the previous token's ``h`` (zeros for a request's
-    first), every projection reads a mix of its own, ``m_s = h + (h' - h) * mu_s``: ``r``, ``k``, ``v``
+    """Time mixing in the manner of RWKV.  With ``h'`` the ``h`` of the token before (zeros ahead of a
+    request's first), every projection reads a mix of its own, ``m_s = h + (h' - h) * mu_s``: ``r``, ``k``, ``v``
     (``n_heads x head_dim``), a gate ``silu(Wg m_g)`` and the decay, per head and key channel, through a
     narrow middle of ``decay_rank``, ``w = exp(-exp(W2 tanh(W1 m_w) + w0))``.  Per head
 
-        ``o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t``,   ``S_t = diag(w_t) S_(t-1) + k_t v_t^T``
+        ``o_t = S_(t-1)^T r_t + (r_t . (u * k_t)) v_t``,   ``S_t = diag(w_t) S_(t-1) + k_t v_t^T``
 
     with the bonus ``u`` for the current token only.  Each head's ``o`` is divided by its root mean
     square (``eps``), the heads side by side times ``norm`` (``n_heads * head_dim`` values) and the

@@ -47,7 +47,7 @@ def causal_conv(u, taps_w):
 
 def delta_recurrence(q, k, v, g, beta):
     """One head: ``q``, ``k`` ``[T, N]``, ``v`` ``[T, P]``, ``g``, ``beta`` ``[T]``.
-    ``S <- g S; S <- S + k (beta (v - S^T k))^T; o = S^T q``."""
+    The state decays, then takes the step towards ``v`` at ``k``, then answers ``q``."""
     S = torch.zeros(q.shape[1], v.shape[1], dtype=q.dtype)
     out = []
     for t in range(q.shape[0]):
@@ -73,7 +73,7 @@ def delta_mixer(h, w, p, m, eps):
 
 def wkv_recurrence(r, k, v, decay, u):
     """One head: ``r``, ``k``, ``decay`` ``[T, N]``, ``v`` ``[T, N]``, ``u`` ``[N]``.
-    ``o = (S + diag(u) k v^T)^T r; S <- diag(decay) S + k v^T``."""
+    The state as it was and the bonus answer ``r``; then the state decays and takes ``k v^T``."""
     S = torch.zeros(r.shape[1], v.shape[1], dtype=r.dtype)
     out = []
     for t in range(r.shape[0]):
