@@ -8,7 +8,8 @@ MODEL_REMAPPING = {}
 _REGISTRY = {}
 _BUILTIN = {"gpt2": "mlx_lm_amd.models.gpt2", "pafutar": "mlx_lm_amd.models.pafutar",
             "ruzolorn": "mlx_lm_amd.models.ruzolorn", "zatinex": "mlx_lm_amd.models.zatinex",
-            "sazilorn": "mlx_lm_amd.models.sazilorn", "gilidra": "mlx_lm_amd.models.gilidra"}
+            "sazilorn": "mlx_lm_amd.models.sazilorn", "gilidra": "mlx_lm_amd.models.gilidra",
+            "lutodra": "mlx_lm_amd.models.lutodra"}
 
 
 def register_model(model_type, model_cls, args_cls):

@@ -58,6 +58,11 @@ struct AttnArgs {
   float softcap;
   const float* dist_bias;
   int n_dist;
+  // sinks [n_heads]: exp(sinks[h]) in the softmax's denominator; head_gate (rows of stride ldhg): head
+  // h's output times the sigmoid of column h
+  const float* sinks;
+  const float* head_gate;
+  int ldhg;
 };
 
 // A scaled score with the optional terms that depend on the head and the distance.
@@ -325,7 +330,7 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(AttnArgs p) {
   for (int i = 0; i < 4; ++i) {
     const int qi = wave * 4 + i;
     if (qi >= nq) continue;
-    const float inv = 1.0f / l[i];
+    const float inv = head_gate_of(p, row0 + qi, h) / with_sink(p, h, m[i], l[i]);
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int d = lane + 64 * j;
@@ -439,7 +444,7 @@ __global__ __launch_bounds__(256) void attn_tile_wide_kernel(AttnArgs p) {
   for (int i = 0; i < 4; ++i) {
     const int qi = wave * 4 + i;
     if (qi >= nq) continue;
-    const float inv = 1.0f / l[i];
+    const float inv = head_gate_of(p, row0 + qi, h) / with_sink(p, h, m[i], l[i]);
 #pragma unroll
     for (int j = 0; j < NJ; ++j) {
       const int d = lane + 64 * j;
@@ -582,7 +587,7 @@ __global__ __launch_bounds__(256) void attn_tile_mfma_kernel(AttnArgs p, int n_t
   }
 
   if (x < nq) {
-    const float inv = 1.0f / l;
+    const float inv = head_gate_of(p, row0 + x, h) / with_sink(p, h, m, l);
     float* orow = (float*)p.out + (size_t)(row0 + x) * p.ldo + h * HD + 16 * g;
 #pragma unroll
     for (int v = 0; v < NV; ++v)
@@ -704,13 +709,14 @@ __global__ __launch_bounds__(256) void attn_row_kernel(AttnArgs p) {
     w[i] = (Ms[i] == -INFINITY) ? 0.f : expf(Ms[i] - M);
     L += Ls[i] * w[i];
   }
+  const float scale_out = p.n_splits == 1 ? head_gate_of(p, row, h) / with_sink(p, h, M, L) : 0.f;
   for (int d = tid; d < hd; d += 256) {
     float acc = 0.f;
 #pragma unroll
     for (int i = 0; i < 4; ++i) acc += Os[i * hd + d] * w[i];
     if (p.n_splits == 1) {
       ((T*)p.out)[(size_t)row * p.ldo + h * hd + d] =
-          from_f32<T>(acc / L * gate_of(p, row, h * hd + d, sizeof(T) == 2));
+          from_f32<T>(acc * scale_out * gate_of(p, row, h * hd + d, sizeof(T) == 2));
     } else {
       const size_t base = ((size_t)item * p.n_heads + h) * p.n_splits + split;
       p.part_o[base * hd + d] = acc;
@@ -733,6 +739,7 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(AttnArgs p) {
     const float ms = p.part_ml[(base + s) * 2];
     if (ms != -INFINITY) L += p.part_ml[(base + s) * 2 + 1] * expf(ms - M);
   }
+  const float scale_out = head_gate_of(p, row, h) / with_sink(p, h, M, L);
   for (int d = threadIdx.x; d < hd; d += 64) {
     float acc = 0.f;
     for (int s = 0; s < p.n_splits; ++s) {
@@ -740,7 +747,7 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(AttnArgs p) {
       if (ms != -INFINITY) acc += p.part_o[(base + s) * hd + d] * expf(ms - M);
     }
     ((T*)p.out)[(size_t)row * p.ldo + h * hd + d] =
-        from_f32<T>(acc / L * gate_of(p, row, h * hd + d, sizeof(T) == 2));
+        from_f32<T>(acc * scale_out * gate_of(p, row, h * hd + d, sizeof(T) == 2));
   }
 }
 
@@ -820,6 +827,7 @@ static int fill_args(AttnArgs& p, const char* who, void* out, const void* q, int
   p.window = window, p.n_splits = 1, p.scale = scale;
   p.head_scale = nullptr, p.slopes = nullptr, p.gate = nullptr, p.ldg = 0, p.keep_first = 0;
   p.softcap = 0.f, p.dist_bias = nullptr, p.n_dist = 0;
+  p.sinks = p.head_gate = nullptr, p.ldhg = 0;
   return 0;
 }
 
@@ -832,6 +840,7 @@ static int fill_extras(AttnArgs& p, const char* who, const float* head_scale, co
   p.keep_first = p.window > 0 ? keep_first : 0;  // (without a window every key is visible anyway)
   return 0;
 }
+// (the sink and the heads' gate enter behind the scores: every kernel here takes them)
 static bool has_extras(const AttnArgs& p) {
   return p.head_scale || p.slopes || p.gate || p.keep_first > 0 || p.softcap > 0.f || p.dist_bias;
 }
@@ -840,7 +849,9 @@ static int fill_shape(AttnArgs& p, const char* who, const AttnTerms* t) {
   if (!t) return 0;
   if (t->softcap < 0.f) FAIL("%s: softcap %g must not be negative", who, (double)t->softcap);
   if (t->dist_bias && t->n_dist <= 0) FAIL("%s: a distance table of %d entries a head", who, t->n_dist);
+  if (t->head_gate && t->ldhg < p.n_heads) FAIL("%s: the heads' gate has rows of %d columns", who, t->ldhg);
   p.softcap = t->softcap, p.dist_bias = t->dist_bias, p.n_dist = t->n_dist;
+  p.sinks = t->sinks, p.head_gate = t->head_gate, p.ldhg = t->ldhg;
   return 0;
 }
 

@@ -67,6 +67,11 @@ struct DecodeArgs {
   float softcap;
   const float* dist_bias;
   int n_dist;
+  // sinks [n_heads]: exp(sinks[h]) in the softmax's denominator; head_gate (rows of stride ldhg): head
+  // h's output times the sigmoid of column h
+  const float* sinks;
+  const float* head_gate;
+  int ldhg;
 };
 
 template <typename T>
@@ -341,13 +346,15 @@ __global__ __launch_bounds__(64 * (CPK >= 16 ? MAX_WAVES / 2 : MAX_WAVES)) void 
           Mj = M2;
         }
       }
-      put((T*)p.out + out_at(p, row, h * HD + tid), aj / Lj * gate_at<T>(p, row, h * HD + tid));
+      put((T*)p.out + out_at(p, row, h * HD + tid),
+          aj / with_sink(p, h, Mj, Lj) * head_gate_of(p, row, h) * gate_at<T>(p, row, h * HD + tid));
     }
     return;
   }
   if (tid < HD) {
     if (n_splits == 1) {
-      put((T*)p.out + out_at(p, row, h * HD + tid), acc / L * gate_at<T>(p, row, h * HD + tid));
+      put((T*)p.out + out_at(p, row, h * HD + tid),
+          acc / with_sink(p, h, M, L) * head_gate_of(p, row, h) * gate_at<T>(p, row, h * HD + tid));
     } else {
       const size_t base = ((size_t)item * p.n_heads + h) * p.n_splits + split;
       p.part_o[base * HD + tid] = acc;
@@ -488,7 +495,7 @@ __global__ __launch_bounds__(256) void attn_decode_group_kernel(DecodeArgs p, in
     }
     const int hq = kv_head * group + ht * 16 + hh;
     if (p.n_splits == 1) {
-      put((uint16_t*)p.out + out_at(p, row, hq * HD + col), acc / L);
+      put((uint16_t*)p.out + out_at(p, row, hq * HD + col), acc / with_sink(p, hq, M, L) * head_gate_of(p, row, hq));
     } else {
       const size_t base = ((size_t)item * p.n_heads + hq) * p.n_splits + split;
       p.part_o[base * HD + col] = acc;
@@ -514,7 +521,7 @@ __global__ void attn_decode_merge_kernel(DecodeArgs p) {
     L += p.part_ml[(base + s) * 2 + 1] * w;
     acc += p.part_o[(base + s) * HD + d] * w;
   }
-  put((T*)p.out + out_at(p, row, h * HD + d), acc / L * gate_at<T>(p, row, h * HD + d));
+  put((T*)p.out + out_at(p, row, h * HD + d), acc / with_sink(p, h, M, L) * head_gate_of(p, row, h) * gate_at<T>(p, row, h * HD + d));
 }
 
 DEFINE_LAST_ERROR(mlxlm_last_error)
@@ -595,6 +602,9 @@ static int decode_rows_launch(void* out, const void* q, int ldq, int ldo, const 
   p.keep_first = window > 0 ? keep_first : 0;
   p.softcap = shape ? shape->softcap : 0.f, p.dist_bias = shape ? shape->dist_bias : nullptr;
   p.n_dist = shape ? shape->n_dist : 0;
+  p.sinks = shape ? shape->sinks : nullptr, p.head_gate = shape ? shape->head_gate : nullptr;
+  p.ldhg = shape ? shape->ldhg : 0;
+  if (p.head_gate && p.ldhg < n_heads) FAIL("attn_decode: the heads' gate has rows of %d columns", p.ldhg);
   if (ahead && (((uintptr_t)ahead & 15) || ahead_chunk_bytes % 16 != 0 || ahead_chunks < 0))
     FAIL("attn_decode: what is read ahead must be chunks of 16-byte pieces");
   p.ahead = (const uint4*)ahead, p.ahead_pieces = ahead ? ahead_chunk_bytes / 16 : 0;
@@ -681,12 +691,13 @@ extern "C" int attn_decode_rows(void* out, const void* q, int ldq, int ldo, cons
 // attn_decode_group: the rows of attn_decode_rows for bfloat16 caches with head_dim 64, 128 or 256,
 // all query heads of a key head in one block (see attn_decode_group_kernel).  n_splits parts of a
 // row's keys (part_o: n_rows * n_heads * n_splits * head_dim floats, part_ml: two a part; joined
-// by a second kernel).  ldo == 0: out in the packed order.
+// by a second kernel).  ldo == 0: out in the packed order.  t: of the optional terms the sinks and the
+// heads' gate, or null.
 extern "C" int attn_decode_group(void* out, const void* q, int ldq, int ldo, const void* k_pages, const void* v_pages,
                                  size_t page_stride, const int* block_table, int max_blocks, const int* token_req,
                                  const int* positions, const int* rows, int n_rows, int n_heads, int n_kv_heads,
                                  int head_dim, int page_size, int window, float scale, int n_splits, float* part_o,
-                                 float* part_ml, int rows_are_requests, hipStream_t stream) {
+                                 float* part_ml, int rows_are_requests, const AttnTerms* t, hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (head_dim != 64 && head_dim != 128 && head_dim != 256) FAIL("attn_decode_group: head_dim %d is not 64, 128 or 256", head_dim);
   if (n_heads <= 0 || n_kv_heads <= 0 || n_heads % n_kv_heads != 0)
@@ -707,6 +718,12 @@ extern "C" int attn_decode_group(void* out, const void* q, int ldq, int ldo, con
   p.n_heads = n_heads, p.n_kv_heads = n_kv_heads, p.page_size = page_size, p.window = window, p.n_splits = n_splits;
   p.scale = scale, p.out_head_dim = head_dim, p.rows_are_requests = rows_are_requests ? 1 : 0;
   p.table_in_lds = max_blocks > 0 && max_blocks <= 8192;
+  if (t) {
+    if (t->head_scale || t->slopes || t->gate || t->keep_first > 0 || t->softcap > 0.f || t->dist_bias)
+      FAIL("attn_decode_group: of the optional terms only sinks and the heads' gate");
+    if (t->head_gate && t->ldhg < n_heads) FAIL("attn_decode_group: the heads' gate has rows of %d columns", t->ldhg);
+    p.sinks = t->sinks, p.head_gate = t->head_gate, p.ldhg = t->ldhg;
+  }
   const int group = n_heads / n_kv_heads, head_tiles = (group + 15) / 16;
   if ((long)n_kv_heads * head_tiles > 65535) FAIL("attn_decode_group: %d key heads in a launch", n_kv_heads);
   const size_t lds = (size_t)4 * 16 * (head_dim + 1) * sizeof(float) + (p.table_in_lds ? (size_t)max_blocks * sizeof(int) : 0);

@@ -53,6 +53,11 @@ struct PrefillArgs {
   float softcap;
   const float* dist_bias;
   int n_dist;
+  // sinks [n_heads]: exp(sinks[h]) in the softmax's denominator; head_gate (rows of stride ldhg): head
+  // h's output times the sigmoid of column h
+  const float* sinks;
+  const float* head_gate;
+  int ldhg;
 };
 
 #define BQ ATTN_PREFILL_TILE_QUERIES  // queries per block
@@ -430,7 +435,9 @@ __global__ __launch_bounds__(256, HD <= 64 ? 2 : 1) void attn_prefill_kernel(Pre
   // the two halves of the wave hold different keys of the same query
   l += __shfl_xor(l, 32, WAVE);
   if (q_live) {
-    const float inv = 1.0f / l;
+    // (m is in units of log 2)
+    if (p.sinks) l += exp2f(fmaf(p.sinks[h], 1.4426950408889634f, -m));
+    const float inv = head_gate_of(p, row0 + qi, h) / l;
     uint16_t* orow = p.out + (size_t)(row0 + qi) * p.ldo + h * HD;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
@@ -498,6 +505,9 @@ static int prefill_launch(void* out, const void* q, int ldq, int ldo, const void
   p.keep_first = window > 0 ? keep_first : 0;
   p.softcap = shape ? shape->softcap : 0.f, p.dist_bias = shape ? shape->dist_bias : nullptr;
   p.n_dist = shape ? shape->n_dist : 0;
+  p.sinks = shape ? shape->sinks : nullptr, p.head_gate = shape ? shape->head_gate : nullptr;
+  p.ldhg = shape ? shape->ldhg : 0;
+  if (p.head_gate && p.ldhg < n_heads) FAIL("attn_prefill: the heads' gate has rows of %d columns", p.ldhg);
   const bool shaped = p.softcap > 0.f || p.dist_bias;
   const bool extras = head_scale || slopes || gate || p.keep_first > 0 || shaped;
   if (n_tiles > 65535) FAIL("attn_prefill: %d tiles in a launch, at most 65535", n_tiles);

@@ -9,7 +9,10 @@
 //   s -= slopes[h] * (query position - key position)
 //   s += dist_bias[h * n_dist + min(distance, n_dist - 1)]      (a table of float, a row a head)
 // keep_first: with a window, the first so many keys stay visible.  gate (rows of stride ldg, the
-// queries' element type): the output is multiplied by its sigmoid.
+// queries' element type): the output is multiplied by its sigmoid.  sinks [n_heads]: the softmax's
+// denominator holds exp(sinks[h]) too, a number beside the scores that brings no value.  head_gate
+// (float rows of stride ldhg, a column a head): head h's output is multiplied by the sigmoid of its
+// column.
 struct AttnTerms {
   const float* head_scale;
   const float* slopes;
@@ -18,7 +21,22 @@ struct AttnTerms {
   float softcap;
   const float* dist_bias;
   int n_dist;
+  const float* sinks;
+  const float* head_gate;
+  int ldhg;
 };
+
+#ifdef __HIPCC__
+// From l = the sum of exp(score - m) over the keys to the whole denominator (m the largest score).
+template <typename Args>
+__device__ __forceinline__ float with_sink(const Args& p, int h, float m, float l) {
+  return p.sinks ? l + expf(p.sinks[h] - m) : l;
+}
+template <typename Args>
+__device__ __forceinline__ float head_gate_of(const Args& p, int row, int h) {
+  return p.head_gate ? 1.0f / (1.0f + expf(-p.head_gate[(size_t)row * p.ldhg + h])) : 1.0f;
+}
+#endif
 
 #define ATTN_TILE_QUERIES 16           // attn_tile (attention.hip): queries a block
 #define ATTN_PREFILL_TILE_QUERIES 128  // attn_prefill (attention_prefill.hip): queries a block

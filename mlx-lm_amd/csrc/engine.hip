@@ -113,7 +113,7 @@ typedef int (*fn_attn_decode)(void*, const void*, int, int, const void*, const v
                               float*, float*, int, const void*, size_t, int, int, int, int, int, hipStream_t);
 typedef int (*fn_attn_decode_group)(void*, const void*, int, int, const void*, const void*, size_t, const int*, int,
                                     const int*, const int*, const int*, int, int, int, int, int, int, float, int,
-                                    float*, float*, int, hipStream_t);
+                                    float*, float*, int, const AttnTerms*, hipStream_t);
 typedef int (*fn_attn_prefill)(void*, const void*, int, int, const void*, const void*, size_t, const int*,
                                int, const int*, const int*, const int*, int, int, int, int, int, int, float,
                                hipStream_t);
@@ -775,7 +775,8 @@ struct Attention : Mixer {
 
   // `terms`: the optional terms of a score and of the output (attention_tiles.h), or null.  With
   // terms the kernels' `_terms` entry points are called; the kernel that takes the query heads of
-  // a key head together knows no terms, so such rows go to the streaming kernel.
+  // a key head together knows only those that enter behind the scores, so with others such rows go to
+  // the streaming kernel.
   int attend(EngCtx* ctx, const EngMat& out, const EngMat& q, const EngScatter& kv, bool out_packed,
              const AttnTerms* terms = nullptr) const {
     const int* tiles = ctx->arrays[array_base + ARR_TILES];
@@ -836,7 +837,9 @@ struct Attention : Mixer {
       // A block is four waves of sixteen keys at a time; a part for every 128 keys of the longest
       // row, as many as give every CU two blocks.
       const int group = n_heads / n_kv_heads;
-      if (!terms && bf16 && group >= 8 && (head_dim == 64 || head_dim == 128 || head_dim == 256)) {
+      const bool plain_scores = !terms || !(terms->head_scale || terms->slopes || terms->gate || terms->keep_first > 0 ||
+                                            terms->softcap > 0.f || terms->dist_bias);
+      if (plain_scores && bf16 && group >= 8 && (head_dim == 64 || head_dim == 128 || head_dim == 256)) {
         const long c = window <= 0 ? max_row_context : (max_row_context < window + 15 ? max_row_context : window + 15);
         const long blocks = (long)n_rows * n_kv_heads * ((group + 15) / 16);
         long ns = c / 128, most = 2L * ctx->n_compute_units / (blocks < 1 ? 1 : blocks);
@@ -852,7 +855,7 @@ struct Attention : Mixer {
         }
         KERNEL(k_attn_decode_group, ctx, out.p, q.p, q.ld, out_packed ? 0 : out.ld, kv.k, kv.v, kv.page_stride,
                kv.block_table, kv.max_blocks, kv.token_req, kv.positions, rows, n_rows, n_heads, n_kv_heads, head_dim,
-               kv.page_size, window, scale, (int)ns, (float*)group_o.p, (float*)group_ml.p, rows_are_requests, ctx->stream);
+               kv.page_size, window, scale, (int)ns, (float*)group_o.p, (float*)group_ml.p, rows_are_requests, terms, ctx->stream);
         return 0;
       }
       if (fast)
@@ -1300,6 +1303,7 @@ static int attend_slot(EngCtx* ctx, const EngMat* out, const EngMat* q, int slot
   EngScatter kv;
   TRY(a.scatter_for(ctx, slot, &kv));
   if (terms && terms->gate && terms->ldg < q->cols) FAIL("eng_attend: the gate's rows are shorter than the queries'");
+  if (terms && terms->head_gate && terms->ldhg < n_heads) FAIL("eng_attend: the heads' gate has rows of %d columns", terms->ldhg);
   return a.attend(ctx, *out, *q, kv, false, terms);
 }
 

@@ -1,6 +1,7 @@
 // A feed-forward of many small gated experts of which every token uses a few:
-//   router_choice   s = softmax(z) over all router outputs; the `top` largest of s + correction
-//                   are chosen (the lower index on a tie); their weights are s itself.
+//   router_choice   s = softmax(z) over all router outputs, or the logistic function of each; the `top`
+//                   largest of s + correction are chosen (the lower index on a tie), out of all or out
+//                   of the best groups of neighbours; their weights are s itself.
 //   silu_mul        act = silu(gate) * up for rows [gate | up]   (a dense gated feed-forward)
 //   route_and_gate  both of these in one launch, for a step of few tokens whose router, gate and up
 //                   came out of one product as float rows
@@ -40,13 +41,83 @@ __device__ __forceinline__ float expert_act(const ExpertAct& a, float g, float u
   return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
 }
 
+// How a token's experts are chosen from its router outputs.
+struct RouteArgs {
+  const float* z;  // [tokens, ldz], or null: idx and weight hold the choice already
+  int ldz;
+  const float* correction;  // added to a score for the choice only, or null
+  int n_out, renorm;        // renorm: the picks' weights are divided by their sum (+ 1e-20)
+  float mult;               // and multiplied by this
+  int sigmoid;              // a score is the logistic function of its output instead of the softmax over all
+  int groups, keep;         // groups > 1: only outputs of the `keep` best of so many equal groups of neighbours
+                            // can be chosen; a group counts the sum of its two largest choice scores
+};
+
 // A wave a token, up to ROUTER_PER_LANE outputs a lane.  The k-th pick is the largest choice score
 // not picked yet, the lowest index on a tie.
 #define ROUTER_PER_LANE 8
-// `renorm`: the picks' weights are divided by their sum (+ 1e-20); `mult`: and multiplied by this.
-__device__ __forceinline__ void route_token(const float* __restrict__ zr, const float* __restrict__ correction, int n_out,
-                                            int top, int* __restrict__ idx, float* __restrict__ weight, int lane,
-                                            int renorm = 0, float mult = 1.f) {
+
+// The largest of c over the wave and the lowest index that holds it.
+__device__ __forceinline__ int wave_argmax(const float (&c)[ROUTER_PER_LANE], int lane, float* value) {
+  float best = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < ROUTER_PER_LANE; ++i) best = fmaxf(best, c[i]);
+  best = wave_max(best);
+  float first = -1e9f;  // minus the lowest index that holds the best score (indices are exact in a float)
+#pragma unroll
+  for (int i = ROUTER_PER_LANE - 1; i >= 0; --i)
+    if (c[i] == best) first = -(float)(lane + 64 * i);
+  *value = best;
+  return (int)(-wave_max(first));
+}
+
+// Choice scores outside the best groups become minus infinity.
+__device__ __forceinline__ void limit_groups(float (&c)[ROUTER_PER_LANE], int n_out, int groups, int keep, int lane) {
+  const int size = n_out / groups;
+  float score[ROUTER_PER_LANE];  // group lane + 64 i
+#pragma unroll
+  for (int i = 0; i < ROUTER_PER_LANE; ++i) score[i] = -INFINITY;
+  for (int g = 0; g < groups; ++g) {
+    float m1 = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < ROUTER_PER_LANE; ++i) {
+      const int e = lane + 64 * i;
+      if (e / size == g && e < n_out) m1 = fmaxf(m1, c[i]);
+    }
+    m1 = wave_max(m1);
+    float m2 = -INFINITY;
+    int equal = 0;
+#pragma unroll
+    for (int i = 0; i < ROUTER_PER_LANE; ++i) {
+      const int e = lane + 64 * i;
+      const bool in = e / size == g && e < n_out;
+      equal += __popcll(__ballot(in && c[i] == m1));
+      if (in && c[i] != m1) m2 = fmaxf(m2, c[i]);
+    }
+    m2 = equal > 1 ? m1 : wave_max(m2);
+    const float total = size > 1 ? m1 + m2 : m1;
+#pragma unroll
+    for (int i = 0; i < ROUTER_PER_LANE; ++i)
+      if (lane + 64 * i == g) score[i] = total;
+  }
+  unsigned kept = 0u;  // a bit an output of this lane
+  for (int j = 0; j < keep; ++j) {
+    float best;
+    const int g = wave_argmax(score, lane, &best);
+#pragma unroll
+    for (int i = 0; i < ROUTER_PER_LANE; ++i) {
+      if (lane + 64 * i == g) score[i] = -INFINITY;
+      if ((lane + 64 * i) / size == g) kept |= 1u << i;
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < ROUTER_PER_LANE; ++i)
+    if (!(kept >> i & 1u)) c[i] = -INFINITY;
+}
+
+__device__ __forceinline__ void route_token(const float* __restrict__ zr, const RouteArgs& a, int top, int* __restrict__ idx,
+                                            float* __restrict__ weight, int lane) {
+  const int n_out = a.n_out;
   float v[ROUTER_PER_LANE], c[ROUTER_PER_LANE];
   float m = -INFINITY;
 #pragma unroll
@@ -55,34 +126,34 @@ __device__ __forceinline__ void route_token(const float* __restrict__ zr, const 
     v[i] = e < n_out ? zr[e] : -INFINITY;
     m = fmaxf(m, v[i]);
   }
-  m = wave_max(m);
-  float sum = 0.f;
+  if (a.sigmoid) {
 #pragma unroll
-  for (int i = 0; i < ROUTER_PER_LANE; ++i) {
-    v[i] = lane + 64 * i < n_out ? expf(v[i] - m) : 0.f;
-    sum += v[i];
+    for (int i = 0; i < ROUTER_PER_LANE; ++i) v[i] = 1.0f / (1.0f + expf(-v[i]));
+  } else {
+    m = wave_max(m);
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < ROUTER_PER_LANE; ++i) {
+      v[i] = lane + 64 * i < n_out ? expf(v[i] - m) : 0.f;
+      sum += v[i];
+    }
+    const float inv = 1.0f / wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < ROUTER_PER_LANE; ++i) v[i] *= inv;
   }
-  const float inv = 1.0f / wave_sum(sum);
 #pragma unroll
   for (int i = 0; i < ROUTER_PER_LANE; ++i) {
     const int e = lane + 64 * i;
-    v[i] *= inv;
-    c[i] = e < n_out ? (correction ? v[i] + correction[e] : v[i]) : -INFINITY;
+    c[i] = e < n_out ? (a.correction ? v[i] + a.correction[e] : v[i]) : -INFINITY;
   }
+  if (a.groups > 1) limit_groups(c, n_out, a.groups, a.keep, lane);
   float mine[ROUTER_PER_LANE];  // pick j's weight, kept by lane j % 64 until the picks' sum is known
 #pragma unroll
   for (int i = 0; i < ROUTER_PER_LANE; ++i) mine[i] = 0.f;
   float total = 0.f;
   for (int j = 0; j < top; ++j) {
-    float best = -INFINITY;
-#pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i) best = fmaxf(best, c[i]);
-    best = wave_max(best);
-    float first = -1e9f;  // minus the lowest index that holds the best score (indices are exact in a float)
-#pragma unroll
-    for (int i = ROUTER_PER_LANE - 1; i >= 0; --i)
-      if (c[i] == best) first = -(float)(lane + 64 * i);
-    const int e = (int)(-wave_max(first));
+    float best;
+    const int e = wave_argmax(c, lane, &best);
     float w = 0.f;
 #pragma unroll
     for (int i = 0; i < ROUTER_PER_LANE; ++i)
@@ -96,32 +167,27 @@ __device__ __forceinline__ void route_token(const float* __restrict__ zr, const 
     for (int i = 0; i < ROUTER_PER_LANE; ++i)
       if (lane == (j & 63) && i == (j >> 6)) mine[i] = w;
   }
-  const float factor = renorm ? mult / (total + 1e-20f) : mult;
+  const float factor = a.renorm ? a.mult / (total + 1e-20f) : a.mult;
 #pragma unroll
   for (int i = 0; i < ROUTER_PER_LANE; ++i)
     if (lane + 64 * i < top) weight[lane + 64 * i] = mine[i] * factor;
 }
 
-__global__ __launch_bounds__(256) void router_choice_kernel(const float* __restrict__ z, int ldz,
-                                                            const float* __restrict__ correction, int n_tokens,
-                                                            int n_out, int top, int* __restrict__ idx,
-                                                            float* __restrict__ weight, int renorm, float mult) {
+__global__ __launch_bounds__(256) void router_choice_kernel(RouteArgs a, int n_tokens, int top, int* __restrict__ idx,
+                                                            float* __restrict__ weight) {
   const int lane = threadIdx.x & 63, t = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (t >= n_tokens) return;  // whole waves leave; no barrier follows
-  route_token(z + (size_t)t * ldz, correction, n_out, top, idx + (size_t)t * top, weight + (size_t)t * top, lane, renorm, mult);
+  route_token(a.z + (size_t)t * a.ldz, a, top, idx + (size_t)t * top, weight + (size_t)t * top, lane);
 }
 
 // For a step of few tokens, where one product gave [router | gate | up] as float rows: a block a
 // token, its first wave chooses the experts, all of it makes act = silu(gate) * up.
 template <typename T>
-__global__ __launch_bounds__(256) void route_and_gate_kernel(const float* __restrict__ zu, int ld,
-                                                             const float* __restrict__ correction, int n_out, int top,
-                                                             int F, int* __restrict__ idx, float* __restrict__ weight,
-                                                             T* __restrict__ act, int ldo, int renorm, float mult) {
-  const int t = blockIdx.x, lane = threadIdx.x & 63;
-  const float* row = zu + (size_t)t * ld;
-  if (threadIdx.x < 64)
-    route_token(row, correction, n_out, top, idx + (size_t)t * top, weight + (size_t)t * top, lane, renorm, mult);
+__global__ __launch_bounds__(256) void route_and_gate_kernel(RouteArgs a, int top, int F, int* __restrict__ idx,
+                                                             float* __restrict__ weight, T* __restrict__ act, int ldo) {
+  const int t = blockIdx.x, lane = threadIdx.x & 63, n_out = a.n_out;
+  const float* row = a.z + (size_t)t * a.ldz;
+  if (threadIdx.x < 64) route_token(row, a, top, idx + (size_t)t * top, weight + (size_t)t * top, lane);
   for (int f = threadIdx.x; f < F; f += 256) act[(size_t)t * ldo + f] = from_f32<T>(silu_f(row[n_out + f]) * row[n_out + F + f]);
 }
 
@@ -166,14 +232,6 @@ __device__ __forceinline__ void lane_dots(const T* const* __restrict__ a, const 
   }
 }
 
-// The router's outputs of every token, for a kernel that chooses the experts itself.
-struct RouteArgs {
-  const float* z;  // [tokens, ldz], or null: idx and weight hold the choice already
-  int ldz;
-  const float* correction;
-  int n_out, renorm;
-  float mult;
-};
 #define ROUTED_MOST 64  // picks a token that a block chooses itself
 
 // Block (token x pick, 16 features): a wave four features at once (eight rows of weights in
@@ -193,7 +251,7 @@ __global__ __launch_bounds__(256) void expert_rows_up_kernel(const T* __restrict
   float wt;
   if constexpr (ROUTED) {
     if (wave == 0)
-      route_token(route.z + (size_t)t * route.ldz, route.correction, route.n_out, top, s_idx, s_weight, lane, route.renorm, route.mult);
+      route_token(route.z + (size_t)t * route.ldz, route, top, s_idx, s_weight, lane);
     __syncthreads();
     const int j = item - t * top;
     if (j == 0 && blockIdx.y == 0 && (int)threadIdx.x < top)
@@ -670,57 +728,42 @@ __global__ __launch_bounds__(256) void expert_combine_kernel(const float* __rest
 
 DEFINE_LAST_ERROR(mlxlm_last_error)
 
-static int router_choice_launch(const float* z, int ldz, const float* correction, int n_tokens, int n_out, int top,
-                                int* idx, float* weight, int renorm, float mult, hipStream_t stream) {
+static int check_route(const char* who, const RouteArgs& a, int top) {
+  if (!a.z || a.n_out <= 0 || top <= 0 || top > a.n_out || a.ldz < a.n_out)
+    FAIL("%s: %d of %d outputs, rows of %d", who, top, a.n_out, a.ldz);
+  if (a.n_out > 64 * ROUTER_PER_LANE) FAIL("%s: %d outputs, at most %d", who, a.n_out, 64 * ROUTER_PER_LANE);
+  if (a.groups > 1 && (a.n_out % a.groups || a.keep <= 0 || a.keep > a.groups || top > a.keep * (a.n_out / a.groups)))
+    FAIL("%s: %d picks of %d of %d groups of %d outputs", who, top, a.keep, a.groups, a.n_out);
+  return 0;
+}
+
+// router_choice: a.z are the tokens' router outputs; idx, weight: [n_tokens, top].
+extern "C" int router_choice(const RouteArgs* args, int n_tokens, int top, int* idx, float* weight, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
-  if (!z || !idx || !weight) FAIL("router_choice: null pointer");
-  if (n_out <= 0 || top <= 0 || top > n_out || ldz < n_out) FAIL("router_choice: %d of %d outputs, rows of %d", top, n_out, ldz);
-  if (n_out > 64 * ROUTER_PER_LANE) FAIL("router_choice: %d outputs, at most %d", n_out, 64 * ROUTER_PER_LANE);
-  hipLaunchKernelGGL(router_choice_kernel, dim3((n_tokens + 3) / 4), dim3(256), 0, stream, z, ldz, correction,
-                     n_tokens, n_out, top, idx, weight, renorm, mult);
+  if (!args || !idx || !weight) FAIL("router_choice: null pointer");
+  if (check_route("router_choice", *args, top)) return 1;
+  hipLaunchKernelGGL(router_choice_kernel, dim3((n_tokens + 3) / 4), dim3(256), 0, stream, *args, n_tokens, top, idx, weight);
   CHECK_LAUNCH("router_choice");
   return 0;
 }
 
-extern "C" int router_choice(const float* z, int ldz, const float* correction, int n_tokens, int n_out, int top,
-                             int* idx, float* weight, hipStream_t stream) {
-  return router_choice_launch(z, ldz, correction, n_tokens, n_out, top, idx, weight, 0, 1.f, stream);
-}
-
-// router_choice_scaled: the picks' weights divided by their sum (+ 1e-20) where `renorm`, then times `mult`.
-extern "C" int router_choice_scaled(const float* z, int ldz, const float* correction, int n_tokens, int n_out, int top,
-                                    int* idx, float* weight, int renorm, float mult, hipStream_t stream) {
-  return router_choice_launch(z, ldz, correction, n_tokens, n_out, top, idx, weight, renorm, mult, stream);
-}
-
-static int route_and_gate_launch(const float* zu, int ld, const float* correction, int n_tokens, int n_out, int top, int F,
-                                 int* idx, float* weight, void* act, int ldo, int dtype, int renorm, float mult,
-                                 hipStream_t stream) {
+// route_and_gate: a.z are rows [router outputs | F gate columns | F up columns].
+extern "C" int route_and_gate(const RouteArgs* args, int n_tokens, int top, int F, int* idx, float* weight, void* act, int ldo,
+                              int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
-  if (!zu || !idx || !weight || !act) FAIL("route_and_gate: null pointer");
-  if (n_out <= 0 || top <= 0 || top > n_out || F <= 0 || ld < n_out + 2 * F || ldo < F)
-    FAIL("route_and_gate: %d of %d outputs and 2 x %d columns in rows of %d", top, n_out, F, ld);
-  if (n_out > 64 * ROUTER_PER_LANE) FAIL("route_and_gate: %d outputs, at most %d", n_out, 64 * ROUTER_PER_LANE);
+  if (!args || !idx || !weight || !act) FAIL("route_and_gate: null pointer");
+  if (check_route("route_and_gate", *args, top)) return 1;
+  if (F <= 0 || args->ldz < args->n_out + 2 * F || ldo < F)
+    FAIL("route_and_gate: %d outputs and 2 x %d columns in rows of %d", args->n_out, F, args->ldz);
   if (dtype != DT_F32 && dtype != DT_BF16) FAIL("route_and_gate: unknown dtype code %d", dtype);
   if (dtype == DT_F32)
-    hipLaunchKernelGGL(route_and_gate_kernel<float>, dim3(n_tokens), dim3(256), 0, stream, zu, ld, correction, n_out, top, F,
-                       idx, weight, (float*)act, ldo, renorm, mult);
+    hipLaunchKernelGGL(route_and_gate_kernel<float>, dim3(n_tokens), dim3(256), 0, stream, *args, top, F, idx, weight,
+                       (float*)act, ldo);
   else
-    hipLaunchKernelGGL(route_and_gate_kernel<bf16>, dim3(n_tokens), dim3(256), 0, stream, zu, ld, correction, n_out, top, F,
-                       idx, weight, (bf16*)act, ldo, renorm, mult);
+    hipLaunchKernelGGL(route_and_gate_kernel<bf16>, dim3(n_tokens), dim3(256), 0, stream, *args, top, F, idx, weight,
+                       (bf16*)act, ldo);
   CHECK_LAUNCH("route_and_gate");
   return 0;
-}
-
-extern "C" int route_and_gate(const float* zu, int ld, const float* correction, int n_tokens, int n_out, int top, int F,
-                              int* idx, float* weight, void* act, int ldo, int dtype, hipStream_t stream) {
-  return route_and_gate_launch(zu, ld, correction, n_tokens, n_out, top, F, idx, weight, act, ldo, dtype, 0, 1.f, stream);
-}
-
-extern "C" int route_and_gate_scaled(const float* zu, int ld, const float* correction, int n_tokens, int n_out, int top,
-                                     int F, int* idx, float* weight, void* act, int ldo, int dtype, int renorm, float mult,
-                                     hipStream_t stream) {
-  return route_and_gate_launch(zu, ld, correction, n_tokens, n_out, top, F, idx, weight, act, ldo, dtype, renorm, mult, stream);
 }
 
 // act_mul: out = act(gate) * up for rows [gate | up]; `activation` 0: silu, 1: the tanh form of gelu.
@@ -771,8 +814,7 @@ extern "C" int expert_rows(const void* x, int ldx, const void* w_gate, const voi
   const ExpertAct fn = {act_kind, act_limit};
   if (route) {
     if (n_experts <= 0 || top > ROUTED_MOST) FAIL("expert_rows: %d picks of %d experts are not chosen here", top, n_experts);
-    if (!route->z || route->n_out <= 0 || top > route->n_out || route->ldz < route->n_out || route->n_out > 64 * ROUTER_PER_LANE)
-      FAIL("expert_rows: %d of %d outputs, rows of %d", top, route->n_out, route->ldz);
+    if (check_route("expert_rows", *route, top)) return 1;
   }
   const NextNorm nn = next ? *next : NextNorm{};
   if (next && (!nn.out || !nn.alpha || !nn.w || !nn.b || !accumulate)) FAIL("expert_rows: the next norm's pointers, or rows that are not complete here");

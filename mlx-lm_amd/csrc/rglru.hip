@@ -1,0 +1,330 @@
+// The real-gated linear recurrent unit with its short convolution, over W channels in B equal parts:
+//   u = conv(x) + bias (per channel, `taps` inputs, zeros before the start)
+//   r = sigmoid(Ra[b] u_b + ra.b),  i = sigmoid(Ri[b] u_b + ri.b)        (a square matrix a part)
+//   log a = -8 r softplus(lam),  a = exp(log a)
+//   S_t = a S_(t-1) + sqrt(1 - a^2) i u,   out = S * gelu_tanh(y)
+// x and y are float columns of a projection's rows.  The convolution's last inputs lie in the request's
+// state row as a ring, position p in row p % taps: a step's rows are none of those it still reads, so
+// blocks that need the same inputs run side by side.
+//
+//   rglru_gates  portions: a block a (64 tokens of a request, part): the convolution into LDS, both gates on
+//                the matrix cores, a and sqrt(1 - a^2) i u as rows, and what the 64 tokens do to the
+//                state (S -> A S + B a channel), each lane's tokens composed, then lanes, then waves
+//   rglru_scan   a thread a channel of 64 tokens: the state ahead of them from the A, B of the request's
+//                earlier ones, then token by token, the output's gate on the way out; the request's
+//                last one leaves the state and the ring
+//   rglru_step   one token a request: a block sixteen channels of a part for up to sixteen requests, all
+//                of the above in one launch
+//
+// All 32-bit but `out` (the gates' products: rows_product.h).
+#include "common.h"
+#include "rows_product.h"
+
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+
+#define SPAN 64
+
+struct RglruArgs {
+  const float* x;  // [rows, ldx]: W columns that the convolution reads
+  const float* y;  // [rows, ldx]: W columns of the output's gate, ahead of its gelu
+  int ldx;
+  const float* conv_w;  // [W][taps]
+  const float* conv_b;  // [W] or null
+  int taps;
+  const void* ra;  // [B][w][wp], columns from w on zero
+  const void* ri;
+  const float* ra_b;  // [W]
+  const float* ri_b;
+  const float* lam;  // [W]
+  float* state;      // a request's row: W floats of S at state_offset, the ring [taps][W] at ring_offset
+  size_t state_stride, state_offset, ring_offset;
+  const int* positions;
+  const int* seq_start;
+  const int* seq_len;
+  const int* slot_ids;
+  const int* span_req;    // portions: [spans]
+  const int* span_start;  // first token, counted from the request's first of this step
+  const int* span_first;  // [requests]
+  float* a;        // [rows, W]
+  float* b;        // [rows, W]
+  float2* does;    // [spans, W]
+  float* s0;       // [requests, W] the state ahead of the step
+  void* out;       // [rows, ldo]
+  int ldo, dtype;  // of the weights and of out
+  int n_requests, n_spans, W, B, w, wp;
+  float decay;  // the 8 of log a
+};
+
+// The convolution's output for channel c of the token at flat row `row`, `local` tokens into its portion.
+__device__ __forceinline__ float conv_at(const RglruArgs& p, const float* ring, int row, int local, int pos, int c) {
+  const float* w = p.conv_w + (size_t)c * p.taps;
+  float acc = 0.f;
+  for (int j = p.taps - 1; j >= 0; --j) {  // the oldest input first
+    float in = 0.f;
+    if (local - j >= 0)
+      in = p.x[(size_t)(row - j) * p.ldx + c];
+    else if (pos - j >= 0)
+      in = ring[(size_t)((pos - j) % p.taps) * p.W + c];
+    acc += w[p.taps - 1 - j] * in;
+  }
+  return acc + (p.conv_b ? p.conv_b[c] : 0.f);
+}
+
+struct Gated {
+  float a, b;
+};
+__device__ __forceinline__ Gated gated(float zr, float zi, float u, float rate) {
+  const float log_a = -rate * sigmoid_f(zr);
+  return Gated{expf(log_a), sqrtf(-expm1f(2.0f * log_a)) * sigmoid_f(zi) * u};
+}
+
+// TT: tokens in LDS at a time (64, or 16 for wide parts); four waves: TT / 16 tiles of rows, the
+// remaining factor over the columns.
+template <typename T, int TT>
+__global__ __launch_bounds__(256) void rglru_gates_kernel(RglruArgs p) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  constexpr int RT = TT / 16, CW = 4 / RT;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lg = lane >> 4;
+  const int rt = wave % RT, cw = wave / RT;
+  const int w = p.w, wp = p.wp, ld = wp + 4;
+  float* U = lds;                            // [TT][ld]
+  float2* does = (float2*)(U + TT * ld);     // [RT][wp16]
+  const int w16 = (w + 15) & ~15;
+  const int span = blockIdx.x, part = blockIdx.y, c0 = part * w;
+  const int r = p.span_req[span], lo = p.span_start[span], n = min(SPAN, p.seq_len[r] - lo);
+  const int row0 = p.seq_start[r] + lo, pos0 = p.positions[row0];
+  const float* srow = p.state + (size_t)p.slot_ids[r] * p.state_stride;
+  const float* ring = srow + p.ring_offset;
+  if (lo == 0)
+    for (int c = tid; c < w; c += 256) p.s0[(size_t)r * p.W + c0 + c] = srow[p.state_offset + c0 + c];
+  const T* Ra = (const T*)p.ra + (size_t)part * w * wp;
+  const T* Ri = (const T*)p.ri + (size_t)part * w * wp;
+  for (int t0 = 0; t0 < n; t0 += TT) {
+    if (t0 > 0) __syncthreads();  // the tile before is done with U
+    for (int e = tid; e < TT * wp; e += 256) {
+      const int t = e / wp, c = e - t * wp;
+      U[t * ld + c] = c < w && t0 + t < n ? conv_at(p, ring, row0 + t0 + t, lo + t0 + t, pos0 + t0 + t, c0 + c) : 0.f;
+    }
+    __syncthreads();
+    const float* urow = U + (16 * rt + lr) * ld;
+    auto row = [&](int k) { return *(const float4*)(urow + k); };
+    for (int ct = 4 * cw; 16 * ct < w; ct += 4 * CW) {  // four tiles of sixteen channels at a time
+      const T* wr[4];
+      const T* wi[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int f = min(16 * (ct + j) + lr, w - 1);
+        wr[j] = Ra + (size_t)f * wp, wi[j] = Ri + (size_t)f * wp;
+      }
+      f32x4_t zr[4], zi[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) zr[j] = zi[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      rows_product<4>(row, wr, wp, 0, 1, zr);
+      rows_product<4>(row, wi, wp, 0, 1, zi);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int cc = 16 * (ct + j) + lr;
+        if (16 * (ct + j) >= w) continue;  // (the same for the whole wave)
+        const bool live = cc < w;
+        const int c = c0 + min(cc, w - 1);
+        const float rb = p.ra_b[c], ib = p.ri_b[c], rate = p.decay * softplus_f(p.lam[c]);
+        float A = 1.f, Bv = 0.f;
+#pragma unroll
+        for (int x = 0; x < 4; ++x) {
+          const int t = 16 * rt + 4 * lg + x;
+          if (t0 + t < n && live) {
+            const Gated g = gated(zr[j][x] + rb, zi[j][x] + ib, U[t * ld + cc], rate);
+            const size_t at = (size_t)(row0 + t0 + t) * p.W + c;
+            p.a[at] = g.a, p.b[at] = g.b;
+            Bv = g.a * Bv + g.b, A *= g.a;
+          }
+        }
+        // lanes of the same channel, sixteen apart, hold four tokens each, in order
+#pragma unroll
+        for (int step = 16; step < 64; step *= 2) {
+          const float A2 = __shfl_xor(A, step, 64), B2 = __shfl_xor(Bv, step, 64);
+          const bool later = lane & step;
+          Bv = later ? A * B2 + Bv : A2 * Bv + B2;
+          A *= A2;
+        }
+        if (lg == 0) {
+          float2* at = does + rt * w16 + cc;
+          if (TT < SPAN && t0 > 0)
+            *at = make_float2(at->x * A, A * at->y + Bv);  // (RT == 1: this tile's tokens follow the last one's)
+          else
+            *at = make_float2(A, Bv);
+        }
+      }
+    }
+  }
+  __syncthreads();
+  for (int c = tid; c < w; c += 256) {
+    float A = 1.f, Bv = 0.f;
+#pragma unroll
+    for (int i = 0; i < RT; ++i) {
+      const float2 d = does[i * w16 + c];
+      Bv = d.x * Bv + d.y, A *= d.x;
+    }
+    p.does[(size_t)span * p.W + c0 + c] = make_float2(A, Bv);
+  }
+}
+
+// Block (span, 256 channels).
+template <typename T>
+__global__ __launch_bounds__(256) void rglru_scan_kernel(RglruArgs p) {
+  const int c = blockIdx.y * 256 + threadIdx.x, span = blockIdx.x;
+  if (c >= p.W) return;  // (no barrier follows)
+  const int r = p.span_req[span], lo = p.span_start[span], len = p.seq_len[r], n = min(SPAN, len - lo);
+  const int row0 = p.seq_start[r] + lo;
+  float S = p.s0[(size_t)r * p.W + c];
+  const int first = p.span_first[r];
+  for (int s = first; s < span; s += 8) {
+    float2 d[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) d[i] = p.does[(size_t)min(s + i, span - 1) * p.W + c];
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+      if (s + i < span) S = d[i].x * S + d[i].y;
+  }
+  for (int t = 0; t < n; t += 16) {
+    float a[16], b[16], y[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const size_t row = (size_t)(row0 + min(t + i, n - 1));
+      a[i] = p.a[row * p.W + c], b[i] = p.b[row * p.W + c], y[i] = p.y[row * p.ldx + c];
+    }
+#pragma unroll
+    for (int i = 0; i < 16; ++i)
+      if (t + i < n) {
+        S = a[i] * S + b[i];
+        ((T*)p.out)[(size_t)(row0 + t + i) * p.ldo + c] = from_f32<T>(S * gelu_tanh(y[i]));
+      }
+  }
+  if (lo + n == len) {  // the request's last tokens of this step
+    float* srow = p.state + (size_t)p.slot_ids[r] * p.state_stride;
+    srow[p.state_offset + c] = S;
+    if (p.taps > 1) {
+      const int start = p.seq_start[r], pos = p.positions[start];
+      for (int t = max(0, len - (p.taps - 1)); t < len; ++t)
+        srow[p.ring_offset + (size_t)((pos + t) % p.taps) * p.W + c] = p.x[(size_t)(start + t) * p.ldx + c];
+    }
+  }
+}
+
+// Block (part x 16 channels, 16 requests of one token each): four waves share K, a thread then a (request, channel).
+template <typename T>
+__global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs p) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ float part[2][4][16][17];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lg = lane >> 4;
+  const int w = p.w, wp = p.wp, ld = wp + 4, tiles = (w + 15) / 16;
+  const int b = blockIdx.x / tiles, f0 = 16 * (blockIdx.x % tiles), c0 = b * w;
+  const int r0 = blockIdx.y * 16, n = min(16, p.n_requests - r0);
+  float* U = lds;  // [16][ld]
+  // what the end of the block reads, asked for first
+  const int er = tid >> 4, ec = f0 + (tid & 15);
+  const bool mine = er < n && ec < w;
+  const int req = r0 + min(er, n - 1), c = c0 + min(ec, w - 1), erow = p.seq_start[req];
+  float* srow = p.state + (size_t)p.slot_ids[req] * p.state_stride;
+  const float S = srow[p.state_offset + c], y = p.y[(size_t)erow * p.ldx + c], x = p.x[(size_t)erow * p.ldx + c];
+  const float rb = p.ra_b[c], ib = p.ri_b[c], lam = p.lam[c];
+  for (int e = tid; e < n * wp; e += 256) {
+    const int t = e / wp, k = e - t * wp, row = p.seq_start[r0 + t];
+    const float* ring = p.state + (size_t)p.slot_ids[r0 + t] * p.state_stride + p.ring_offset;
+    U[t * ld + k] = k < w ? conv_at(p, ring, row, 0, p.positions[row], c0 + k) : 0.f;
+  }
+  for (int e = n * ld + tid; e < 16 * ld; e += 256) U[e] = 0.f;
+  __syncthreads();
+  const float* urow = U + lr * ld;
+  auto row = [&](int k) { return *(const float4*)(urow + k); };
+  const size_t f = (size_t)(b * w + min(f0 + lr, w - 1)) * wp;
+  const T* const gates[2] = {(const T*)p.ra + f, (const T*)p.ri + f};
+  f32x4_t z[2] = {f32x4_t{0.f, 0.f, 0.f, 0.f}, f32x4_t{0.f, 0.f, 0.f, 0.f}};
+  rows_product<2>(row, gates, wp, wave, 4, z);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) part[0][wave][4 * lg + i][lr] = z[0][i], part[1][wave][4 * lg + i][lr] = z[1][i];
+  __syncthreads();
+  if (!mine) return;
+  const int q = tid & 15;
+  const float zr = ((part[0][0][er][q] + part[0][1][er][q]) + (part[0][2][er][q] + part[0][3][er][q])) + rb;
+  const float zi = ((part[1][0][er][q] + part[1][1][er][q]) + (part[1][2][er][q] + part[1][3][er][q])) + ib;
+  const Gated g = gated(zr, zi, U[er * ld + ec], p.decay * softplus_f(lam));
+  const float Sn = g.a * S + g.b;
+  srow[p.state_offset + c] = Sn;
+  if (p.taps > 1) srow[p.ring_offset + (size_t)(p.positions[erow] % p.taps) * p.W + c] = x;
+  ((T*)p.out)[(size_t)erow * p.ldo + c] = from_f32<T>(Sn * gelu_tanh(y));
+}
+
+DEFINE_LAST_ERROR(mlxlm_last_error)
+
+#define LDS_MOST (150 * 1024)
+static size_t gates_lds(int tt, int w, int wp) {
+  return ((size_t)tt * (wp + 4) + 2 * (size_t)(tt / 16) * ((w + 15) / 16 * 16)) * sizeof(float);
+}
+
+// 1 if the kernels take parts of w channels
+extern "C" int rglru_takes(int w) {
+  const int wp = (w + 7) / 8 * 8;
+  return w > 0 && gates_lds(16, w, wp) <= LDS_MOST;
+}
+
+static int check(const RglruArgs& a, const char* who) {
+  if (!a.x || !a.y || !a.conv_w || !a.ra || !a.ri || !a.ra_b || !a.ri_b || !a.lam || !a.state || !a.positions || !a.seq_start ||
+      !a.seq_len || !a.slot_ids || !a.out)
+    FAIL("%s: null pointer", who);
+  if (a.B <= 0 || a.w <= 0 || a.W != a.B * a.w || a.wp % 8 || a.wp < a.w || !rglru_takes(a.w)) FAIL("%s: %d parts of %d channels", who, a.B, a.w);
+  if (a.taps < 1 || a.ldx < a.W || a.ldo < a.W) FAIL("%s: %d taps, rows of %d and %d for %d channels", who, a.taps, a.ldx, a.ldo, a.W);
+  if (a.state_stride < a.state_offset + a.W || (a.taps > 1 && a.state_stride < a.ring_offset + (size_t)a.taps * a.W))
+    FAIL("%s: the state rows are too short", who);
+  if (!(a.decay > 0.f)) FAIL("%s: the decay's constant %g", who, (double)a.decay);
+  if (((uintptr_t)a.ra | (uintptr_t)a.ri) & 15) FAIL("%s: 16-byte aligned weights", who);
+  if (a.dtype != DT_F32 && a.dtype != DT_BF16) FAIL("%s: unknown dtype code %d", who, a.dtype);
+  return 0;
+}
+
+template <typename K>
+static void allow(K kernel) {
+  (void)hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, LDS_MOST);
+}
+
+extern "C" int rglru_step(const RglruArgs* args, hipStream_t stream) {
+  const RglruArgs& a = *args;
+  if (a.n_requests <= 0) return 0;
+  if (check(a, "rglru_step")) return 1;
+  const dim3 grid(a.B * ((a.w + 15) / 16), (a.n_requests + 15) / 16), block(256);
+  const size_t lds = (size_t)16 * (a.wp + 4) * sizeof(float);
+  static bool raised = false;
+  if (!raised) allow(rglru_step_kernel<float>), allow(rglru_step_kernel<bf16>), raised = true;
+  if (a.dtype == DT_F32) hipLaunchKernelGGL(rglru_step_kernel<float>, grid, block, lds, stream, a);
+  else hipLaunchKernelGGL(rglru_step_kernel<bf16>, grid, block, lds, stream, a);
+  CHECK_LAUNCH("rglru_step");
+  return 0;
+}
+
+extern "C" int rglru_portions(const RglruArgs* args, hipStream_t stream) {
+  const RglruArgs& a = *args;
+  if (a.n_requests <= 0 || a.n_spans <= 0) return 0;
+  if (check(a, "rglru_portions")) return 1;
+  if (!a.span_req || !a.span_start || !a.span_first || !a.a || !a.b || !a.does || !a.s0) FAIL("rglru_portions: null pointer");
+  static bool raised = false;
+  if (!raised) {
+    allow(rglru_gates_kernel<float, 64>), allow(rglru_gates_kernel<float, 16>);
+    allow(rglru_gates_kernel<bf16, 64>), allow(rglru_gates_kernel<bf16, 16>);
+    raised = true;
+  }
+  const bool wide = gates_lds(64, a.w, a.wp) > 80 * 1024;  // (two blocks a CU)
+  const dim3 grid(a.n_spans, a.B), scan(a.n_spans, (a.W + 255) / 256), block(256);
+  const size_t lds = gates_lds(wide ? 16 : 64, a.w, a.wp);
+  if (a.dtype == DT_F32) {
+    if (wide) hipLaunchKernelGGL((rglru_gates_kernel<float, 16>), grid, block, lds, stream, a);
+    else hipLaunchKernelGGL((rglru_gates_kernel<float, 64>), grid, block, lds, stream, a);
+    hipLaunchKernelGGL(rglru_scan_kernel<float>, scan, block, 0, stream, a);
+  } else {
+    if (wide) hipLaunchKernelGGL((rglru_gates_kernel<bf16, 16>), grid, block, lds, stream, a);
+    else hipLaunchKernelGGL((rglru_gates_kernel<bf16, 64>), grid, block, lds, stream, a);
+    hipLaunchKernelGGL(rglru_scan_kernel<bf16>, scan, block, 0, stream, a);
+  }
+  CHECK_LAUNCH("rglru_portions");
+  return 0;
+}

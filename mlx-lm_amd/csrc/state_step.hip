@@ -9,6 +9,9 @@
 //                   inputs lie in the request's row as a ring, position p in row p % taps: the one
 //                   that is written is none of those that are read, so the heads that share a key
 //                   head read it side by side.
+//   STEP_CHANNEL_RAW  as STEP_DELTA_RAW with a decay per key channel and an output gate through narrow
+//                   middles: g[n] = exp(-exp(A_log) softplus(A2 z + dt_bias)), gate = G2 y, with z and y
+//                   columns of the projection.
 //   STEP_BONUS      a decay per key channel and a bonus for the current token
 //                     o = S^T r + (r . (u * k)) v;  S <- diag(w) S + k v^T
 //                   with w = exp(-exp(w0 + W2 tanh(z))) made here from the low-rank middle z.
@@ -16,8 +19,8 @@
 // A block a (head, request); S [N][P] lies in the threads' registers, asked for at once and written
 // back once (a thread holds every TY-th row of V neighbouring columns), so a step is one trip to
 // memory each way.  A token needs one joint reduction over the keys (S^T k and S^T q together: o =
-// g S^T q + (q . k) u).  The heads' output is divided by its root mean square (norm weight, silu
-// gate) on the way out.
+// g S^T q + (q . k) u).  The heads' output is divided by its root mean square (norm weight, a silu or
+// sigmoid gate) on the way out.
 //
 //   lowrank_decay   log w = -exp(w0 + W2 tanh(z)) as rows, for the kernels that take chunks of tokens.
 //
@@ -30,7 +33,7 @@ __device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + lo
 
 #define UNIT_EPS 1e-6f  // a unit vector is x / sqrt(sum(x^2) + UNIT_EPS)
 
-enum { STEP_DELTA = 0, STEP_DELTA_RAW = 1, STEP_BONUS = 2 };
+enum { STEP_DELTA = 0, STEP_DELTA_RAW = 1, STEP_BONUS = 2, STEP_CHANNEL_RAW = 3 };
 
 struct StepArgs {
   const float* q;  // key head hk at column hk * qk_stride, value head h at column h * v_stride
@@ -67,6 +70,12 @@ struct StepArgs {
   const void* w2t;   // [rank][H N]
   const float* w0;   // [H N]
   const float* bonus;  // [H N]
+  int gate_sigmoid;    // the gate passes a sigmoid instead of a silu
+  // STEP_CHANNEL_RAW: z and rank as above (rank a multiple of 8), dt_bias [H N]
+  const void* a2;  // [H N][rank]
+  const float* y;  // [tokens, g_rank] (gate is not read then), or null: no gate, or `gate`
+  int ldy, g_rank;
+  const void* g2;  // [H P][g_rank]
 };
 
 struct Sums3 {
@@ -113,6 +122,46 @@ __device__ __forceinline__ float lowrank_logit(const void* w2t, int dtype, const
   return z;
 }
 
+// One row of a narrow matrix with a middle in LDS, by sixteen neighbouring lanes; in all of them.
+__device__ __forceinline__ float lowrank_row(const bf16* __restrict__ w, const float* m, int rank, int l16) {
+  float s = 0.f;
+  for (int k = 8 * l16; k < rank; k += 128) {
+    const u32x4_t v = *(const u32x4_t*)(w + k);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      s += __uint_as_float(v[i] << 16) * m[k + 2 * i];
+      s += __uint_as_float(v[i] & 0xffff0000u) * m[k + 2 * i + 1];
+    }
+  }
+  return group_sum<16>(s);
+}
+__device__ __forceinline__ float lowrank_row(const float* __restrict__ w, const float* m, int rank, int l16) {
+  float s = 0.f;
+  for (int k = 4 * l16; k < rank; k += 64) {
+    const f32x4_t v = *(const f32x4_t*)(w + k);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) s += v[i] * m[k + i];
+  }
+  return group_sum<16>(s);
+}
+// The decays' logits into ds and the gate's into gs, for head h.
+template <typename T, int TH>
+__device__ __forceinline__ void lowrank_rows(const StepArgs& a, int h, const float* tz, const float* ty, float* ds, float* gs) {
+  const int l16 = threadIdx.x & 15, total = a.N + (a.y ? a.P : 0);
+  const T* a2 = (const T*)a.a2 + (size_t)h * a.N * a.rank;
+  const T* g2 = (const T*)a.g2 + (size_t)h * a.P * a.g_rank;
+#pragma unroll 4
+  for (int c = threadIdx.x / 16; c < total; c += TH / 16) {
+    if (c < a.N) {
+      const float s = lowrank_row(a2 + (size_t)c * a.rank, tz, a.rank, l16);
+      if (l16 == 0) ds[c] = s;
+    } else {
+      const float s = lowrank_row(g2 + (size_t)(c - a.N) * a.g_rank, ty, a.g_rank, l16);
+      if (l16 == 0) gs[c - a.N] = s;
+    }
+  }
+}
+
 // V columns a thread, R rows of the state a thread, TH threads
 template <int MODE, int V, int R, int TH, typename T>
 __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
@@ -129,6 +178,8 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
   float* ks = qs + N;                           // [N]
   float* ds = ks + N;                           // [N] the decays (STEP_BONUS)
   float* tz = ds + N;                           // [rank]
+  float* gs = tz + a.rank;                      // [P] the gate's logits (STEP_CHANNEL_RAW)
+  float* my = gs + P;                           // [g_rank]
   const int start = a.seq_start[rq], n = a.seq_len[rq];
   float* row_state = a.state + (size_t)a.slot_ids[rq] * a.state_stride;
   float* Sg = row_state + a.state_offset + (size_t)h * N * P;
@@ -138,11 +189,16 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
 
   for (int t = 0; t < n; ++t) {
     const size_t row = (size_t)(start + t);
-    const float gv = a.gate && tid < P ? a.gate[row * a.ldg + (size_t)h * P + tid] : 0.f;
+    float gv = a.gate && tid < P ? a.gate[row * a.ldg + (size_t)h * P + tid] : 0.f;
     const float nw = tid < P ? a.norm_w[(size_t)h * a.norm_stride + tid] : 0.f;
     float g = 1.f, beta = 0.f;
     if (t > 0) __syncthreads();  // the token before is done with the arrays
-    if constexpr (MODE == STEP_DELTA_RAW) {
+    if constexpr (MODE == STEP_DELTA_RAW || MODE == STEP_CHANNEL_RAW) {
+      if constexpr (MODE == STEP_CHANNEL_RAW) {
+        for (int i = tid; i < a.rank; i += TH) tz[i] = a.z[row * a.ldz + i];
+        if (a.y)
+          for (int i = tid; i < a.g_rank; i += TH) my[i] = a.y[row * a.ldy + i];
+      }
       const int C = 2 * a.Hk * N + a.H * P, pos = a.positions[row];
       float* ring = row_state + a.ring_offset;
       const bool keeps_keys = h % group == 0;
@@ -162,7 +218,17 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
         (kind == 0 ? qs : kind == 1 ? ks : vs)[i] = silu_f(acc);
       }
       beta = sigmoid_f(a.beta[row * a.ld_gb + h]);
-      g = expf(-expf(a.A_log[h]) * softplus_f(a.log_g[row * a.ld_gb + h] + a.dt_bias[h]));
+      if constexpr (MODE == STEP_DELTA_RAW) {
+        g = expf(-expf(a.A_log[h]) * softplus_f(a.log_g[row * a.ld_gb + h] + a.dt_bias[h]));
+      } else {
+        __syncthreads();
+        if (a.w2_dtype == DT_BF16) lowrank_rows<bf16, TH>(a, h, tz, my, ds, gs);
+        else lowrank_rows<float, TH>(a, h, tz, my, ds, gs);
+        __syncthreads();
+        const float rate = expf(a.A_log[h]);
+        for (int i = tid; i < N; i += TH) ds[i] = expf(-rate * softplus_f(ds[i] + a.dt_bias[(size_t)h * N + i]));
+        if (a.y && tid < P) gv = gs[tid];
+      }
     } else {
       for (int i = tid; i < N; i += TH) {
         qs[i] = a.q[row * a.ldq + (size_t)hk * a.qk_stride + i];
@@ -185,7 +251,7 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
     Sums3 s = {0.f, 0.f, 0.f};
     for (int i = tid; i < N; i += TH) {
       const float q = qs[i], k = ks[i];
-      if constexpr (MODE == STEP_DELTA_RAW) s.a += q * q, s.b += k * k;
+      if constexpr (MODE == STEP_DELTA_RAW || MODE == STEP_CHANNEL_RAW) s.a += q * q, s.b += k * k;
       s.c += MODE == STEP_BONUS ? q * k * a.bonus[(size_t)h * N + i] : q * k;
     }
     float qf = 1.f, kf = 1.f;  // what queries and keys are still to be multiplied by
@@ -201,7 +267,7 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
             pq.v += qs[i] * S[r].v;
             S[r].v = ds[i] * S[r].v + ks[i] * vc.v;
           } else {
-            S[r].v *= g;
+            S[r].v *= MODE == STEP_CHANNEL_RAW ? ds[i] : g;
             pq.v += qs[i] * S[r].v;
             pk.v += ks[i] * S[r].v;
           }
@@ -212,7 +278,7 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
     }
     s = block_sums(s, red);  // (its barriers also stand between the partial sums and their readers)
     float dot = s.c;
-    if constexpr (MODE == STEP_DELTA_RAW) {
+    if constexpr (MODE == STEP_DELTA_RAW || MODE == STEP_CHANNEL_RAW) {
       qf = a.q_scale / sqrtf(s.a + UNIT_EPS), kf = 1.0f / sqrtf(s.b + UNIT_EPS);
       dot *= qf * kf;
     }
@@ -245,7 +311,7 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
     const float ss = block_sum(tid < P ? o * o : 0.f, red);
     if (tid < P) {
       o *= nw / sqrtf(ss / (float)P + a.eps);
-      if (a.gate) o *= silu_f(gv);
+      if (a.gate || (MODE == STEP_CHANNEL_RAW && a.y)) o *= a.gate_sigmoid ? sigmoid_f(gv) : silu_f(gv);
       ((T*)a.out)[row * a.ldo + (size_t)h * P + tid] = from_f32<T>(o);
     }
   }
@@ -343,9 +409,16 @@ extern "C" int state_step(const StepArgs* args, hipStream_t stream) {
   if (s.V == 4 && (a.state_stride % 4 || a.state_offset % 4 || ((uintptr_t)a.state & 15))) FAIL("state_step: the states must be 16-byte aligned");
   if (a.out_dtype != DT_F32 && a.out_dtype != DT_BF16) FAIL("state_step: unknown dtype code %d", a.out_dtype);
   int rank = 0;
-  if (a.mode == STEP_DELTA || a.mode == STEP_DELTA_RAW) {
-    if (!a.log_g || !a.beta || a.ld_gb < a.H) FAIL("state_step: a decay and a step size for every head");
-    if (a.mode == STEP_DELTA_RAW) {
+  if (a.mode == STEP_DELTA || a.mode == STEP_DELTA_RAW || a.mode == STEP_CHANNEL_RAW) {
+    if ((!a.log_g && a.mode != STEP_CHANNEL_RAW) || !a.beta || a.ld_gb < a.H) FAIL("state_step: a decay and a step size for every head");
+    if (a.mode == STEP_CHANNEL_RAW) {
+      if (!a.z || !a.a2 || a.rank <= 0 || a.rank % 8 || a.ldz < a.rank || a.rank > 2048) FAIL("state_step: decays per key channel from a middle of %d columns (a multiple of 8, at most 2048)", a.rank);
+      if (a.y && (!a.g2 || a.g_rank <= 0 || a.g_rank % 8 || a.ldy < a.g_rank || a.g_rank > 2048)) FAIL("state_step: a gate from a middle of %d columns (a multiple of 8, at most 2048)", a.g_rank);
+      if (((uintptr_t)a.a2 | (a.y ? (uintptr_t)a.g2 : 0)) & 15) FAIL("state_step: 16-byte aligned matrices");
+      if (a.w2_dtype != DT_F32 && a.w2_dtype != DT_BF16) FAIL("state_step: unknown dtype code %d", a.w2_dtype);
+      rank = a.rank + a.P + (a.y ? a.g_rank : 0);
+    }
+    if (a.mode != STEP_DELTA) {
       if (!a.A_log || !a.dt_bias || !a.conv_w || !a.positions || a.taps < 1) FAIL("state_step: null pointer, or %d taps", a.taps);
       if (a.qk_stride != a.N || a.v_stride != a.P) FAIL("state_step: the projection's heads lie side by side");
       if (a.taps > 1 && a.state_stride < a.ring_offset + (size_t)a.taps * (2 * a.Hk * a.N + a.H * a.P))
@@ -367,6 +440,9 @@ extern "C" int state_step(const StepArgs* args, hipStream_t stream) {
   if (a.mode == STEP_DELTA) {
     if (f32) launch_step<STEP_DELTA, float>(a, s, lds, stream);
     else launch_step<STEP_DELTA, bf16>(a, s, lds, stream);
+  } else if (a.mode == STEP_CHANNEL_RAW) {
+    if (f32) launch_step<STEP_CHANNEL_RAW, float>(a, s, lds, stream);
+    else launch_step<STEP_CHANNEL_RAW, bf16>(a, s, lds, stream);
   } else if (a.mode == STEP_DELTA_RAW) {
     if (f32) launch_step<STEP_DELTA_RAW, float>(a, s, lds, stream);
     else launch_step<STEP_DELTA_RAW, bf16>(a, s, lds, stream);

@@ -66,7 +66,7 @@ def build_parser():
     p.add_argument("--num-pages", type=int, default=None,
                    help="pages of the pool (default: what --max-tokens needs)")
     p.add_argument("--page-stats", action="store_true", help="print every step's page statistics")
-    p.add_argument("--max-requests", type=int, default=8, help="most requests live at a time")
+    p.add_argument("--max-requests", type=int, default=4, help="most requests live at a time")
     return p
 
 

@@ -650,7 +650,7 @@ class AttnTerms(ctypes.Structure):
     """Mirror of ``AttnTerms`` in csrc/attention_tiles.h."""
 
     _fields_ = [("head_scale", _vp), ("slopes", _vp), ("gate", _vp), ("ldg", _c_int), ("keep_first", _c_int),
-                ("softcap", _c_float), ("dist_bias", _vp), ("n_dist", _c_int)]
+                ("softcap", _c_float), ("dist_bias", _vp), ("n_dist", _c_int), ("sinks", _vp), ("head_gate", _vp), ("ldhg", _c_int)]
 
 
 class ScoreTerms:
@@ -661,9 +661,13 @@ class ScoreTerms:
     ``keep_first`` (with a window, the first so many keys stay visible), ``softcap`` (a scaled
     score ``s`` becomes ``softcap * tanh(s / softcap)``) and ``distance_bias`` (float32 ``[n_heads,
     n]``: entry ``min(distance, n - 1)`` of the head's row is added to a score).  A score takes
-    them in this order: scale, cap, slope, table."""
+    them in this order: scale, cap, slope, table.  ``sinks`` (float32 ``[n_heads]``): the softmax's
+    denominator holds ``exp(sinks[h])`` too, which brings no value.  ``head_gate`` (float32 rows of at least
+    ``n_heads`` columns): head ``h``'s output is multiplied by the sigmoid of its column."""
 
-    def __init__(self, head_scale=None, slopes=None, gate=None, keep_first=0, softcap=0.0, distance_bias=None):
+    def __init__(self, head_scale=None, slopes=None, gate=None, keep_first=0, softcap=0.0, distance_bias=None, sinks=None,
+                 head_gate=None):
+        self.sinks, self.head_gate = sinks, head_gate
         self.head_scale, self.slopes, self.gate, self.keep_first = head_scale, slopes, gate, int(keep_first)
         self.softcap, self.distance_bias = float(softcap), distance_bias
 
@@ -679,6 +683,14 @@ class ScoreTerms:
             _need(self.distance_bias.dim() == 2 and self.distance_bias.shape[0] == n_heads and self.distance_bias.is_contiguous(),
                   "distance_bias: a contiguous row a head")
             t.dist_bias, t.n_dist = _ptr(self.distance_bias), self.distance_bias.shape[1]
+        if self.sinks is not None:
+            _dev(self.sinks, "sinks", torch.float32)
+            _need(self.sinks.numel() == n_heads, "sinks: one value a head")
+            t.sinks = _ptr(self.sinks)
+        if self.head_gate is not None:
+            t.ldhg = _f32_rows(self.head_gate, "head_gate", n_heads)
+            _need(self.head_gate.shape[0] >= q.shape[0], "head_gate: fewer rows than queries")
+            t.head_gate = _ptr(self.head_gate)
         return t
 
     def args(self, q, n_heads):
@@ -856,10 +868,11 @@ def attn_decode(out, q, kv, block_table, token_req, positions, rows, n_rows, n_h
 
 
 def attn_decode_group(out, q, kv, block_table, token_req, positions, rows, n_rows, n_heads, scale, window=0, n_splits=1,
-                      part_o=None, part_ml=None, rows_are_requests=False):
+                      part_o=None, part_ml=None, rows_are_requests=False, terms=None):
     """``attn_row`` for bfloat16 caches with head_dim 64, 128 or 256 where many query heads share a key
     head: a block takes sixteen query heads of a key head at once, on the matrix cores, so a key is
-    read once for all of them.  ``n_splits`` parts of a row's keys, joined by a second kernel."""
+    read once for all of them.  ``n_splits`` parts of a row's keys, joined by a second kernel.  Of the
+    ``terms`` only sinks and the heads' gate."""
     lib = build.load("attention_decode")
     ldq, ldo = _rows2d(q, "q"), _rows2d(out, "out")
     _need(q.dtype == torch.bfloat16 and out.dtype == q.dtype, "attn_decode_group: bfloat16 only")
@@ -878,7 +891,7 @@ def attn_decode_group(out, q, kv, block_table, token_req, positions, rows, n_row
         _ptr(out), _ptr(q), _c_int(ldq), _c_int(ldo), _ptr(kv.k), _ptr(kv.v), _c_size_t(kv.page_stride), _ptr(block_table),
         _c_int(block_table.shape[1]), _ptr(token_req), _ptr(positions), _ptr(rows), _c_int(n_rows), _c_int(n_heads),
         _c_int(kv.n_kv_heads), _c_int(kv.head_dim), _c_int(kv.page_size), _c_int(window), _c_float(scale), _c_int(n_splits),
-        _ptr(part_o), _ptr(part_ml), _c_int(1 if rows_are_requests else 0), _stream())
+        _ptr(part_o), _ptr(part_ml), _c_int(1 if rows_are_requests else 0), *_terms(terms, q, n_heads), _stream())
     build.check(lib, rc, "attn_decode_group")
     return out
 
@@ -1374,40 +1387,69 @@ def gated_group_rmsnorm(out, y, z, weight, groups, eps):
 # experts chosen per token (csrc/experts.hip)
 
 
-def router_choice(idx, weight, z, correction, top, renormalize=False, weight_scale=1.0):
-    """From float32 router outputs ``z`` ``[tokens, outputs]``: softmax, the ``top`` largest of
-    softmax + ``correction`` into ``idx`` (int32 ``[tokens, top]``), their softmax values into
-    ``weight``; with ``renormalize`` divided by their sum (+ 1e-20); times ``weight_scale``."""
-    lib = build.load("experts")
-    ldz = _f32_rows(z, "z", 1)
-    T, n_out = z.shape
+class RouteArgs(ctypes.Structure):
+    """Mirror of ``RouteArgs`` in csrc/experts.hip."""
+
+    _fields_ = [("z", _vp), ("ldz", _c_int), ("correction", _vp), ("n_out", _c_int), ("renorm", _c_int), ("mult", _c_float),
+                ("sigmoid", _c_int), ("groups", _c_int), ("keep", _c_int)]
+
+
+ROUTER_SCORES = ("softmax", "sigmoid")
+
+
+class Route:
+    """How experts are chosen from router outputs: a score is the ``softmax`` over all outputs or the
+    ``sigmoid`` of each; the ``top`` largest of score + ``correction`` (float32 ``[outputs]`` or None) are
+    chosen, with ``groups = (count, keep)`` only out of the ``keep`` best of ``count`` equal groups of
+    neighbours (a group counts the sum of its two largest choice scores); a pick's weight is its score,
+    with ``renormalize`` divided by the picks' sum (+ 1e-20), times ``weight_scale``."""
+
+    def __init__(self, correction=None, renormalize=False, weight_scale=1.0, scores="softmax", groups=None):
+        _need(scores in ROUTER_SCORES, f"router scores {scores!r} (known: {ROUTER_SCORES})")
+        self.correction, self.renormalize, self.weight_scale, self.scores = correction, bool(renormalize), float(weight_scale), scores
+        self.groups = tuple(int(n) for n in groups) if groups is not None else (1, 1)
+
+    def struct(self, z, n_out, n_tokens):
+        a = RouteArgs()
+        a.ldz, a.z, a.n_out = _f32_rows(z, "z", n_out), z.data_ptr(), int(n_out)
+        _need(z.shape[0] >= n_tokens, "router: fewer rows of outputs than tokens")
+        if self.correction is not None:
+            _dev(self.correction, "correction", torch.float32)
+            _need(self.correction.numel() == n_out, "router: correction length")
+            a.correction = self.correction.data_ptr()
+        a.renorm, a.mult, a.sigmoid = int(self.renormalize), self.weight_scale, int(self.scores == "sigmoid")
+        a.groups, a.keep = self.groups
+        return a
+
+
+def _picks(idx, weight, T, top):
     _dev(idx, "idx", torch.int32)
     _dev(weight, "weight", torch.float32)
-    _need(idx.numel() >= T * top and weight.numel() >= T * top, "router_choice: idx / weight too short")
-    if correction is not None:
-        _dev(correction, "correction", torch.float32)
-        _need(correction.numel() == n_out, "router_choice: correction length")
-    rc = lib.router_choice_scaled(_ptr(z), _c_int(ldz), _ptr(correction), _c_int(T), _c_int(n_out), _c_int(top), _ptr(idx),
-                                  _ptr(weight), _c_int(int(bool(renormalize))), _c_float(weight_scale), _stream())
+    _need(idx.numel() >= T * top and weight.numel() >= T * top, "router: idx / weight too short")
+
+
+def router_choice(idx, weight, z, correction, top, renormalize=False, weight_scale=1.0, scores="softmax", groups=None):
+    """From float32 router outputs ``z`` ``[tokens, outputs]`` every token's experts into ``idx`` (int32
+    ``[tokens, top]``) and their weights into ``weight`` (``Route``)."""
+    lib = build.load("experts")
+    T, n_out = z.shape
+    _picks(idx, weight, T, top)
+    a = Route(correction, renormalize, weight_scale, scores, groups).struct(z, n_out, T)
+    rc = lib.router_choice(ctypes.byref(a), _c_int(T), _c_int(top), _ptr(idx), _ptr(weight), _stream())
     build.check(lib, rc, "router_choice")
 
 
-def route_and_gate(idx, weight, act, zu, correction, top, n_out, renormalize=False, weight_scale=1.0):
+def route_and_gate(idx, weight, act, zu, correction, top, n_out, renormalize=False, weight_scale=1.0, scores="softmax", groups=None):
     """``router_choice`` on the first ``n_out`` columns of the float32 rows ``zu`` and ``silu_mul`` on
     the ``2 * act.shape[1]`` columns behind them, in one launch (for steps of few tokens)."""
     lib = build.load("experts")
-    ld, ldo = _f32_rows(zu, "zu", 1), _rows2d(act, "act")
+    ldo = _rows2d(act, "act")
     T, F = act.shape
     _need(zu.shape[0] >= T and zu.shape[1] == n_out + 2 * F and act.dtype in DT, "route_and_gate: shapes")
-    _dev(idx, "idx", torch.int32)
-    _dev(weight, "weight", torch.float32)
-    _need(idx.numel() >= T * top and weight.numel() >= T * top, "route_and_gate: idx / weight too short")
-    if correction is not None:
-        _dev(correction, "correction", torch.float32)
-        _need(correction.numel() == n_out, "route_and_gate: correction length")
-    rc = lib.route_and_gate_scaled(_ptr(zu), _c_int(ld), _ptr(correction), _c_int(T), _c_int(n_out), _c_int(top), _c_int(F),
-                                   _ptr(idx), _ptr(weight), _ptr(act), _c_int(ldo), _c_int(DT[act.dtype]),
-                                   _c_int(int(bool(renormalize))), _c_float(weight_scale), _stream())
+    _picks(idx, weight, T, top)
+    a = Route(correction, renormalize, weight_scale, scores, groups).struct(zu, n_out, T)
+    rc = lib.route_and_gate(ctypes.byref(a), _c_int(T), _c_int(top), _c_int(F), _ptr(idx), _ptr(weight), _ptr(act), _c_int(ldo),
+                            _c_int(DT[act.dtype]), _stream())
     build.check(lib, rc, "route_and_gate")
 
 
@@ -1436,12 +1478,6 @@ def _expert_activation(activation, limit):
     return _c_int(EXPERT_ACTIVATIONS[activation]), _c_float(limit)
 
 
-class RouteArgs(ctypes.Structure):
-    """Mirror of ``RouteArgs`` in csrc/experts.hip."""
-
-    _fields_ = [("z", _vp), ("ldz", _c_int), ("correction", _vp), ("n_out", _c_int), ("renorm", _c_int), ("mult", _c_float)]
-
-
 class NextNorm(ctypes.Structure):
     """Mirror of ``NextNorm`` in csrc/experts.hip."""
 
@@ -1465,8 +1501,8 @@ def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=Tr
     weights (``w_gate``, ``w_up``: ``[experts, F, width]``, ``w_down``: ``[experts, width, F]``); a
     pick at or beyond the number of experts gives ``weight * x``.  ``act``: room for ``[tokens *
     top, F]`` of ``x``'s dtype.  ``activation``: ``silu(g) * u``, or ``clamped``: ``g sigmoid(1.702 g) (u
-    + 1)`` with ``g`` at most ``limit`` and ``u`` within ``[-limit, limit]``.  ``route = (z, correction,
-    renormalize, weight_scale)``: the choice is made here (``router_choice``), into ``idx`` and ``weight``.
+    + 1)`` with ``g`` at most ``limit`` and ``u`` within ``[-limit, limit]``.  ``route = (z, Route)``:
+    the choice is made here (``router_choice``), into ``idx`` and ``weight``.
     ``after = (out, norm)``: the rows that this completes (``accumulate``) pass ``dynamic_tanh`` with
     ``norm`` into ``out`` (``x``'s dtype) too."""
     lib = build.load("experts")
@@ -1487,15 +1523,7 @@ def expert_rows(y, x, w_gate, w_up, w_down, idx, weight, top, act, accumulate=Tr
     _need(idx.numel() >= T * top and weight.numel() >= T * top, "expert_rows: idx / weight too short")
     rt, nn = None, None
     if route is not None:
-        z, correction, renormalize, weight_scale = route
-        rt = RouteArgs()
-        rt.ldz, rt.z, rt.n_out = _f32_rows(z, "z", 1), z.data_ptr(), z.shape[1]
-        _need(z.shape[0] >= T, "expert_rows: fewer rows of router outputs than tokens")
-        if correction is not None:
-            _dev(correction, "correction", torch.float32)
-            _need(correction.numel() == z.shape[1], "expert_rows: correction length")
-            rt.correction = correction.data_ptr()
-        rt.renorm, rt.mult = int(bool(renormalize)), float(weight_scale)
+        rt = route[1].struct(route[0], route[0].shape[1], T)
     if after is not None:
         nn = _next_norm(after, x, accumulate)
     rc = lib.expert_rows(_ptr(x), _c_int(ldx), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _ptr(idx), _ptr(weight),
@@ -1758,22 +1786,38 @@ class StepArgs(ctypes.Structure):
                 ("H", _c_int), ("Hk", _c_int), ("N", _c_int), ("P", _c_int), ("mode", _c_int), ("log_g", _vp), ("beta", _vp),
                 ("ld_gb", _c_int), ("A_log", _vp), ("dt_bias", _vp), ("conv_w", _vp), ("taps", _c_int), ("ring_offset", _c_size_t),
                 ("positions", _vp), ("q_scale", _c_float), ("z", _vp), ("ldz", _c_int), ("rank", _c_int), ("w2_dtype", _c_int),
-                ("w2t", _vp), ("w0", _vp), ("bonus", _vp)]
+                ("w2t", _vp), ("w0", _vp), ("bonus", _vp), ("gate_sigmoid", _c_int), ("a2", _vp), ("y", _vp), ("ldy", _c_int), ("g_rank", _c_int),
+                ("g2", _vp)]
 
 
-STEP_DELTA, STEP_DELTA_RAW, STEP_BONUS = 0, 1, 2
+STEP_DELTA, STEP_DELTA_RAW, STEP_BONUS, STEP_CHANNEL_RAW = 0, 1, 2, 3
 
 
 class DeltaRaw:
     """What ``state_step`` needs to make the delta rule's operands from the projection's own columns:
     the convolution's weights (float32 ``[channels, taps]``, channels of queries, keys and values in
     this order), where its ring of inputs starts in a request's state row (``[taps, channels]``,
-    position ``p`` in row ``p % taps``), ``A_log`` and ``dt_bias`` a head, the queries' factor."""
+    position ``p`` in row ``p % taps``), ``A_log`` a head and ``dt_bias`` a head (or a key channel of every
+    head), the queries' factor."""
 
     def __init__(self, conv_w, ring_offset, a_log, dt_bias, q_scale):
         for name, t in (("conv_w", conv_w), ("a_log", a_log), ("dt_bias", dt_bias)):
             _dev(t, name, torch.float32)
         self.conv_w, self.ring_offset, self.a_log, self.dt_bias, self.q_scale = conv_w, int(ring_offset), a_log, dt_bias, float(q_scale)
+
+
+class NarrowMiddle:
+    """Gates of a recurrence through narrow middles, ``logits = W2 m`` with the middle ``m`` in columns of a
+    projection's float32 rows: ``a2`` ``[heads * key_dim, rank]`` for a decay per key channel, ``g2`` ``[heads
+    * value_dim, rank]`` for an output gate.  Ranks are multiples of 8 (zero columns beyond the middle's
+    own), the middles start at multiples of 4 columns (``a_col``, ``g_col``)."""
+
+    def __init__(self, a2, a_col, g2, g_col):
+        for name, t in (("a2", a2), ("g2", g2)):
+            _dev(t, name)
+            _need(t.dtype in DT and t.dim() == 2 and t.is_contiguous() and t.shape[1] % 8 == 0, f"{name}: rows of a multiple of 8 columns")
+        _need(a2.dtype == g2.dtype and a_col % 4 == 0 and g_col % 4 == 0, "a2 and g2 share a dtype, their middles start at multiples of 4")
+        self.a2, self.a_col, self.g2, self.g_col = a2, int(a_col), g2, int(g_col)
 
 
 class LowRankDecay:
@@ -1806,16 +1850,18 @@ def state_step_takes(key_dim, value_dim):
 
 def state_step(out, q, k, v, state, state_offset, seq_start, seq_len, slot_ids, n_requests, n_heads, n_key_heads, key_dim,
                value_dim, norm_weight, eps, gate=None, qk_stride=None, v_stride=None, log_g=None, beta=None, raw=None,
-               positions=None, z=None, decay=None, bonus=None):
+               positions=None, z=None, decay=None, bonus=None, narrow=None, gate_activation="silu"):
     """A recurrence over a matrix state token by token, a block a (head, request), the state in
     registers; the heads' output divided by its root mean square, times ``norm_weight`` (``value_dim``
-    values, or that many a head) and ``silu(gate)``.
+    values, or that many a head) and ``silu(gate)`` (``gate_activation``: or ``sigmoid``).
 
     * the gated delta rule ``u = beta (v - g S^T k); S <- g S + k u^T; o = S^T q`` on prepared
       rows: ``log_g``, ``beta`` float32 ``[rows, n_heads]``;
     * with ``raw`` (a ``DeltaRaw``; every request brings one token) the same from the projection's
       columns, ``beta`` and ``log_g`` the columns that become them (convolution, silu, unit vectors,
       ``beta = sigmoid(.)``, ``g = exp(-exp(A_log) softplus(. + dt_bias))``);
+    * with ``raw`` and ``narrow = (u, NarrowMiddle)`` the same with a decay per key channel, ``g[n] =
+      exp(-exp(A_log) softplus(a2 m + dt_bias))``, and the gate's logits from their middle, both columns of ``u``;
     * with ``decay`` (a ``LowRankDecay`` over ``z``, float32 ``[rows, >= rank]``) and ``bonus``: ``o =
       (S + diag(bonus) k v^T)^T q; S <- diag(w) S + k v^T``.
 
@@ -1853,17 +1899,30 @@ def state_step(out, q, k, v, state, state_offset, seq_start, seq_len, slot_ids, 
         _need(bonus.numel() == n_heads * key_dim and z.shape[0] >= T, "state_step: a bonus for every key channel")
         a.bonus = bonus.data_ptr()
     else:
-        ld = _f32_rows(log_g, "log_g", n_heads)
-        _need(_f32_rows(beta, "beta", n_heads) == ld and log_g.shape[0] >= T and beta.shape[0] >= T, "state_step: log_g and beta are rows of one stride")
-        a.log_g, a.beta, a.ld_gb, a.mode = log_g.data_ptr(), beta.data_ptr(), ld, STEP_DELTA
+        ld = _f32_rows(beta, "beta", n_heads)
+        _need(beta.shape[0] >= T, "state_step: fewer rows of beta than of out")
+        a.beta, a.ld_gb, a.mode = beta.data_ptr(), ld, STEP_DELTA
+        if narrow is None:
+            _need(_f32_rows(log_g, "log_g", n_heads) == ld and log_g.shape[0] >= T, "state_step: log_g and beta are rows of one stride")
+            a.log_g = log_g.data_ptr()
         if raw is not None:
             channels, taps = raw.conv_w.shape
             _dev(positions, "positions", torch.int32)
             _need(channels == 2 * n_key_heads * key_dim + n_heads * value_dim and raw.a_log.numel() == n_heads
-                  and raw.dt_bias.numel() == n_heads and positions.numel() >= T, "state_step: the convolution's channels, gates a head")
+                  and raw.dt_bias.numel() == n_heads * (key_dim if narrow is not None else 1) and positions.numel() >= T,
+                  "state_step: the convolution's channels, gates a head")
             _need(taps == 1 or raw.ring_offset + taps * channels <= state.shape[1], "state_step: the state rows are too short")
             a.mode, a.conv_w, a.taps, a.ring_offset = STEP_DELTA_RAW, raw.conv_w.data_ptr(), taps, raw.ring_offset
             a.A_log, a.dt_bias, a.positions, a.q_scale = raw.a_log.data_ptr(), raw.dt_bias.data_ptr(), positions.data_ptr(), raw.q_scale
+        if narrow is not None:
+            u, nm = narrow
+            ldu = _f32_rows(u, "u", max(nm.a_col + nm.a2.shape[1], nm.g_col + nm.g2.shape[1]))
+            _need(raw is not None and gate is None and u.shape[0] >= T and nm.a2.shape[0] == n_heads * key_dim
+                  and nm.g2.shape[0] == n_heads * value_dim, "state_step: a row of a2 a key channel, of g2 a value column")
+            a.mode, a.ldz, a.ldy, a.rank, a.g_rank, a.w2_dtype = STEP_CHANNEL_RAW, ldu, ldu, nm.a2.shape[1], nm.g2.shape[1], DT[nm.a2.dtype]
+            a.z, a.y, a.a2, a.g2 = u.data_ptr() + 4 * nm.a_col, u.data_ptr() + 4 * nm.g_col, nm.a2.data_ptr(), nm.g2.data_ptr()
+    _need(gate_activation in ("silu", "sigmoid"), f"state_step: gate activation {gate_activation!r}")
+    a.gate_sigmoid = int(gate_activation == "sigmoid")
     rc = lib.state_step(ctypes.byref(a), _stream())
     build.check(lib, rc, "state_step")
     return out
@@ -1894,7 +1953,16 @@ class DeltaChunkArgs(ctypes.Structure):
                 ("state", _vp), ("state_stride", _c_size_t), ("state_offset", _c_size_t), ("span_req", _vp), ("span_start", _vp),
                 ("span_first", _vp), ("seq_start", _vp), ("seq_len", _vp), ("slot_ids", _vp), ("n_chunks", _c_int), ("n_requests", _c_int),
                 ("H", _c_int), ("Hk", _c_int), ("N", _c_int), ("P", _c_int), ("norm_w", _vp), ("norm_stride", _c_int), ("eps", _c_float),
-                ("gate", _vp), ("ldg", _c_int), ("out", _vp), ("ldo", _c_int), ("out_dtype", _c_int)]
+                ("gate", _vp), ("ldg", _c_int), ("out", _vp), ("ldo", _c_int), ("out_dtype", _c_int), ("gate_sigmoid", _c_int), ("k_end", _vp),
+                ("q_hat", _vp), ("scores", _vp), ("shrink", _vp)]
+
+
+class LowRankGates(ctypes.Structure):
+    """Mirror of ``LowRankGates`` in csrc/delta_chunks.hip."""
+
+    _fields_ = [("u", _vp), ("ldu", _c_int), ("n_rows", _c_int), ("a_col", _c_int), ("a_rank", _c_int), ("a2", _vp), ("A_log", _vp),
+                ("dt_bias", _vp), ("log_g", _vp), ("g_col", _c_int), ("g_rank", _c_int), ("g2", _vp), ("gate", _vp), ("H", _c_int),
+                ("N", _c_int), ("P", _c_int), ("dtype", _c_int)]
 
 
 DELTA_CHUNK = 64  # tokens a chunk
@@ -1905,18 +1973,21 @@ def _sixteens(n):
 
 
 def delta_prepare(alloc, u, b_col, a_col, n_heads, n_key_heads, key_dim, value_dim, raw, state, token_req, positions, seq_start,
-                  seq_len, slot_ids):
+                  seq_len, slot_ids, narrow=None):
     """The delta rule's operands from the projection's float32 rows ``u`` (queries, keys and values from
     column 0 on, the columns that become ``beta`` and ``g`` from ``b_col`` and ``a_col``): ``(q, k, v,
     log_g, beta)`` in memory that ``alloc(shape, dtype)`` gives, heads padded by zeros to multiples of
-    sixteen columns.  ``raw``: a ``DeltaRaw``.  The requests' last inputs go to their rings."""
+    sixteen columns.  ``raw``: a ``DeltaRaw``.  The requests' last inputs go to their rings.  With ``narrow`` (a
+    ``NarrowMiddle``; ``a_col`` is not used) ``log_g`` has a column for every (padded) key channel of a head, and the
+    output gate's logits, float32 ``[rows, heads * value_dim]``, come sixth."""
     lib = build.load("delta_chunks")
     T = u.shape[0]
     channels, taps = raw.conv_w.shape
     a = DeltaPrepareArgs()
+    a_col = 0 if narrow is not None else a_col
     a.ldu, a.u = _f32_rows(u, "u", max(channels, b_col + n_heads, a_col + n_heads)), u.data_ptr()
     _need(channels == 2 * n_key_heads * key_dim + n_heads * value_dim and raw.a_log.numel() == n_heads
-          and raw.dt_bias.numel() == n_heads, "delta_prepare: the convolution's channels, gates a head")
+          and raw.dt_bias.numel() == n_heads * (key_dim if narrow is not None else 1), "delta_prepare: the convolution's channels, gates a head")
     _dev(state, "state", torch.float32)
     _need(state.dim() == 2 and (taps == 1 or raw.ring_offset + taps * channels <= state.shape[1]), "delta_prepare: the state rows are too short")
     a.b_col, a.a_col, a.n_rows, a.H, a.Hk, a.N, a.P = int(b_col), int(a_col), T, int(n_heads), int(n_key_heads), int(key_dim), int(value_dim)
@@ -1929,11 +2000,25 @@ def delta_prepare(alloc, u, b_col, a_col, n_heads, n_key_heads, key_dim, value_d
         setattr(a, name, t.data_ptr())
     q, k = (alloc((T, n_key_heads * _sixteens(key_dim)), torch.float32) for _ in range(2))
     v = alloc((T, n_heads * _sixteens(value_dim)), torch.float32)
-    log_g, beta = alloc((T, n_heads), torch.float32), alloc((T, n_heads), torch.float32)
-    a.q, a.k, a.v, a.log_g, a.beta = (t.data_ptr() for t in (q, k, v, log_g, beta))
+    log_g = alloc((T, n_heads * (_sixteens(key_dim) if narrow is not None else 1)), torch.float32)
+    beta = alloc((T, n_heads), torch.float32)
+    a.q, a.k, a.v, a.beta = (t.data_ptr() for t in (q, k, v, beta))
+    a.log_g = log_g.data_ptr() if narrow is None else None
     rc = lib.delta_prepare(ctypes.byref(a), _stream())
     build.check(lib, rc, "delta_prepare")
-    return q, k, v, log_g, beta
+    if narrow is None:
+        return q, k, v, log_g, beta
+    gate = alloc((T, n_heads * value_dim), torch.float32)
+    g = LowRankGates()
+    g.ldu = _f32_rows(u, "u", max(narrow.a_col + narrow.a2.shape[1], narrow.g_col + narrow.g2.shape[1]))
+    _need(narrow.a2.shape[0] == n_heads * key_dim and narrow.g2.shape[0] == n_heads * value_dim, "delta_prepare: a row of a2 a key channel, of g2 a value column")
+    g.u, g.n_rows, g.a_col, g.a_rank, g.a2 = u.data_ptr(), T, narrow.a_col, narrow.a2.shape[1], narrow.a2.data_ptr()
+    g.A_log, g.dt_bias, g.log_g = raw.a_log.data_ptr(), raw.dt_bias.data_ptr(), log_g.data_ptr()
+    g.g_col, g.g_rank, g.g2, g.gate = narrow.g_col, narrow.g2.shape[1], narrow.g2.data_ptr(), gate.data_ptr()
+    g.H, g.N, g.P, g.dtype = a.H, a.N, a.P, DT[narrow.a2.dtype]
+    rc = lib.lowrank_gates(ctypes.byref(g), _stream())
+    build.check(lib, rc, "lowrank_gates")
+    return q, k, v, log_g, beta, gate
 
 
 def delta_chunks_takes(key_dim, value_dim):
@@ -1941,24 +2026,32 @@ def delta_chunks_takes(key_dim, value_dim):
 
 
 def delta_chunks(out, operands, state, state_offset, spans, seq_start, seq_len, slot_ids, n_requests, n_heads, n_key_heads, key_dim,
-                 value_dim, norm_weight, eps, gate, alloc):
+                 value_dim, norm_weight, eps, gate, alloc, by_channel=False, gate_activation="silu"):
     """The gated delta rule over ``operands`` (what ``delta_prepare`` returned) in chunks of 64 tokens;
     the rest as in ``state_step``.  ``spans``: ``(number of chunks, request of each, its first token
-    counted from the request's first of this step, every request's first chunk)``, int32 on the device."""
+    counted from the request's first of this step, every request's first chunk)``, int32 on the device.  ``by_channel``: ``log_g`` has
+    a column for every padded key channel of a head; ``gate_activation``: ``silu`` or ``sigmoid``."""
     lib = build.load("delta_chunks")
     q, k, v, log_g, beta = operands
     n_chunks, span_req, span_start, span_first = spans
     T, Np, Pp = out.shape[0], _sixteens(key_dim), _sixteens(value_dim)
     a = DeltaChunkArgs()
     for name, t, shape in (("q", q, (T, n_key_heads * Np)), ("k", k, (T, n_key_heads * Np)), ("v", v, (T, n_heads * Pp)),
-                           ("log_g", log_g, (T, n_heads)), ("beta", beta, (T, n_heads))):
+                           ("log_g", log_g, (T, n_heads * Np if by_channel else n_heads)), ("beta", beta, (T, n_heads))):
         _dev(t, name, torch.float32)
         _need(tuple(t.shape) == shape, f"delta_chunks: {name} is {tuple(t.shape)}, want {shape}")
         setattr(a, name, t.data_ptr())
-    work = {"cum": alloc((T, n_heads), torch.float32), "w": alloc((T, n_heads * Np), torch.float32),
+    work = {"w": alloc((T, n_heads * Np), torch.float32),
             "u": alloc((T, n_heads * Pp), torch.float32), "states": alloc((n_chunks, n_heads, Np, Pp), torch.float32)}
+    if by_channel:
+        work.update(k_end=alloc((T, n_heads * Np), torch.float32), q_hat=alloc((T, n_heads * Np), torch.float32),
+                    scores=alloc((n_chunks, n_heads, DELTA_CHUNK, DELTA_CHUNK), torch.float32), shrink=alloc((n_chunks, n_heads, Np), torch.float32))
+    else:
+        work["cum"] = alloc((T, n_heads), torch.float32)
     for name, t in work.items():
         setattr(a, name, t.data_ptr())
+    _need(gate_activation in ("silu", "sigmoid"), f"delta_chunks: gate activation {gate_activation!r}")
+    a.gate_sigmoid = int(gate_activation == "sigmoid")
     _dev(state, "state", torch.float32)
     _need(state.dim() == 2 and state_offset + n_heads * key_dim * value_dim <= state.shape[1], "delta_chunks: the state rows are too short")
     a.state, a.state_stride, a.state_offset = state.data_ptr(), state.stride(0), int(state_offset)
@@ -1979,4 +2072,156 @@ def delta_chunks(out, operands, state, state_offset, spans, seq_start, seq_len, 
     a.out, a.out_dtype = out.data_ptr(), DT[out.dtype]
     rc = lib.delta_chunks(ctypes.byref(a), _stream())
     build.check(lib, rc, "delta_chunks")
+    return out
+
+
+# ---------------------------------------------------------------------------
+# a residual stream kept as several streams (csrc/hyper.hip)
+
+
+class HyperArgs(ctypes.Structure):
+    """Mirror of ``HyperArgs`` in csrc/hyper.hip."""
+
+    _fields_ = [("xs", _vp), ("first", _vp), ("ld_first", _c_int), ("xs_out", _vp), ("y", _vp), ("ldy", _c_int), ("n_parts", _c_int),
+                ("y_part", _c_size_t), ("bias", _vp), ("mix", _vp), ("out", _vp), ("in_", _vp), ("gamma", _vp), ("beta", _vp),
+                ("eps", _c_float), ("norm_out", _vp), ("norm_dtype", _c_int), ("sum_out", _vp), ("ld_sum", _c_int), ("T", _c_int),
+                ("D", _c_int), ("S", _c_int)]
+
+
+HYPER_MAX_STREAMS, HYPER_MAX_WIDTH = 8, 32768
+
+
+class HyperWrite:
+    """A sublayer's output on its way into the streams: ``x_t <- sum_s mix[s, t] x_s + out[t] y``.  ``y`` float32
+    ``[tokens, width]``; where ``pending`` (a ``PendingSum``) waits on it, its value still lies in that sum's parts."""
+
+    def __init__(self, y, mix, out, pending=None):
+        self.y, self.mix, self.out, self.pending = y, mix, out, pending
+
+
+def hyper_step(n_streams, width, xs=None, first=None, xs_out=None, write=None, read=None, norm_out=None, gamma=None, beta=None, eps=0.0,
+               sum_out=None):
+    """One pass over the streams ``xs`` (float32 ``[tokens, streams, width]``; all of them are ``first``, ``[tokens,
+    width]``, where ``xs`` is None): ``write`` (a ``HyperWrite``) first, the new streams into ``xs_out`` (may be
+    ``xs``), then ``u = sum_s read[s] x_s`` (``read`` None: the plain sum), its LayerNorm into ``norm_out`` and ``u``
+    itself into ``sum_out``."""
+    lib = build.load("hyper")
+    a = HyperArgs()
+    src = xs if xs is not None else first
+    T = src.shape[0]
+    for name, t, shape in (("xs", xs, (T, n_streams, width)), ("xs_out", xs_out, (T, n_streams, width))):
+        if t is not None:
+            _dev(t, name, torch.float32)
+            _need(tuple(t.shape) == shape and t.is_contiguous(), f"hyper_step: {name} is {tuple(t.shape)}, want {shape}")
+            setattr(a, name, t.data_ptr())
+    if xs is None:
+        a.ld_first, a.first = _f32_rows(first, "first", width), first.data_ptr()
+    if write is not None:
+        y = write.y
+        _need(tuple(y.shape) == (T, width), "hyper_step: y")
+        a.ldy, a.n_parts, a.y = _f32_rows(y, "y", width), 1, y.data_ptr()
+        if write.pending is not None and write.pending.waits_on(y):
+            c = write.pending.c
+            a.y, a.ldy, a.n_parts, a.y_part, a.bias = c.ws, width, c.n_splits, T * width, c.bias
+            c.target = None  # (this adds the parts; nobody else has to)
+        for name, t, n in (("mix", write.mix, n_streams * n_streams), ("out", write.out, n_streams)):
+            _dev(t, name, torch.float32)
+            _need(t.numel() == n and t.is_contiguous(), f"hyper_step: {name} has {n} values")
+            setattr(a, name, t.data_ptr())
+    for field, name, t, n in (("in_", "read", read, n_streams), ("gamma", "gamma", gamma, width), ("beta", "beta", beta, width)):
+        if t is not None:
+            _dev(t, name, torch.float32)
+            _need(t.numel() == n, f"hyper_step: {name} has {n} values")
+            setattr(a, field, t.data_ptr())
+    if norm_out is not None:
+        _need(tuple(norm_out.shape) == (T, width) and norm_out.is_contiguous() and norm_out.dtype in DT, "hyper_step: norm_out")
+        a.norm_out, a.norm_dtype, a.eps = norm_out.data_ptr(), DT[norm_out.dtype], float(eps)
+    if sum_out is not None:
+        _need(sum_out.shape[0] >= T, "hyper_step: sum_out")
+        a.ld_sum, a.sum_out = _f32_rows(sum_out, "sum_out", width), sum_out.data_ptr()
+    a.T, a.D, a.S = T, int(width), int(n_streams)
+    rc = lib.hyper_step(ctypes.byref(a), _stream())
+    build.check(lib, rc, "hyper_step")
+
+
+# ---------------------------------------------------------------------------
+# the real-gated linear recurrent unit (csrc/rglru.hip)
+
+
+class RglruArgs(ctypes.Structure):
+    """Mirror of ``RglruArgs`` in csrc/rglru.hip."""
+
+    _fields_ = [("x", _vp), ("y", _vp), ("ldx", _c_int), ("conv_w", _vp), ("conv_b", _vp), ("taps", _c_int), ("ra", _vp), ("ri", _vp),
+                ("ra_b", _vp), ("ri_b", _vp), ("lam", _vp), ("state", _vp), ("state_stride", _c_size_t), ("state_offset", _c_size_t),
+                ("ring_offset", _c_size_t), ("positions", _vp), ("seq_start", _vp), ("seq_len", _vp),
+                ("slot_ids", _vp), ("span_req", _vp), ("span_start", _vp), ("span_first", _vp), ("a", _vp), ("b", _vp), ("does", _vp),
+                ("s0", _vp), ("out", _vp), ("ldo", _c_int), ("dtype", _c_int), ("n_requests", _c_int), ("n_spans", _c_int),
+                ("W", _c_int), ("B", _c_int), ("w", _c_int), ("wp", _c_int), ("decay", _c_float)]
+
+
+def rglru_takes(part):
+    """Whether the unit's kernels take gate matrices of ``part`` channels."""
+    return bool(build.load("rglru").rglru_takes(_c_int(int(part))))
+
+
+class RglruWeights:
+    """The unit's weights: ``conv_w`` float32 ``[width, taps]``, ``conv_b`` ``[width]`` or None; the gates'
+    matrices ``[blocks, part, part]`` of the compute dtype (kept padded by zero columns to a multiple of 8), their
+    shifts and ``lam`` float32 ``[width]``; ``decay``: the constant of ``log a = -decay r softplus(lam)``."""
+
+    def __init__(self, conv_w, conv_b, ra, ra_b, ri, ri_b, lam, decay):
+        self.blocks, self.part = ra.shape[0], ra.shape[1]
+        self.width, self.taps = conv_w.shape
+        _need(tuple(ra.shape) == tuple(ri.shape) == (self.blocks, self.part, self.part) and self.blocks * self.part == self.width
+              and ra.dtype == ri.dtype and ra.dtype in DT, "rglru: square gate matrices, one a block")
+        pad = -self.part % 8
+        self.ra, self.ri = (torch.cat([t, t.new_zeros(self.blocks, self.part, pad)], 2).contiguous() if pad else t.contiguous() for t in (ra, ri))
+        self.conv_w, self.conv_b, self.decay = conv_w.contiguous(), conv_b, float(decay)
+        self.ra_b, self.ri_b, self.lam = ra_b.reshape(-1).contiguous(), ri_b.reshape(-1).contiguous(), lam.contiguous()
+        for name, t in (("conv_w", self.conv_w), ("ra_b", self.ra_b), ("ri_b", self.ri_b), ("lam", self.lam)):
+            _dev(t, name, torch.float32)
+            _need(t.numel() == self.width * (self.taps if name == "conv_w" else 1), f"rglru: {name}")
+
+
+def rglru(out, x, y, weights, state, state_offset, ring_offset, positions, seq_start, seq_len, slot_ids, n_requests, spans, alloc):
+    """``out = S * gelu_tanh(y)`` with ``S`` the unit's state over ``conv(x)``, for every token: ``x`` and ``y``
+    float32 columns of the same rows, ``out`` of the gates' dtype.  A request's row of ``state`` holds ``S`` (``width``
+    floats at ``state_offset``) and the convolution's inputs (a ring ``[taps, width]`` at ``ring_offset``, position
+    ``p`` in row ``p % taps``; none for one tap).  ``spans``: None where every request brings one token, otherwise
+    ``(number of spans of 64 tokens, request of each, its first token counted from the request's first of this
+    step, every request's first span)``."""
+    lib = build.load("rglru")
+    w, a = weights, RglruArgs()
+    T = out.shape[0]
+    a.ldx, a.x, a.y = _f32_rows(x, "x", w.width), x.data_ptr(), y.data_ptr()
+    _need(_f32_rows(y, "y", w.width) == a.ldx and x.shape[0] >= T and y.shape[0] >= T, "rglru: x and y are columns of the same rows")
+    a.conv_w, a.conv_b, a.taps = w.conv_w.data_ptr(), native.ptr(w.conv_b), w.taps
+    a.ra, a.ri, a.ra_b, a.ri_b, a.lam = (t.data_ptr() for t in (w.ra, w.ri, w.ra_b, w.ri_b, w.lam))
+    _dev(state, "state", torch.float32)
+    _need(state.dim() == 2 and state_offset + w.width <= state.shape[1]
+          and (w.taps == 1 or ring_offset + w.taps * w.width <= state.shape[1]), "rglru: the state rows are too short")
+    a.state, a.state_stride, a.state_offset, a.ring_offset = state.data_ptr(), state.stride(0), int(state_offset), int(ring_offset)
+    for name, t, n in (("positions", positions, T), ("seq_start", seq_start, n_requests), ("seq_len", seq_len, n_requests),
+                       ("slot_ids", slot_ids, n_requests)):
+        _dev(t, name, torch.int32)
+        _need(t.numel() >= n, f"rglru: {name} too short")
+        setattr(a, name, t.data_ptr())
+    a.ldo, a.out, a.dtype = _rows2d(out, "out"), out.data_ptr(), DT[out.dtype]
+    _need(out.dtype == w.ra.dtype and out.shape[1] >= w.width, "rglru: out has the gates' dtype and a column a channel")
+    a.n_requests, a.W, a.B, a.w, a.wp, a.decay = int(n_requests), w.width, w.blocks, w.part, w.ra.shape[2], w.decay
+    if spans is None:
+        rc = lib.rglru_step(ctypes.byref(a), _stream())
+        build.check(lib, rc, "rglru_step")
+        return out
+    n_spans, span_req, span_start, span_first = spans
+    for name, t, n in (("span_req", span_req, n_spans), ("span_start", span_start, n_spans), ("span_first", span_first, n_requests)):
+        _dev(t, name, torch.int32)
+        _need(t.numel() >= n, f"rglru: {name} too short")
+        setattr(a, name, t.data_ptr())
+    a.n_spans = int(n_spans)
+    work = [alloc((T, w.width), torch.float32), alloc((T, w.width), torch.float32), alloc((n_spans, w.width, 2), torch.float32),
+            alloc((n_requests, w.width), torch.float32)]
+    a.a, a.b, a.does, a.s0 = (t.data_ptr() for t in work)
+    rc = lib.rglru_portions(ctypes.byref(a), _stream())
+    build.check(lib, rc, "rglru_portions")
     return out

@@ -1,7 +1,7 @@
 """Parts that models are put together from; importing this registers the built-in kinds."""
 
 from . import (attention, block, convolution, delta_rule, differential_attention, embedding, experts, feed_forward,  # noqa: F401
-               gated_attention, head, latent_attention, linear_state, norms, positions, scored_attention, time_mix)
+               gated_attention, head, latent_attention, linear_state, norms, positions, recurrent_unit, scored_attention, time_mix)
 from .base import (
     BLOCKS,
     EMBEDDINGS,

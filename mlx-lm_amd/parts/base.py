@@ -180,6 +180,22 @@ class ProjectsFirst:
         return rows[:, : self.in_cols]
 
 
+class OutputProduct:
+    """What a mixer or feed-forward that ends with one product adds so that its arrangement can say where
+    that goes: added into the rows it is given, or (``overwrite``) written there; with ``pending`` (a
+    ``PendingSum``) a product that splits K may leave its parts for the arrangement's next kernel."""
+
+    can_overwrite = True
+    overwrite = False
+    pending = None
+
+    def output(self, rows, x, w):
+        from ..ops import kernels
+
+        kernels.linear(rows, x, w, accumulate=not self.overwrite, pending=self.pending,
+                       splits=None if self.pending is not None else kernels.splits_alone(x.shape[0]))
+
+
 class FeedForward(Part):
     native_kind = native.FFN
 

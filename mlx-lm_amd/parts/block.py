@@ -404,7 +404,127 @@ class SharedNormBlock(Block):
         return h
 
 
+class HyperBlock(Block):
+    """Hyper-connected sublayers: the residual stream is kept as ``streams`` streams ``x_s``, all equal to the
+    embedding's rows at the start and summed up at the end, and a sublayer ``f`` with its tensors ``in``, ``out``
+    (a value a stream) and ``mix`` (``[from, to]``) does
+
+        ``y = f(norm(sum_s in[s] x_s))``,   ``x_t <- sum_s mix[s, t] x_s + out[t] y``.
+
+    The mixer is the first sublayer (tensors ``<names[0]>in`` ...), the feed-forward the second
+    (``<names[1]>``...); it may be absent.  The norms are LayerNorms.  Between two sublayers one kernel writes the
+    first one's output into the streams, reads for the second and norms (csrc/hyper.hip), so the write of a
+    layer's last sublayer waits for the next run's first kernel: the runs of a step share streams and the waiting
+    write through ``ctx.shared``, and the last of ``n_runs`` runs leaves the sum in ``h``.  A sublayer
+    that ends with a product leaves its float32 rows, or the parts of a product that splits K, to that kernel
+    (``OutputProduct``).  All of it is 32-bit.  No counterpart in mlx_lm/models/gpt2.py, which has one stream
+    (:98-108).
+    """
+
+    PARTS = {"mixer_norm": "norm", "mixer": "mixer", "ffn_norm": "norm", "ffn": "feed_forward"}
+    OPTIONAL = ("ffn_norm", "ffn")
+
+    def __init__(self, mixer_norm, mixer, ffn_norm=None, ffn=None, streams=1, n_runs=1, names=("hc1.", "hc2."), prefix=""):
+        from ..ops import kernels
+
+        super().__init__(prefix)
+        if (ffn is None) != (ffn_norm is None):
+            raise ValueError("a layer has a feed-forward and its norm, or neither")
+        for norm in (mixer_norm, ffn_norm):
+            if norm is not None and not hasattr(norm, "has_bias"):
+                raise ValueError(f"this arrangement fuses LayerNorms, not a {type(norm).__name__}")
+        self.mixer_norm, self.mixer, self.ffn_norm, self.ffn = mixer_norm, mixer, ffn_norm, ffn
+        self.width, self.streams, self.n_runs = mixer_norm.width, int(streams), int(n_runs)
+        if not 1 <= self.streams <= kernels.HYPER_MAX_STREAMS or self.width % 4 or self.width > kernels.HYPER_MAX_WIDTH:
+            raise ValueError(f"{streams} streams (1 to {kernels.HYPER_MAX_STREAMS}) of {self.width} columns")
+        self.names = [self._name(n) for n in names][: 1 if ffn is None else 2]
+        for part in (mixer, ffn):
+            if part is not None and getattr(part, "can_overwrite", False):
+                part.overwrite = True
+        self.graph_safe = all(getattr(p, "graph_safe", False) for p in self.parts() if p is not self)
+
+    def parts(self):
+        out = []
+
+        def walk(part):
+            if part is None:
+                return
+            out.append(part)
+            for sub in getattr(part, "sub_parts", lambda: ())():
+                walk(sub)
+
+        for p in (self.mixer_norm, self.mixer, self.ffn_norm, self.ffn):
+            walk(p)
+        return tuple(out) + (self,)  # (the arrangement owns tensors itself, so it is one of its own parts)
+
+    def tensors(self):
+        t = {}
+        for n in self.names:
+            t[n + "in"], t[n + "out"] = TensorSpec((self.streams,), "vector"), TensorSpec((self.streams,), "vector")
+            t[n + "mix"] = TensorSpec((self.streams, self.streams), "vector")
+        return t
+
+    def load(self, tensors):
+        from ..ops import kernels
+
+        self.connections = [tuple(tensors[n + x].contiguous() for x in ("in", "mix", "out")) for n in self.names]
+        self.pending = kernels.PendingSum()
+        self.pending.c.allowed = 2
+        for part in (self.mixer, self.ffn):
+            if part is not None and hasattr(part, "pending"):
+                part.pending = self.pending
+
+    def cache_need(self):
+        return self.mixer.cache_need()
+
+    def state_need(self):
+        if getattr(self.mixer, "wants_state", False) and hasattr(self.mixer, "state_need"):
+            return self.mixer.state_need()
+        return None
+
+    def forward(self, ctx, h, cache, writes_cache=True, state=None):
+        import torch
+
+        from ..ops import kernels
+
+        T, D = h.shape
+        step = ctx.shared.get("hyper")
+        if step is None:
+            step = ctx.shared["hyper"] = {"runs": 0, "live": False, "write": None, "y": ctx.scratch((T, D), torch.float32),
+                                          "xs": ctx.scratch((T, self.streams, D), torch.float32)}
+        mark = ctx.scratch_mark()
+        u = ctx.scratch((T, D), ctx.dtype)
+        for part, norm, (read, mix, out) in zip((self.mixer, self.ffn), (self.mixer_norm, self.ffn_norm), self.connections):
+            y = step["y"]
+            self._pass(ctx, h, step, keep=True, read=read, norm_out=u, gamma=norm.weight, beta=norm.bias, eps=norm.eps)
+            if not getattr(part, "overwrite", False):
+                y.zero_()
+            if part is self.ffn:
+                part.forward(ctx, u, y)
+            elif getattr(part, "wants_state", False):
+                part.forward(ctx, u, y, cache, writes_cache, state=state)
+            else:
+                part.forward(ctx, u, y, cache, writes_cache)
+            step["write"] = kernels.HyperWrite(y, mix, out, self.pending)
+        ctx.scratch_release(mark)
+        step["runs"] += 1
+        if step["runs"] == self.n_runs:
+            self._pass(ctx, h, step, keep=False, sum_out=h)
+            del ctx.shared["hyper"]
+        return h
+
+    def _pass(self, ctx, h, step, keep, **what):
+        """What waits to be written, and then a read.  Until the first write every stream is ``h`` itself."""
+        from ..ops import kernels
+
+        write, xs = step["write"], step["xs"] if step["live"] else None
+        out = step["xs"] if keep and write is not None else None
+        kernels.hyper_step(self.streams, self.width, xs=xs, first=h if xs is None else None, xs_out=out, write=write, **what)
+        step["write"], step["live"] = None, step["live"] or out is not None
+
+
 register_block("pre_norm", PreNormBlock)
+register_block("hyper", HyperBlock)
 register_block("shared_norm", SharedNormBlock)
 register_block("sandwich", SandwichBlock)
 register_block("post_norm", PostNormBlock)

@@ -15,6 +15,9 @@ class GatedExperts(FeedForward):
       of the products of the compute dtype's operands); the ``top`` largest of ``s + correction``
       are chosen (``correction``: a tensor, or none), and weigh in with ``s`` itself; with
       ``renormalize`` divided by the chosen ones' sum (+ 1e-20); times ``weight_scale``;
+    * ``scores = "sigmoid"``: ``s`` is the logistic function of each output instead; ``groups = (count,
+      keep)``: only experts of the ``keep`` best of ``count`` equal groups of neighbours can be chosen, a
+      group counting the sum of its two largest choice scores;
     * the last ``n_identity`` router outputs stand for experts that give their input back;
     * ``shared_inner > 0``: one more expert of that inner size (``shared.gate`` ...) that every
       token uses with weight one;
@@ -39,7 +42,7 @@ class GatedExperts(FeedForward):
     TILES_FROM, TILES_MIN, TILES_EACH = 64, 8, 3
 
     def __init__(self, width, n_experts, inner, top, n_identity=0, shared_inner=0, correction=True, renormalize=False,
-                 weight_scale=1.0, activation="silu", limit=0.0, prefix=""):
+                 weight_scale=1.0, activation="silu", limit=0.0, scores="softmax", groups=None, prefix=""):
         super().__init__(prefix)
         if activation not in kernels.EXPERT_ACTIVATIONS:
             raise ValueError(f"experts' activation {activation!r} (known: {sorted(kernels.EXPERT_ACTIVATIONS)})")
@@ -47,7 +50,8 @@ class GatedExperts(FeedForward):
             raise ValueError(f"clamped activations need a positive limit, got {limit}")
         self.activation, self.limit = activation, float(limit)
         self.projection_given = False  # the router's outputs come out of a product that another part makes
-        self.renormalize, self.weight_scale = bool(renormalize), float(weight_scale)
+        self.renormalize, self.weight_scale, self.scores = bool(renormalize), float(weight_scale), scores
+        self.groups = tuple(groups) if groups is not None else None
         if n_experts < 0 or n_identity < 0 or n_experts + n_identity <= 0:
             raise ValueError(f"{n_experts} experts and {n_identity} identity experts")
         if not 0 < top <= n_experts + n_identity:
@@ -61,6 +65,12 @@ class GatedExperts(FeedForward):
         self.n_out = n_experts + n_identity
         self.shared_padded = (self.shared_inner + 7) // 8 * 8  # zero weights beyond: silu(0) * 0 = 0 meets zero columns
         self.overwrite = False
+        if scores not in kernels.ROUTER_SCORES:
+            raise ValueError(f"router scores {scores!r} (known: {kernels.ROUTER_SCORES})")
+        if self.groups is not None:
+            count, keep = self.groups
+            if count <= 0 or self.n_out % count or not 0 < keep <= count or top > keep * (self.n_out // count):
+                raise ValueError(f"{top} picks out of {keep} of {count} groups of {self.n_out} experts")
 
     def tensors(self):
         n, t = self._name, {}
@@ -92,6 +102,8 @@ class GatedExperts(FeedForward):
             self.router_w = kernels.for_decode(tensors[n("router")].contiguous())
             self.first_weight = self.router_w
         self.correction = tensors[n("correction")] if self.has_correction else None
+        self.choice = dict(renormalize=self.renormalize, weight_scale=self.weight_scale, scores=self.scores, groups=self.groups)
+        self.route = kernels.Route(self.correction, **self.choice)
         self.shared_in = self.shared_out = None
         if self.shared_inner:
             g, u, d = tensors[n("shared.gate")], tensors[n("shared.up")], tensors[n("shared.down")]
@@ -124,7 +136,7 @@ class GatedExperts(FeedForward):
             zu = ctx.scratch((T, self.n_out + 2 * self.shared_padded), torch.float32)
             kernels.linear(zu, x, self.merged_in)
             act = ctx.scratch((T, self.shared_padded), ctx.dtype)
-            kernels.route_and_gate(idx, weight, act, zu, self.correction, self.top, self.n_out, self.renormalize, self.weight_scale)
+            kernels.route_and_gate(idx, weight, act, zu, self.correction, self.top, self.n_out, **self.choice)
             kernels.linear(residual, act, self.shared_out, accumulate=accumulate)
             accumulate = True
         else:
@@ -133,9 +145,9 @@ class GatedExperts(FeedForward):
                 z = ctx.scratch((T, self.n_out), torch.float32)
                 kernels.linear(z, x, self.router_w, splits=kernels.splits_alone(T))
             if not tiles and self.n_experts and self.top <= kernels.ROUTED_MOST:
-                route = (z, self.correction, self.renormalize, self.weight_scale)  # (chosen by the kernel that reads the experts)
+                route = (z, self.route)  # (chosen by the kernel that reads the experts)
             else:
-                kernels.router_choice(idx, weight, z, self.correction, self.top, self.renormalize, self.weight_scale)
+                kernels.router_choice(idx, weight, z, self.correction, self.top, **self.choice)
         if self.shared_inner and not merged:
             gu = ctx.scratch((T, 2 * self.shared_padded), ctx.dtype)
             kernels.linear(gu, x, self.shared_in, splits=kernels.splits_alone(T))

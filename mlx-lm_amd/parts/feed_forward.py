@@ -5,7 +5,7 @@ import ctypes
 import torch
 
 from ..ops import kernels, native
-from .base import FeedForward, TensorSpec, register_feed_forward, value_of
+from .base import FeedForward, OutputProduct, TensorSpec, register_feed_forward, value_of
 
 _TANH_GELU = ("gelu_new", "gelu_pytorch_tanh", "gelu_tanh", "gelu_approx")
 
@@ -118,12 +118,12 @@ class Relu2MLP(FeedForward):
         native.check(rc, "relu2_mlp")
 
 
-class GatedMLP(FeedForward):
+class GatedMLP(OutputProduct, FeedForward):
     """``down(act(gate(x)) * up(x))``, dense, no biases; ``activation``: ``silu`` or ``gelu_tanh``.
 
     One product gives ``[gate | up]``; the activation and the product of the two halves are one
     kernel (``silu_mul``, which the experts' shared expert uses too); the second product adds into
-    ``residual``.  No counterpart in mlx_lm/models/gpt2.py, whose MLP (:71-80) has no gate.
+    ``residual`` (or writes it: ``OutputProduct``).  No counterpart in mlx_lm/models/gpt2.py, whose MLP (:71-80) has no gate.
     """
 
     graph_safe = True  # launches kernels only: a step of such parts can be recorded
@@ -166,7 +166,7 @@ class GatedMLP(FeedForward):
         kernels.linear(gate_up, x, self.gate_up_w, splits=kernels.splits_alone(T))
         act = ctx.scratch((T, F), ctx.dtype)
         kernels.silu_mul(act, gate_up, self.activation)
-        kernels.linear(residual, act, self.down_w, accumulate=True, splits=kernels.splits_alone(T))
+        self.output(residual, act, self.down_w)
         ctx.scratch_release(mark)
 
 

@@ -10,14 +10,16 @@ class LayerNorm(Norm):
     """``(x - mean) / sqrt(var + eps) * weight + bias`` with biased variance.
 
     ``nn.LayerNorm(n_embd, eps=layer_norm_epsilon)`` in
-    mlx_lm/models/gpt2.py:92-96,123.  Reads the float32 residual stream,
+    mlx_lm/models/gpt2.py:92-96,123.  ``scale``: a constant that the consumer's output would be
+    multiplied by; it rides on weight and bias.  Reads the float32 residual stream,
     computes in float32, writes the compute dtype.
     """
 
     graph_safe = True  # launches kernels only: a step of such parts can be recorded
 
-    def __init__(self, width, eps, bias=True, weight_name="weight", bias_name="bias", prefix=""):
+    def __init__(self, width, eps, bias=True, weight_name="weight", bias_name="bias", scale=1.0, prefix=""):
         super().__init__(prefix)
+        self.scale = float(scale)
         self.width, self.eps, self.has_bias = width, float(eps), bias
         self.weight_name, self.bias_name = self._name(weight_name), self._name(bias_name)
         self.weight = self.bias = None
@@ -31,6 +33,9 @@ class LayerNorm(Norm):
     def load(self, tensors):
         self.weight = tensors[self.weight_name]
         self.bias = tensors[self.bias_name] if self.has_bias else None
+        if self.scale != 1.0:
+            self.weight = self.weight * self.scale
+            self.bias = self.bias * self.scale if self.has_bias else None
 
     settles_pending = True  # adds a sum that is pending on ``x`` before (or while) it norms the rows
     reads_ahead = True  # ``forward`` takes ``ahead``, the weights that its result meets first

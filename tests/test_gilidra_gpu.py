@@ -412,7 +412,7 @@ def test_the_choice_and_the_next_norm_inside_the_experts_kernels(dtype, F, width
     y, y2, out = start.clone(), start.clone(), torch.empty(T, width, dtype=dtype, device="cuda")
     kernels.expert_rows(y, x, gate, up, down, idx, weight, top, act, activation="clamped", limit=0.8)
     idx2, weight2 = torch.full_like(idx, -1), torch.zeros_like(weight)
-    kernels.expert_rows(y2, x, gate, up, down, idx2, weight2, top, act, activation="clamped", limit=0.8, route=(z, correction, True, 1.5),
+    kernels.expert_rows(y2, x, gate, up, down, idx2, weight2, top, act, activation="clamped", limit=0.8, route=(z, kernels.Route(correction, True, 1.5)),
                         after=(out, norm))
     assert torch.equal(idx, idx2) and torch.equal(weight, weight2) and torch.equal(y, y2)
     want = torch.empty_like(out)
