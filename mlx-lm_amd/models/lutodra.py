@@ -173,7 +173,9 @@ class Model:
             head=PartSpec("linear", {"vocab_size": args.vocab, "width": D, "weight_name": "head"}))
 
     def sanitize(self, weights):
-        return dict(weights)
+        # (a layer without a feed-forward may come with that sublayer's norm and connections: nothing reads them)
+        unread = tuple(f"l{i}.{x}" for i, entry in enumerate(self.args.layers) if entry.get("mlp") is None for x in ("norm2", "hc2."))
+        return {k: v for k, v in weights.items() if not (unread and k.startswith(unread))}
 
     @staticmethod
     def random_weights(args: ModelArgs, seed, scheme="a"):
