@@ -36,8 +36,9 @@ window of 512 that keeps the first 64 tokens.  Ruzolorn runs at the same layer s
 (``ruzolorn_config``), without a window and with one of 512, and Zatinex (``zatinex_config``:
 differential attention, gated linear attention and latent attention by turns, a dense gated
 feed-forward), Sazilorn (``sazilorn_config``: its parallel, HGRN2 and attention mixers by turns,
-dense and expert feed-forwards) and Gilidra (``gilidra_config``: its time-mixing, latent-attention and
-delta-rule mixers by turns, clamped experts).  It prints one JSON line of its own.
+dense and expert feed-forwards), Gilidra (``gilidra_config``: its time-mixing, latent-attention and
+delta-rule mixers by turns, clamped experts) and Lutodra (``lutodra_config``: its delta rule, recurrent
+unit and attention by turns in four hyper-connected streams, grouped experts).  It prints one JSON line of its own.
 """
 
 import argparse
@@ -81,6 +82,8 @@ def design_config(design, size, window=None):
         return sazilorn_config(s)
     if design == "gilidra":
         return gilidra_config(s)
+    if design == "lutodra":
+        return lutodra_config(s)
     mixer = {"heads": s["heads"], "kv_heads": s["heads"], "dim": s["dim"], "vdim": s["dim"], "scale": s["dim"] ** -0.5}
     if window:
         mixer["mask"] = {"size": window[0], "keep_first": window[1]}
@@ -195,6 +198,25 @@ def gilidra_config(s):
             "logit_scale": 0.5, "layers": layers}
 
 
+def lutodra_config(s):
+    """Lutodra at GPT-2's layer sizes in four streams, its three mixers by turns.  Delta rule: Gilidra's heads, key
+    heads and taps, a decay per key channel and a gate through middles of a head's width.  Recurrent unit: as
+    many channels as the stream is wide in parts of 256, four taps.  Attention: as many heads of the same size
+    over a quarter as many key heads, half of every head turning.  Feed-forward: Gilidra's sixteen experts of
+    three sixteenths of GPT-2's inner size, four a token, out of the best two of four groups."""
+    H, d, D = s["heads"], s["dim"], s["width"]
+    scaling = {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 1024}
+    mixers = [("channel_delta", {"heads": H, "kv_heads": H // 2, "dim": d, "vdim": d, "conv": 4, "decay_rank": d, "gate_rank": d}),
+              ("rglru", {"width": D, "blocks": D // 256, "conv": 4}),
+              ("attention", {"heads": H, "kv_heads": H // 4, "dim": d, "vdim": d, "scale": d ** -0.5,
+                             "rot": {"dims": d // 2, "base": 500000.0, "scaling": scaling}})]
+    mlp = {"kind": "moe", "expert": {"ff": s["ff"] * 3 // 16},
+           "router": {"experts": 16, "top": 4, "scale": 1.0, "groups": {"count": 4, "keep": 2}}}
+    layers = [{"type": mixers[i % 3][0], "mixer": mixers[i % 3][1], "mlp": mlp} for i in range(s["layers"])]
+    return {"architecture": "Lutodra", "vocab": DESIGN_VOCAB, "width": D, "streams": 4, "max_positions": DESIGN_POSITIONS,
+            "norm": {"eps": 1e-6}, "logit_scale": 0.5, "layers": layers}
+
+
 def bench_design(config, dtype, batches, steps, warmup):
     """Prefill of 2 x 1,024 tokens (three warm-up trials, the mean of five) and decode from
     context 512 at each of ``batches``, for the model that ``config`` describes."""
@@ -243,7 +265,7 @@ def compare_designs(a):
         entry = {"layer_sizes": DESIGN_SIZES[size]}
         runs = {"gpt2": ("gpt2", None), "pafutar": ("pafutar", None), "pafutar_window_512_keep_64": ("pafutar", (512, 64)),
                 "ruzolorn": ("ruzolorn", None), "ruzolorn_window_512": ("ruzolorn", (512, 0)), "zatinex": ("zatinex", None), "sazilorn": ("sazilorn", None),
-                "gilidra": ("gilidra", None)}
+                "gilidra": ("gilidra", None), "lutodra": ("lutodra", None)}
         for name, (design, window) in runs.items():
             if a.design_only and name not in a.design_only.split(","):
                 continue
@@ -352,7 +374,7 @@ def main():
     ap.add_argument("--designs", action="store_true",
                     help="a mode of its own: Pafutar beside GPT-2 at equal layer sizes (prefill and decode)")
     ap.add_argument("--design-size", choices=sorted(DESIGN_SIZES), default=None, help="with --designs: one size only")
-    ap.add_argument("--design-only", default=None, help="with --designs: one of gpt2, pafutar, pafutar_window_512_keep_64, ruzolorn, ruzolorn_window_512, zatinex, sazilorn, gilidra (or several, separated by commas)")
+    ap.add_argument("--design-only", default=None, help="with --designs: one of gpt2, pafutar, pafutar_window_512_keep_64, ruzolorn, ruzolorn_window_512, zatinex, sazilorn, gilidra, lutodra (or several, separated by commas)")
     a = ap.parse_args()
     if a.designs:
         if a.gpus != 1:

@@ -296,13 +296,16 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaChunkArgs a) {
 
 #define FAR_APART 60.0f  // how far log g may fall within eight tokens for one reference in the middle of sixteen
 
+// (L is kept in units of log 2: the hardware's exponential is that of 2)
+#define LOG2E 1.4426950408889634f
+__device__ __forceinline__ float exp_2(float x) { return __builtin_amdgcn_exp2f(x); }
 __device__ __forceinline__ float4 exp_diff(const float4& a, const float4& b) {
-  return make_float4(expf(a.x - b.x), expf(a.y - b.y), expf(a.z - b.z), expf(a.w - b.w));
+  return make_float4(exp_2(a.x - b.x), exp_2(a.y - b.y), exp_2(a.z - b.z), exp_2(a.w - b.w));
 }
 __device__ __forceinline__ float4 mul4(const float4& a, const float4& b) { return make_float4(a.x * b.x, a.y * b.y, a.z * b.z, a.w * b.w); }
 
 __global__ __launch_bounds__(256) void delta_solve_channel_kernel(DeltaChunkArgs a) {
-  extern __shared__ __attribute__((aligned(16))) float Ls[];  // [C + 1][Np + 4]: L, row 0 before the first token
+  extern __shared__ __attribute__((aligned(16))) float Ls[];  // [C + 1][Np + 4]: L / log 2, row 0 before the first token
   __shared__ float A[C * CS], Tm[C * CS], tmp[4][16 * SS], bt[C];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lg = lane >> 4;
   const int h = blockIdx.x, hk = h / (a.H / a.Hk), Np = (a.N + 15) & ~15, Pp = (a.P + 15) & ~15, LS = Np + 4;
@@ -325,7 +328,7 @@ __global__ __launch_bounds__(256) void delta_solve_channel_kernel(DeltaChunkArgs
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
         if (t0 + i < n) s += g[i];
-        Ls[(t0 + i + 1) * LS + c] = s;
+        Ls[(t0 + i + 1) * LS + c] = s * LOG2E;
       }
     }
     a.shrink[((size_t)blockIdx.y * a.H + h) * Np + c] = expf(s);
@@ -371,7 +374,7 @@ __global__ __launch_bounds__(256) void delta_solve_channel_kernel(DeltaChunkArgs
       qk[jt] = MFMA(qm.z, b.z, qk[jt]), qk[jt] = MFMA(qm.w, b.w, qk[jt]);
     }
   }
-  if (wave_max(fall) > FAR_APART) {  // (the whole wave) pair by pair: four rows of this lane's column
+  if (wave_max(fall) > FAR_APART * LOG2E) {  // (the whole wave) pair by pair: four rows of this lane's column
     const float* kj = kb + (size_t)min(t_row, n - 1) * ldk;
     const float* lj = Ls + (t_row + 1) * LS;
     const float* kt[4];
@@ -387,7 +390,7 @@ __global__ __launch_bounds__(256) void delta_solve_channel_kernel(DeltaChunkArgs
       const float kv = kj[c], lv = lj[c];
 #pragma unroll
       for (int x = 0; x < 4; ++x) {
-        const float e = kv * expf(fminf(ltp[x][c] - lv, 0.f));
+        const float e = kv * exp_2(fminf(ltp[x][c] - lv, 0.f));
         sk[x] += kt[x][c] * e, sq[x] += qt[x][c] * e;
       }
     }
@@ -428,8 +431,8 @@ __global__ __launch_bounds__(256) void delta_solve_channel_kernel(DeltaChunkArgs
 #pragma unroll
       for (int s = 0; s < 16; ++s) {
         const int t = 4 * s + lg;
-        const float l = lc[(t + 1) * LS], down = expf(l);
-        if (t < n) a.k_end[(row0 + t) * ldh + col] = b[s] * expf(end - l), a.q_hat[(row0 + t) * ldh + col] = q[s] * down;
+        const float l = lc[(t + 1) * LS], down = exp_2(l);
+        if (t < n) a.k_end[(row0 + t) * ldh + col] = b[s] * exp_2(end - l), a.q_hat[(row0 + t) * ldh + col] = q[s] * down;
         b[s] *= bt[t] * down;  // (bt is zero from n on)
       }
     } else {

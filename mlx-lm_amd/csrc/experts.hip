@@ -58,46 +58,49 @@ struct RouteArgs {
 #define ROUTER_PER_LANE 8
 
 // The largest of c over the wave and the lowest index that holds it.
-__device__ __forceinline__ int wave_argmax(const float (&c)[ROUTER_PER_LANE], int lane, float* value) {
+template <int PL>
+__device__ __forceinline__ int wave_argmax(const float (&c)[PL], int lane, float* value) {
   float best = -INFINITY;
 #pragma unroll
-  for (int i = 0; i < ROUTER_PER_LANE; ++i) best = fmaxf(best, c[i]);
+  for (int i = 0; i < PL; ++i) best = fmaxf(best, c[i]);
   best = wave_max(best);
   float first = -1e9f;  // minus the lowest index that holds the best score (indices are exact in a float)
 #pragma unroll
-  for (int i = ROUTER_PER_LANE - 1; i >= 0; --i)
+  for (int i = PL - 1; i >= 0; --i)
     if (c[i] == best) first = -(float)(lane + 64 * i);
   *value = best;
   return (int)(-wave_max(first));
 }
 
 // Choice scores outside the best groups become minus infinity.
-__device__ __forceinline__ void limit_groups(float (&c)[ROUTER_PER_LANE], int n_out, int groups, int keep, int lane) {
+template <int PL>
+__device__ __forceinline__ void limit_groups(float (&c)[PL], int n_out, int groups, int keep, int lane) {
   const int size = n_out / groups;
-  float score[ROUTER_PER_LANE];  // group lane + 64 i
+  int group[PL];  // of output lane + 64 i
 #pragma unroll
-  for (int i = 0; i < ROUTER_PER_LANE; ++i) score[i] = -INFINITY;
+  for (int i = 0; i < PL; ++i) group[i] = lane + 64 * i < n_out ? (lane + 64 * i) / size : -1;
+  float score[PL];  // group lane + 64 i
+#pragma unroll
+  for (int i = 0; i < PL; ++i) score[i] = -INFINITY;
   for (int g = 0; g < groups; ++g) {
     float m1 = -INFINITY;
 #pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i) {
-      const int e = lane + 64 * i;
-      if (e / size == g && e < n_out) m1 = fmaxf(m1, c[i]);
+    for (int i = 0; i < PL; ++i) {
+      if (group[i] == g) m1 = fmaxf(m1, c[i]);
     }
     m1 = wave_max(m1);
     float m2 = -INFINITY;
     int equal = 0;
 #pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i) {
-      const int e = lane + 64 * i;
-      const bool in = e / size == g && e < n_out;
+    for (int i = 0; i < PL; ++i) {
+      const bool in = group[i] == g;
       equal += __popcll(__ballot(in && c[i] == m1));
       if (in && c[i] != m1) m2 = fmaxf(m2, c[i]);
     }
     m2 = equal > 1 ? m1 : wave_max(m2);
     const float total = size > 1 ? m1 + m2 : m1;
 #pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i)
+    for (int i = 0; i < PL; ++i)
       if (lane + 64 * i == g) score[i] = total;
   }
   unsigned kept = 0u;  // a bit an output of this lane
@@ -105,58 +108,59 @@ __device__ __forceinline__ void limit_groups(float (&c)[ROUTER_PER_LANE], int n_
     float best;
     const int g = wave_argmax(score, lane, &best);
 #pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i) {
+    for (int i = 0; i < PL; ++i) {
       if (lane + 64 * i == g) score[i] = -INFINITY;
-      if ((lane + 64 * i) / size == g) kept |= 1u << i;
+      if (group[i] == g) kept |= 1u << i;
     }
   }
 #pragma unroll
-  for (int i = 0; i < ROUTER_PER_LANE; ++i)
+  for (int i = 0; i < PL; ++i)
     if (!(kept >> i & 1u)) c[i] = -INFINITY;
 }
 
-__device__ __forceinline__ void route_token(const float* __restrict__ zr, const RouteArgs& a, int top, int* __restrict__ idx,
+template <int PL>
+__device__ __forceinline__ void route_outputs(const float* __restrict__ zr, const RouteArgs& a, int top, int* __restrict__ idx,
                                             float* __restrict__ weight, int lane) {
   const int n_out = a.n_out;
-  float v[ROUTER_PER_LANE], c[ROUTER_PER_LANE];
+  float v[PL], c[PL];
   float m = -INFINITY;
 #pragma unroll
-  for (int i = 0; i < ROUTER_PER_LANE; ++i) {
+  for (int i = 0; i < PL; ++i) {
     const int e = lane + 64 * i;
     v[i] = e < n_out ? zr[e] : -INFINITY;
     m = fmaxf(m, v[i]);
   }
   if (a.sigmoid) {
 #pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i) v[i] = 1.0f / (1.0f + expf(-v[i]));
+    for (int i = 0; i < PL; ++i) v[i] = 1.0f / (1.0f + expf(-v[i]));
   } else {
     m = wave_max(m);
     float sum = 0.f;
 #pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i) {
+    for (int i = 0; i < PL; ++i) {
       v[i] = lane + 64 * i < n_out ? expf(v[i] - m) : 0.f;
       sum += v[i];
     }
     const float inv = 1.0f / wave_sum(sum);
 #pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i) v[i] *= inv;
+    for (int i = 0; i < PL; ++i) v[i] *= inv;
   }
 #pragma unroll
-  for (int i = 0; i < ROUTER_PER_LANE; ++i) {
+  for (int i = 0; i < PL; ++i) {
     const int e = lane + 64 * i;
     c[i] = e < n_out ? (a.correction ? v[i] + a.correction[e] : v[i]) : -INFINITY;
   }
   if (a.groups > 1) limit_groups(c, n_out, a.groups, a.keep, lane);
-  float mine[ROUTER_PER_LANE];  // pick j's weight, kept by lane j % 64 until the picks' sum is known
+  float mine[PL];  // pick j's weight, kept by lane j % 64 until the picks' sum is known
 #pragma unroll
-  for (int i = 0; i < ROUTER_PER_LANE; ++i) mine[i] = 0.f;
+  for (int i = 0; i < PL; ++i) mine[i] = 0.f;
   float total = 0.f;
   for (int j = 0; j < top; ++j) {
     float best;
     const int e = wave_argmax(c, lane, &best);
     float w = 0.f;
 #pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i)
+    for (int i = 0; i < PL; ++i)
       if (lane + 64 * i == e) {
         idx[j] = e, w = v[i];
         c[i] = -INFINITY;  // picked
@@ -164,13 +168,20 @@ __device__ __forceinline__ void route_token(const float* __restrict__ zr, const 
     w = wave_sum(w);  // (one lane holds it)
     total += w;
 #pragma unroll
-    for (int i = 0; i < ROUTER_PER_LANE; ++i)
+    for (int i = 0; i < PL; ++i)
       if (lane == (j & 63) && i == (j >> 6)) mine[i] = w;
   }
   const float factor = a.renorm ? a.mult / (total + 1e-20f) : a.mult;
 #pragma unroll
-  for (int i = 0; i < ROUTER_PER_LANE; ++i)
+  for (int i = 0; i < PL; ++i)
     if (lane + 64 * i < top) weight[lane + 64 * i] = mine[i] * factor;
+}
+
+// (up to 64 outputs: one a lane)
+__device__ __forceinline__ void route_token(const float* __restrict__ zr, const RouteArgs& a, int top, int* __restrict__ idx,
+                                            float* __restrict__ weight, int lane) {
+  if (a.n_out <= 64) route_outputs<1>(zr, a, top, idx, weight, lane);
+  else route_outputs<ROUTER_PER_LANE>(zr, a, top, idx, weight, lane);
 }
 
 __global__ __launch_bounds__(256) void router_choice_kernel(RouteArgs a, int n_tokens, int top, int* __restrict__ idx,

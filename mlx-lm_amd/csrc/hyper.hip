@@ -9,10 +9,13 @@
 //                  with y: the write;  xs_out (may be xs itself): the new streams
 //                  u = sum_s in[s] x_s (in null: the plain sum)
 //                  norm_out = LayerNorm(u) * gamma + beta, and/or sum_out = u
+//                  rows_out = W norm_out for a small matrix W (a router's): a step of few tokens saves the
+//                  launch that this product would be
 // All 32-bit; only norm_out may be bfloat16.
 #include "common.h"
 
 #define MAX_STREAMS 8
+#define MAX_ROWS 128  // of the small matrix
 
 struct HyperArgs {
   const float* xs;
@@ -34,12 +37,51 @@ struct HyperArgs {
   float* sum_out;
   int ld_sum;
   int T, D, S;
+  const void* w;  // [n_rows][D] of norm_out's dtype, or null
+  float* rows_out;  // [T, n_rows]
+  int n_rows;
 };
+
+__device__ __forceinline__ f32x4_t four(const bf16* p) {
+  const uint2 v = *(const uint2*)p;
+  return f32x4_t{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16), __uint_as_float(v.y & 0xffff0000u)};
+}
+__device__ __forceinline__ f32x4_t four(const float* p) { return *(const f32x4_t*)p; }
+
+// rows_out[t] = W u for the normed row that the block's threads hold (u[i]: columns 4 (tid + TH i) ..)
+template <typename T, int NV, int TH>
+__device__ __forceinline__ void small_rows(const HyperArgs& a, int t, const f32x4_t (&u)[NV], float (*part)[MAX_ROWS]) {
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const T* w = (const T*)a.w;
+  for (int e0 = 0; e0 < a.n_rows; e0 += 8) {
+    f32x4_t wv[8][NV];
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+#pragma unroll
+      for (int i = 0; i < NV; ++i) wv[e][i] = four(w + (size_t)min(e0 + e, a.n_rows - 1) * a.D + min(4 * (tid + TH * i), a.D - 4));
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float s = 0.f;
+#pragma unroll
+      for (int i = 0; i < NV; ++i)
+        if (4 * (tid + TH * i) < a.D) s += (wv[e][i][0] * u[i][0] + wv[e][i][1] * u[i][1]) + (wv[e][i][2] * u[i][2] + wv[e][i][3] * u[i][3]);
+      s = wave_sum(s);
+      if (lane == 0 && e0 + e < a.n_rows) part[wave][e0 + e] = s;
+    }
+  }
+  __syncthreads();
+  for (int e = tid; e < a.n_rows; e += TH) {
+    float s = 0.f;
+    for (int i = 0; i < TH / 64; ++i) s += part[i][e];
+    a.rows_out[(size_t)t * a.n_rows + e] = s;
+  }
+}
 
 // NV: pieces of four columns a thread, TH threads
 template <int S, int NV, int TH>
 __global__ __launch_bounds__(TH) void hyper_step_kernel(HyperArgs a) {
   __shared__ float red[20];
+  __shared__ float part[TH / 64][MAX_ROWS];
   const int t = blockIdx.x, tid = threadIdx.x, D = a.D;
   float mix[S][S], wo[S], wi[S];
 #pragma unroll
@@ -114,11 +156,18 @@ __global__ __launch_bounds__(TH) void hyper_step_kernel(HyperArgs a) {
     f32x4_t v = u[i] * rstd;
     if (a.gamma) v *= *(const f32x4_t*)(a.gamma + c);
     if (a.beta) v += *(const f32x4_t*)(a.beta + c);
-    if (a.norm_dtype == DT_BF16)
-      *(uint2*)((bf16*)a.norm_out + (size_t)t * D + c) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
-    else
+    if (a.norm_dtype == DT_BF16) {
+      const uint2 b = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
+      *(uint2*)((bf16*)a.norm_out + (size_t)t * D + c) = b;
+      u[i] = four((const bf16*)&b);  // (the product takes the row as it is written)
+    } else {
       *(f32x4_t*)((float*)a.norm_out + (size_t)t * D + c) = v;
+      u[i] = v;
+    }
   }
+  if (!a.w) return;
+  if (a.norm_dtype == DT_BF16) small_rows<bf16, NV, TH>(a, t, u, part);
+  else small_rows<float, NV, TH>(a, t, u, part);
 }
 
 DEFINE_LAST_ERROR(mlxlm_last_error)
@@ -144,6 +193,8 @@ extern "C" int hyper_step(const HyperArgs* args, hipStream_t stream) {
   if (a.y && (!a.mix || !a.out || a.n_parts < 1 || a.ldy < a.D || a.ldy % 4 || a.y_part % 4)) FAIL("hyper_step: a write needs its weights and whole rows");
   if (a.sum_out && (a.ld_sum < a.D || a.ld_sum % 4)) FAIL("hyper_step: the sum's row stride %d", a.ld_sum);
   if (a.norm_out && a.norm_dtype != DT_F32 && a.norm_dtype != DT_BF16) FAIL("hyper_step: unknown dtype code %d", a.norm_dtype);
+  if (a.w && (!a.norm_out || !a.rows_out || a.n_rows <= 0 || a.n_rows > MAX_ROWS || ((uintptr_t)a.w & 15)))
+    FAIL("hyper_step: a product of %d rows (1 to %d) with the norm", a.n_rows, MAX_ROWS);
   if (((uintptr_t)a.xs | (uintptr_t)a.first | (uintptr_t)a.xs_out | (uintptr_t)a.y | (uintptr_t)a.norm_out | (uintptr_t)a.sum_out |
        (uintptr_t)a.gamma | (uintptr_t)a.beta | (uintptr_t)a.bias) & 15)
     FAIL("hyper_step: 16-byte aligned rows");

@@ -7,7 +7,7 @@
 // state row as a ring, position p in row p % taps: a step's rows are none of those it still reads, so
 // blocks that need the same inputs run side by side.
 //
-//   rglru_gates  portions: a block a (64 tokens of a request, part): the convolution into LDS, both gates on
+//   rglru_gates  portions: a block a (64 tokens of a request, 64 channels of a part): the convolution into LDS, both gates on
 //                the matrix cores, a and sqrt(1 - a^2) i u as rows, and what the 64 tokens do to the
 //                state (S -> A S + B a channel), each lane's tokens composed, then lanes, then waves
 //   rglru_scan   a thread a channel of 64 tokens: the state ahead of them from the A, B of the request's
@@ -71,6 +71,32 @@ __device__ __forceinline__ float conv_at(const RglruArgs& p, const float* ring, 
   return acc + (p.conv_b ? p.conv_b[c] : 0.f);
 }
 
+// The same for CONV_TILE tokens in a row of one channel, all inputs asked for at once (up to CONV_TAPS
+// taps).  `live` of the tokens exist; at or below -CONV_TAPS nothing is read.
+#define CONV_TAPS 8
+#define CONV_TILE 8
+__device__ __forceinline__ void conv_run(const RglruArgs& p, const float* ring, int row, int local, int pos, int live, int c, float* out, int ld) {
+  float w[CONV_TAPS], in[CONV_TILE + CONV_TAPS - 1];
+#pragma unroll
+  for (int j = 0; j < CONV_TAPS; ++j) w[j] = j < p.taps ? p.conv_w[(size_t)c * p.taps + p.taps - 1 - j] : 0.f;  // (of the input j tokens back)
+#pragma unroll
+  for (int i = 0; i < CONV_TILE + CONV_TAPS - 1; ++i) {
+    const int d = i - (CONV_TAPS - 1);  // tokens from the first of the run
+    in[i] = 0.f;
+    if (d >= live || -d >= p.taps) continue;
+    if (local + d >= 0) in[i] = p.x[(size_t)(row + d) * p.ldx + c];
+    else if (pos + d >= 0) in[i] = ring[(size_t)((pos + d) % p.taps) * p.W + c];
+  }
+  const float shift = p.conv_b ? p.conv_b[c] : 0.f;
+#pragma unroll
+  for (int t = 0; t < CONV_TILE; ++t) {
+    float acc = 0.f;
+#pragma unroll
+    for (int j = CONV_TAPS - 1; j >= 0; --j) acc += w[j] * in[t + CONV_TAPS - 1 - j];  // the oldest input first
+    out[t * ld] = t < live ? acc + shift : 0.f;
+  }
+}
+
 struct Gated {
   float a, b;
 };
@@ -80,93 +106,91 @@ __device__ __forceinline__ Gated gated(float zr, float zi, float u, float rate) 
 }
 
 // TT: tokens in LDS at a time (64, or 16 for wide parts); four waves: TT / 16 tiles of rows, the
-// remaining factor over the columns.
+// remaining factor over the block's 64 channels (every block makes the whole part's convolution).
 template <typename T, int TT>
 __global__ __launch_bounds__(256) void rglru_gates_kernel(RglruArgs p) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  constexpr int RT = TT / 16, CW = 4 / RT;
+  __shared__ float2 does[4][64];
+  constexpr int RT = TT / 16, NJ = RT == 4 ? 4 : 1;  // NJ: tiles of sixteen channels a wave
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lg = lane >> 4;
-  const int rt = wave % RT, cw = wave / RT;
+  const int rt = RT == 4 ? wave : 0, j0 = RT == 4 ? 0 : wave;
   const int w = p.w, wp = p.wp, ld = wp + 4;
-  float* U = lds;                            // [TT][ld]
-  float2* does = (float2*)(U + TT * ld);     // [RT][wp16]
-  const int w16 = (w + 15) & ~15;
-  const int span = blockIdx.x, part = blockIdx.y, c0 = part * w;
+  float* U = lds;  // [TT][ld]
+  const int slices = (w + 63) / 64, span = blockIdx.x, part = blockIdx.y / slices, s0 = blockIdx.y % slices * 64, c0 = part * w;
   const int r = p.span_req[span], lo = p.span_start[span], n = min(SPAN, p.seq_len[r] - lo);
   const int row0 = p.seq_start[r] + lo, pos0 = p.positions[row0];
   const float* srow = p.state + (size_t)p.slot_ids[r] * p.state_stride;
   const float* ring = srow + p.ring_offset;
-  if (lo == 0)
-    for (int c = tid; c < w; c += 256) p.s0[(size_t)r * p.W + c0 + c] = srow[p.state_offset + c0 + c];
-  const T* Ra = (const T*)p.ra + (size_t)part * w * wp;
-  const T* Ri = (const T*)p.ri + (size_t)part * w * wp;
+  if (lo == 0 && tid < 64 && s0 + tid < w) p.s0[(size_t)r * p.W + c0 + s0 + tid] = srow[p.state_offset + c0 + s0 + tid];
+  const T* gate[2 * NJ];
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) {
+    const size_t f = (size_t)(part * w + min(s0 + 16 * (j0 + j) + lr, w - 1)) * wp;
+    gate[j] = (const T*)p.ra + f, gate[NJ + j] = (const T*)p.ri + f;
+  }
+  const bool run = p.taps <= CONV_TAPS;
   for (int t0 = 0; t0 < n; t0 += TT) {
     if (t0 > 0) __syncthreads();  // the tile before is done with U
-    for (int e = tid; e < TT * wp; e += 256) {
-      const int t = e / wp, c = e - t * wp;
-      U[t * ld + c] = c < w && t0 + t < n ? conv_at(p, ring, row0 + t0 + t, lo + t0 + t, pos0 + t0 + t, c0 + c) : 0.f;
+    if (run) {
+      for (int e = tid; e < TT / CONV_TILE * wp; e += 256) {
+        const int t = e / wp * CONV_TILE, c = e % wp, first = t0 + t;
+        conv_run(p, ring, row0 + first, lo + first, pos0 + first, c < w ? n - first : -CONV_TAPS, c0 + min(c, w - 1), U + t * ld + c, ld);
+      }
+    } else {
+      for (int e = tid; e < TT * wp; e += 256) {
+        const int t = e / wp, c = e - t * wp;
+        U[t * ld + c] = c < w && t0 + t < n ? conv_at(p, ring, row0 + t0 + t, lo + t0 + t, pos0 + t0 + t, c0 + c) : 0.f;
+      }
     }
     __syncthreads();
     const float* urow = U + (16 * rt + lr) * ld;
-    auto row = [&](int k) { return *(const float4*)(urow + k); };
-    for (int ct = 4 * cw; 16 * ct < w; ct += 4 * CW) {  // four tiles of sixteen channels at a time
-      const T* wr[4];
-      const T* wi[4];
+    f32x4_t z[2 * NJ];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int f = min(16 * (ct + j) + lr, w - 1);
-        wr[j] = Ra + (size_t)f * wp, wi[j] = Ri + (size_t)f * wp;
+    for (int j = 0; j < 2 * NJ; ++j) z[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    rows_product<2 * NJ>([&](int k) { return *(const float4*)(urow + k); }, gate, wp, 0, 1, z);
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+      const int sc = 16 * (j0 + j) + lr, cc = s0 + sc;
+      const bool live = cc < w;
+      const int c = c0 + min(cc, w - 1);
+      const float rb = p.ra_b[c], ib = p.ri_b[c], rate = p.decay * softplus_f(p.lam[c]);
+      float A = 1.f, Bv = 0.f;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        const int t = 16 * rt + 4 * lg + x;
+        if (t0 + t < n && live) {
+          const Gated g = gated(z[j][x] + rb, z[NJ + j][x] + ib, U[t * ld + cc], rate);
+          const size_t at = (size_t)(row0 + t0 + t) * p.W + c;
+          p.a[at] = g.a, p.b[at] = g.b;
+          Bv = g.a * Bv + g.b, A *= g.a;
+        }
       }
-      f32x4_t zr[4], zi[4];
+      // lanes of the same channel, sixteen apart, hold four tokens each, in order
 #pragma unroll
-      for (int j = 0; j < 4; ++j) zr[j] = zi[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-      rows_product<4>(row, wr, wp, 0, 1, zr);
-      rows_product<4>(row, wi, wp, 0, 1, zi);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int cc = 16 * (ct + j) + lr;
-        if (16 * (ct + j) >= w) continue;  // (the same for the whole wave)
-        const bool live = cc < w;
-        const int c = c0 + min(cc, w - 1);
-        const float rb = p.ra_b[c], ib = p.ri_b[c], rate = p.decay * softplus_f(p.lam[c]);
-        float A = 1.f, Bv = 0.f;
-#pragma unroll
-        for (int x = 0; x < 4; ++x) {
-          const int t = 16 * rt + 4 * lg + x;
-          if (t0 + t < n && live) {
-            const Gated g = gated(zr[j][x] + rb, zi[j][x] + ib, U[t * ld + cc], rate);
-            const size_t at = (size_t)(row0 + t0 + t) * p.W + c;
-            p.a[at] = g.a, p.b[at] = g.b;
-            Bv = g.a * Bv + g.b, A *= g.a;
-          }
-        }
-        // lanes of the same channel, sixteen apart, hold four tokens each, in order
-#pragma unroll
-        for (int step = 16; step < 64; step *= 2) {
-          const float A2 = __shfl_xor(A, step, 64), B2 = __shfl_xor(Bv, step, 64);
-          const bool later = lane & step;
-          Bv = later ? A * B2 + Bv : A2 * Bv + B2;
-          A *= A2;
-        }
-        if (lg == 0) {
-          float2* at = does + rt * w16 + cc;
-          if (TT < SPAN && t0 > 0)
-            *at = make_float2(at->x * A, A * at->y + Bv);  // (RT == 1: this tile's tokens follow the last one's)
-          else
-            *at = make_float2(A, Bv);
-        }
+      for (int step = 16; step < 64; step *= 2) {
+        const float A2 = __shfl_xor(A, step, 64), B2 = __shfl_xor(Bv, step, 64);
+        const bool later = lane & step;
+        Bv = later ? A * B2 + Bv : A2 * Bv + B2;
+        A *= A2;
+      }
+      if (lg == 0) {
+        float2* at = &does[rt][sc];
+        if (TT < SPAN && t0 > 0)
+          *at = make_float2(at->x * A, A * at->y + Bv);  // (RT == 1: this tile's tokens follow the last one's)
+        else
+          *at = make_float2(A, Bv);
       }
     }
   }
   __syncthreads();
-  for (int c = tid; c < w; c += 256) {
+  if (tid < 64 && s0 + tid < w) {
     float A = 1.f, Bv = 0.f;
 #pragma unroll
     for (int i = 0; i < RT; ++i) {
-      const float2 d = does[i * w16 + c];
+      const float2 d = does[i][tid];
       Bv = d.x * Bv + d.y, A *= d.x;
     }
-    p.does[(size_t)span * p.W + c0 + c] = make_float2(A, Bv);
+    p.does[(size_t)span * p.W + c0 + s0 + tid] = make_float2(A, Bv);
   }
 }
 
@@ -229,17 +253,37 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs p) {
   float* srow = p.state + (size_t)p.slot_ids[req] * p.state_stride;
   const float S = srow[p.state_offset + c], y = p.y[(size_t)erow * p.ldx + c], x = p.x[(size_t)erow * p.ldx + c];
   const float rb = p.ra_b[c], ib = p.ri_b[c], lam = p.lam[c];
+  const size_t f = (size_t)(b * w + min(f0 + lr, w - 1)) * wp;
+  const T* const gates[2] = {(const T*)p.ra + f, (const T*)p.ri + f};
+  const bool run = p.taps <= CONV_TAPS;
   for (int e = tid; e < n * wp; e += 256) {
-    const int t = e / wp, k = e - t * wp, row = p.seq_start[r0 + t];
+    const int t = e / wp, k = e - t * wp, row = p.seq_start[r0 + t], pos = p.positions[row];
     const float* ring = p.state + (size_t)p.slot_ids[r0 + t] * p.state_stride + p.ring_offset;
-    U[t * ld + k] = k < w ? conv_at(p, ring, row, 0, p.positions[row], c0 + k) : 0.f;
+    const int ch = c0 + min(k, w - 1);
+    float u;
+    if (run) {  // all inputs asked for at once
+      float in[CONV_TAPS], cw[CONV_TAPS];
+#pragma unroll
+      for (int j = 0; j < CONV_TAPS; ++j) {
+        in[j] = cw[j] = 0.f;
+        if (j >= p.taps) continue;
+        cw[j] = p.conv_w[(size_t)ch * p.taps + p.taps - 1 - j];
+        in[j] = j == 0 ? p.x[(size_t)row * p.ldx + ch] : ring[(size_t)((pos + p.taps - j) % p.taps) * p.W + ch];
+      }
+      u = p.conv_b ? p.conv_b[ch] : 0.f;
+      float acc = 0.f;
+#pragma unroll
+      for (int j = CONV_TAPS - 1; j >= 0; --j) acc += pos - j >= 0 ? cw[j] * in[j] : 0.f;
+      u += acc;
+    } else {
+      u = conv_at(p, ring, row, 0, pos, ch);
+    }
+    U[t * ld + k] = k < w ? u : 0.f;
   }
   for (int e = n * ld + tid; e < 16 * ld; e += 256) U[e] = 0.f;
   __syncthreads();
   const float* urow = U + lr * ld;
   auto row = [&](int k) { return *(const float4*)(urow + k); };
-  const size_t f = (size_t)(b * w + min(f0 + lr, w - 1)) * wp;
-  const T* const gates[2] = {(const T*)p.ra + f, (const T*)p.ri + f};
   f32x4_t z[2] = {f32x4_t{0.f, 0.f, 0.f, 0.f}, f32x4_t{0.f, 0.f, 0.f, 0.f}};
   rows_product<2>(row, gates, wp, wave, 4, z);
 #pragma unroll
@@ -260,7 +304,8 @@ DEFINE_LAST_ERROR(mlxlm_last_error)
 
 #define LDS_MOST (150 * 1024)
 static size_t gates_lds(int tt, int w, int wp) {
-  return ((size_t)tt * (wp + 4) + 2 * (size_t)(tt / 16) * ((w + 15) / 16 * 16)) * sizeof(float);
+  (void)w;
+  return (size_t)tt * (wp + 4) * sizeof(float);
 }
 
 // 1 if the kernels take parts of w channels
@@ -314,7 +359,7 @@ extern "C" int rglru_portions(const RglruArgs* args, hipStream_t stream) {
     raised = true;
   }
   const bool wide = gates_lds(64, a.w, a.wp) > 80 * 1024;  // (two blocks a CU)
-  const dim3 grid(a.n_spans, a.B), scan(a.n_spans, (a.W + 255) / 256), block(256);
+  const dim3 grid(a.n_spans, a.B * ((a.w + 63) / 64)), scan(a.n_spans, (a.W + 255) / 256), block(256);
   const size_t lds = gates_lds(wide ? 16 : 64, a.w, a.wp);
   if (a.dtype == DT_F32) {
     if (wide) hipLaunchKernelGGL((rglru_gates_kernel<float, 16>), grid, block, lds, stream, a);

@@ -144,6 +144,48 @@ __device__ __forceinline__ float lowrank_row(const float* __restrict__ w, const 
   }
   return group_sum<16>(s);
 }
+// Up to AHEAD rows a lane group of the two narrow matrices (bfloat16, middles of up to 128 columns), asked
+// for before the middles are known.
+#define AHEAD 8
+__device__ __forceinline__ bool fits_ahead(const StepArgs& a, int threads) {
+  return a.w2_dtype == DT_BF16 && a.rank <= 128 && (!a.y || a.g_rank <= 128) && a.N + (a.y ? a.P : 0) <= AHEAD * (threads / 16);
+}
+template <int TH>
+__device__ __forceinline__ void ask_rows(const StepArgs& a, int h, u32x4_t (&w)[AHEAD]) {
+  const int k = 8 * (threadIdx.x & 15), total = a.N + (a.y ? a.P : 0);
+  const bf16* a2 = (const bf16*)a.a2 + (size_t)h * a.N * a.rank;
+  const bf16* g2 = (const bf16*)a.g2 + (size_t)h * a.P * a.g_rank;
+#pragma unroll
+  for (int i = 0; i < AHEAD; ++i) {
+    const int c = threadIdx.x / 16 + i * (TH / 16);
+    w[i] = u32x4_t{0u, 0u, 0u, 0u};
+    if (c < a.N) {
+      if (k < a.rank) w[i] = *(const u32x4_t*)(a2 + (size_t)c * a.rank + k);
+    } else if (c < total && k < a.g_rank) {
+      w[i] = *(const u32x4_t*)(g2 + (size_t)(c - a.N) * a.g_rank + k);
+    }
+  }
+}
+template <int TH>
+__device__ __forceinline__ void rows_asked(const StepArgs& a, const u32x4_t (&w)[AHEAD], const float* tz, const float* my, float* ds, float* gs) {
+  const int l16 = threadIdx.x & 15, k = 8 * l16, total = a.N + (a.y ? a.P : 0);
+  float z[8], y[8];
+#pragma unroll
+  for (int j = 0; j < 8; ++j) z[j] = k < a.rank ? tz[k + j] : 0.f, y[j] = a.y && k < a.g_rank ? my[k + j] : 0.f;
+#pragma unroll
+  for (int i = 0; i < AHEAD; ++i) {
+    const int c = threadIdx.x / 16 + i * (TH / 16);
+    if (c >= total) continue;  // (the same for sixteen lanes)
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      s += __uint_as_float(w[i][j] << 16) * (c < a.N ? z[2 * j] : y[2 * j]);
+      s += __uint_as_float(w[i][j] & 0xffff0000u) * (c < a.N ? z[2 * j + 1] : y[2 * j + 1]);
+    }
+    s = group_sum<16>(s);
+    if (l16 == 0) (c < a.N ? ds[c] : gs[c - a.N]) = s;
+  }
+}
 // The decays' logits into ds and the gate's into gs, for head h.
 template <typename T, int TH>
 __device__ __forceinline__ void lowrank_rows(const StepArgs& a, int h, const float* tz, const float* ty, float* ds, float* gs) {
@@ -187,6 +229,13 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
 #pragma unroll
   for (int r = 0; r < R; ++r) S[r] = Cols<V>::load(Sg + (size_t)min(ty + TY * r, N - 1) * P + tx * V);
 
+  u32x4_t narrow[AHEAD];
+  bool ahead = false;
+  if constexpr (MODE == STEP_CHANNEL_RAW && TH <= 512) {
+    ahead = fits_ahead(a, TH);
+    if (ahead) ask_rows<TH>(a, h, narrow);
+  }
+
   for (int t = 0; t < n; ++t) {
     const size_t row = (size_t)(start + t);
     float gv = a.gate && tid < P ? a.gate[row * a.ldg + (size_t)h * P + tid] : 0.f;
@@ -222,7 +271,8 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
         g = expf(-expf(a.A_log[h]) * softplus_f(a.log_g[row * a.ld_gb + h] + a.dt_bias[h]));
       } else {
         __syncthreads();
-        if (a.w2_dtype == DT_BF16) lowrank_rows<bf16, TH>(a, h, tz, my, ds, gs);
+        if (TH <= 512 && ahead) rows_asked<TH>(a, narrow, tz, my, ds, gs);
+        else if (a.w2_dtype == DT_BF16) lowrank_rows<bf16, TH>(a, h, tz, my, ds, gs);
         else lowrank_rows<float, TH>(a, h, tz, my, ds, gs);
         __syncthreads();
         const float rate = expf(a.A_log[h]);

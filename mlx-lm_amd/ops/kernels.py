@@ -2085,10 +2085,11 @@ class HyperArgs(ctypes.Structure):
     _fields_ = [("xs", _vp), ("first", _vp), ("ld_first", _c_int), ("xs_out", _vp), ("y", _vp), ("ldy", _c_int), ("n_parts", _c_int),
                 ("y_part", _c_size_t), ("bias", _vp), ("mix", _vp), ("out", _vp), ("in_", _vp), ("gamma", _vp), ("beta", _vp),
                 ("eps", _c_float), ("norm_out", _vp), ("norm_dtype", _c_int), ("sum_out", _vp), ("ld_sum", _c_int), ("T", _c_int),
-                ("D", _c_int), ("S", _c_int)]
+                ("D", _c_int), ("S", _c_int), ("w", _vp), ("rows_out", _vp), ("n_rows", _c_int)]
 
 
 HYPER_MAX_STREAMS, HYPER_MAX_WIDTH = 8, 32768
+HYPER_MAX_ROWS = 128  # of the small matrix whose product with the norm rides along
 
 
 class HyperWrite:
@@ -2100,11 +2101,12 @@ class HyperWrite:
 
 
 def hyper_step(n_streams, width, xs=None, first=None, xs_out=None, write=None, read=None, norm_out=None, gamma=None, beta=None, eps=0.0,
-               sum_out=None):
+               sum_out=None, rows=None):
     """One pass over the streams ``xs`` (float32 ``[tokens, streams, width]``; all of them are ``first``, ``[tokens,
     width]``, where ``xs`` is None): ``write`` (a ``HyperWrite``) first, the new streams into ``xs_out`` (may be
     ``xs``), then ``u = sum_s read[s] x_s`` (``read`` None: the plain sum), its LayerNorm into ``norm_out`` and ``u``
-    itself into ``sum_out``."""
+    itself into ``sum_out``.  ``rows = (w, out)``: the norm's product with a small matrix ``w`` ``[n, width]`` of its dtype into
+    float32 ``out`` ``[tokens, n]``."""
     lib = build.load("hyper")
     a = HyperArgs()
     src = xs if xs is not None else first
@@ -2139,6 +2141,12 @@ def hyper_step(n_streams, width, xs=None, first=None, xs_out=None, write=None, r
     if sum_out is not None:
         _need(sum_out.shape[0] >= T, "hyper_step: sum_out")
         a.ld_sum, a.sum_out = _f32_rows(sum_out, "sum_out", width), sum_out.data_ptr()
+    if rows is not None:
+        w, out = rows
+        _dev(w, "w", norm_out.dtype)
+        _dev(out, "rows", torch.float32)
+        _need(w.dim() == 2 and w.shape[1] == width and w.is_contiguous() and tuple(out.shape) == (T, w.shape[0]) and out.is_contiguous(), "hyper_step: rows")
+        a.w, a.rows_out, a.n_rows = w.data_ptr(), out.data_ptr(), w.shape[0]
     a.T, a.D, a.S = T, int(width), int(n_streams)
     rc = lib.hyper_step(ctypes.byref(a), _stream())
     build.check(lib, rc, "hyper_step")

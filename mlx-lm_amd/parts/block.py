@@ -417,12 +417,15 @@ class HyperBlock(Block):
     layer's last sublayer waits for the next run's first kernel: the runs of a step share streams and the waiting
     write through ``ctx.shared``, and the last of ``n_runs`` runs leaves the sum in ``h``.  A sublayer
     that ends with a product leaves its float32 rows, or the parts of a product that splits K, to that kernel
-    (``OutputProduct``).  All of it is 32-bit.  No counterpart in mlx_lm/models/gpt2.py, which has one stream
-    (:98-108).
+    (``OutputProduct``).  In a step of few tokens that kernel also multiplies the norm with a feed-forward's
+    router (``router_rows``) where that is small.  All of it is 32-bit.  No counterpart in
+    mlx_lm/models/gpt2.py, which has one stream (:98-108).
     """
 
     PARTS = {"mixer_norm": "norm", "mixer": "mixer", "ffn_norm": "norm", "ffn": "feed_forward"}
     OPTIONAL = ("ffn_norm", "ffn")
+    # a router of at most so many weights rides along in steps of at most so many tokens (a block reads all of it)
+    ROUTER_WEIGHTS, ROUTER_TOKENS = 1 << 17, 64
 
     def __init__(self, mixer_norm, mixer, ffn_norm=None, ffn=None, streams=1, n_runs=1, names=("hc1.", "hc2."), prefix=""):
         from ..ops import kernels
@@ -468,6 +471,8 @@ class HyperBlock(Block):
         from ..ops import kernels
 
         self.connections = [tuple(tensors[n + x].contiguous() for x in ("in", "mix", "out")) for n in self.names]
+        router = getattr(self.ffn, "router_rows", None)
+        self.router = router if router is not None and router.numel() <= self.ROUTER_WEIGHTS and router.shape[0] <= kernels.HYPER_MAX_ROWS else None
         self.pending = kernels.PendingSum()
         self.pending.c.allowed = 2
         for part in (self.mixer, self.ffn):
@@ -495,12 +500,15 @@ class HyperBlock(Block):
         mark = ctx.scratch_mark()
         u = ctx.scratch((T, D), ctx.dtype)
         for part, norm, (read, mix, out) in zip((self.mixer, self.ffn), (self.mixer_norm, self.ffn_norm), self.connections):
-            y = step["y"]
-            self._pass(ctx, h, step, keep=True, read=read, norm_out=u, gamma=norm.weight, beta=norm.bias, eps=norm.eps)
+            y, options = step["y"], {}
+            if part is self.ffn and self.router is not None and T <= self.ROUTER_TOKENS:
+                options["rows"] = ctx.scratch((T, self.router.shape[0]), torch.float32)
+            self._pass(ctx, h, step, keep=True, read=read, norm_out=u, gamma=norm.weight, beta=norm.bias, eps=norm.eps,
+                       rows=(self.router, options["rows"]) if options else None)
             if not getattr(part, "overwrite", False):
                 y.zero_()
             if part is self.ffn:
-                part.forward(ctx, u, y)
+                part.forward(ctx, u, y, **options)
             elif getattr(part, "wants_state", False):
                 part.forward(ctx, u, y, cache, writes_cache, state=state)
             else:

@@ -99,7 +99,8 @@ class GatedExperts(FeedForward):
             self.w_up = torch.stack([tensors[n(f"e{e}.up")] for e in range(self.n_experts)]).contiguous()
             self.w_down = torch.stack([tensors[n(f"e{e}.down")] for e in range(self.n_experts)]).contiguous()
         if not self.projection_given:
-            self.router_w = kernels.for_decode(tensors[n("router")].contiguous())
+            self.router_rows = tensors[n("router")].contiguous()  # (an arrangement may take its product along: ``rows``)
+            self.router_w = kernels.for_decode(self.router_rows)
             self.first_weight = self.router_w
         self.correction = tensors[n("correction")] if self.has_correction else None
         self.choice = dict(renormalize=self.renormalize, weight_scale=self.weight_scale, scores=self.scores, groups=self.groups)

@@ -151,7 +151,7 @@ def _spans(lens):
 @pytest.mark.parametrize("streams,width,T", [(1, 64, 3), (2, 72, 1), (3, 1028, 5), (4, 2048, 9), (5, 4100, 2), (6, 200, 4), (7, 8196, 2), (8, 24, 70)])
 def test_the_streams_written_read_and_normed_in_one_pass(streams, width, T, dtype):
     """First reads of streams that are all the same; a write of an output that lies in one piece or in
-    parts; streams updated in place; the sum at the end."""
+    parts; streams updated in place; a small matrix's product with the norm; the sum at the end."""
     from mlx_lm_amd.ops import kernels
 
     g = torch.Generator().manual_seed(width)
@@ -164,11 +164,15 @@ def test_the_streams_written_read_and_normed_in_one_pass(streams, width, T, dtyp
     dev = {k: v.cuda() for k, v in w.items()}
     xs = first.double().expand(S, T, D)
     u = torch.empty(T, D, dtype=dtype, device="cuda")
-    norm = dict(norm_out=u, gamma=dev["n"], beta=dev["n.b"], eps=1e-3, read=dev["c.in"])
+    small = rnd(1 + width % 70, D).to(dtype)
+    z = torch.empty(T, small.shape[0], device="cuda")
+    norm = dict(norm_out=u, gamma=dev["n"], beta=dev["n.b"], eps=1e-3, read=dev["c.in"], rows=(small.cuda(), z))
 
     def check():
         want = plain.layer_norm(plain.hyper_read(xs, wd, "c."), wd, "n", 1e-3)
         assert (u.double().cpu() - want).abs().max() <= tol * want.abs().max()
+        rows = u.double().cpu() @ small.double().t()  # (the row as it was written)
+        assert (z.double().cpu() - rows).abs().max() <= 2e-5 * rows.abs().max()
 
     kernels.hyper_step(S, D, first=first.cuda(), **norm)
     check()
