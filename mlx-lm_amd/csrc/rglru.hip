@@ -20,7 +20,10 @@
 #include "common.h"
 #include "rows_product.h"
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+#define LOG2E 1.4426950408889634f
+// (on the hardware's exponential and reciprocal, an ulp or two each)
+__device__ __forceinline__ float exp_f(float x) { return __builtin_amdgcn_exp2f(x * LOG2E); }
+__device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.0f + exp_f(-z)); }
 __device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 
 #define SPAN 64
@@ -79,13 +82,20 @@ __device__ __forceinline__ void conv_run(const RglruArgs& p, const float* ring, 
   float w[CONV_TAPS], in[CONV_TILE + CONV_TAPS - 1];
 #pragma unroll
   for (int j = 0; j < CONV_TAPS; ++j) w[j] = j < p.taps ? p.conv_w[(size_t)c * p.taps + p.taps - 1 - j] : 0.f;  // (of the input j tokens back)
+  if (local >= CONV_TAPS - 1 && live >= 1) {  // all of them in the step's own rows
+    const float* x = p.x + (size_t)(row - (CONV_TAPS - 1)) * p.ldx + c;
+    const int last = live - 1 + CONV_TAPS - 1;
 #pragma unroll
-  for (int i = 0; i < CONV_TILE + CONV_TAPS - 1; ++i) {
-    const int d = i - (CONV_TAPS - 1);  // tokens from the first of the run
-    in[i] = 0.f;
-    if (d >= live || -d >= p.taps) continue;
-    if (local + d >= 0) in[i] = p.x[(size_t)(row + d) * p.ldx + c];
-    else if (pos + d >= 0) in[i] = ring[(size_t)((pos + d) % p.taps) * p.W + c];
+    for (int i = 0; i < CONV_TILE + CONV_TAPS - 1; ++i) in[i] = x[(size_t)min(i, last) * p.ldx];  // (beyond the last: not used)
+  } else {
+#pragma unroll
+    for (int i = 0; i < CONV_TILE + CONV_TAPS - 1; ++i) {
+      const int d = i - (CONV_TAPS - 1);  // tokens from the first of the run
+      in[i] = 0.f;
+      if (d >= live || -d >= p.taps) continue;
+      if (local + d >= 0) in[i] = p.x[(size_t)(row + d) * p.ldx + c];
+      else if (pos + d >= 0) in[i] = ring[(size_t)((pos + d) % p.taps) * p.W + c];
+    }
   }
   const float shift = p.conv_b ? p.conv_b[c] : 0.f;
 #pragma unroll
@@ -101,8 +111,10 @@ struct Gated {
   float a, b;
 };
 __device__ __forceinline__ Gated gated(float zr, float zi, float u, float rate) {
-  const float log_a = -rate * sigmoid_f(zr);
-  return Gated{expf(log_a), sqrtf(-expm1f(2.0f * log_a)) * sigmoid_f(zi) * u};
+  const float log_a = -rate * sigmoid_f(zr), a = exp_f(log_a), t = 2.0f * log_a;
+  // 1 - a^2 = -(exp(t) - 1): near t = 0 as a series, without cancellation
+  const float series = -t * (1.0f + t * (0.5f + t * (1.0f / 6 + t * (1.0f / 24 + t * (1.0f / 120 + t * (1.0f / 720))))));
+  return Gated{a, sqrtf(t > -0.25f ? series : 1.0f - a * a) * sigmoid_f(zi) * u};
 }
 
 // TT: tokens in LDS at a time (64, or 16 for wide parts); four waves: TT / 16 tiles of rows, the
@@ -236,11 +248,33 @@ __global__ __launch_bounds__(256) void rglru_scan_kernel(RglruArgs p) {
   }
 }
 
+// The two gates' weights that a wave of rglru_step takes first, asked for before the rows are there (bfloat16).
+template <typename T>
+struct Ahead {
+  __device__ __forceinline__ void ask(const T* const (&)[2], int, int) {}
+  template <typename Rows>
+  __device__ __forceinline__ void product(Rows x, const T* const (&w)[2], int K, int wave, f32x4_t (&z)[2]) {
+    rows_product<2>(x, w, K, wave, 4, z);
+  }
+};
+template <>
+struct Ahead<bf16> {
+  PiecesAhead<2, 2> pieces;
+  __device__ __forceinline__ void ask(const bf16* const (&w)[2], int K, int wave) { pieces.ask(w, K, wave, 4); }
+  template <typename Rows>
+  __device__ __forceinline__ void product(Rows x, const bf16* const (&w)[2], int K, int wave, f32x4_t (&z)[2]) {
+    pieces.product(x, K, wave, 4, z);
+    rows_product<2>(x, w, K, wave + 4 * 2, 4, z);
+  }
+};
+
 // Block (part x 16 channels, 16 requests of one token each): four waves share K, a thread then a (request, channel).
 template <typename T>
 __global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs p) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ float part[2][4][16][17];
+  __shared__ int s_row[16], s_pos[16], s_place[16][CONV_TAPS];  // place: where in the ring the input j tokens back lies
+  __shared__ const float* s_ring[16];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lg = lane >> 4;
   const int w = p.w, wp = p.wp, ld = wp + 4, tiles = (w + 15) / 16;
   const int b = blockIdx.x / tiles, f0 = 16 * (blockIdx.x % tiles), c0 = b * w;
@@ -256,9 +290,21 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs p) {
   const size_t f = (size_t)(b * w + min(f0 + lr, w - 1)) * wp;
   const T* const gates[2] = {(const T*)p.ra + f, (const T*)p.ri + f};
   const bool run = p.taps <= CONV_TAPS;
+  Ahead<T> ahead;
+  ahead.ask(gates, wp, wave);
+  if (tid < 16 * CONV_TAPS) {
+    const int t = tid / CONV_TAPS, j = tid % CONV_TAPS;
+    if (t < n) {
+      const int row = p.seq_start[r0 + t], pos = p.positions[row];
+      s_place[t][j] = j < p.taps ? (pos + p.taps - j) % p.taps : 0;
+      if (j == 0) s_row[t] = row, s_pos[t] = pos, s_ring[t] = p.state + (size_t)p.slot_ids[r0 + t] * p.state_stride + p.ring_offset;
+    }
+  }
+  __syncthreads();
+#pragma unroll 2
   for (int e = tid; e < n * wp; e += 256) {
-    const int t = e / wp, k = e - t * wp, row = p.seq_start[r0 + t], pos = p.positions[row];
-    const float* ring = p.state + (size_t)p.slot_ids[r0 + t] * p.state_stride + p.ring_offset;
+    const int t = e / wp, k = e - t * wp, row = s_row[t], pos = s_pos[t];
+    const float* ring = s_ring[t];
     const int ch = c0 + min(k, w - 1);
     float u;
     if (run) {  // all inputs asked for at once
@@ -268,7 +314,7 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs p) {
         in[j] = cw[j] = 0.f;
         if (j >= p.taps) continue;
         cw[j] = p.conv_w[(size_t)ch * p.taps + p.taps - 1 - j];
-        in[j] = j == 0 ? p.x[(size_t)row * p.ldx + ch] : ring[(size_t)((pos + p.taps - j) % p.taps) * p.W + ch];
+        in[j] = j == 0 ? p.x[(size_t)row * p.ldx + ch] : ring[(size_t)s_place[t][j] * p.W + ch];
       }
       u = p.conv_b ? p.conv_b[ch] : 0.f;
       float acc = 0.f;
@@ -285,7 +331,7 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs p) {
   const float* urow = U + lr * ld;
   auto row = [&](int k) { return *(const float4*)(urow + k); };
   f32x4_t z[2] = {f32x4_t{0.f, 0.f, 0.f, 0.f}, f32x4_t{0.f, 0.f, 0.f, 0.f}};
-  rows_product<2>(row, gates, wp, wave, 4, z);
+  ahead.product(row, gates, wp, wave, z);
 #pragma unroll
   for (int i = 0; i < 4; ++i) part[0][wave][4 * lg + i][lr] = z[0][i], part[1][wave][4 * lg + i][lr] = z[1][i];
   __syncthreads();

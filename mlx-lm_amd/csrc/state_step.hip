@@ -192,7 +192,7 @@ __device__ __forceinline__ void lowrank_rows(const StepArgs& a, int h, const flo
   const int l16 = threadIdx.x & 15, total = a.N + (a.y ? a.P : 0);
   const T* a2 = (const T*)a.a2 + (size_t)h * a.N * a.rank;
   const T* g2 = (const T*)a.g2 + (size_t)h * a.P * a.g_rank;
-#pragma unroll 4
+#pragma unroll 1
   for (int c = threadIdx.x / 16; c < total; c += TH / 16) {
     if (c < a.N) {
       const float s = lowrank_row(a2 + (size_t)c * a.rank, tz, a.rank, l16);
@@ -222,7 +222,8 @@ __global__ __launch_bounds__(TH) void state_step_kernel(StepArgs a) {
   float* tz = ds + N;                           // [rank]
   float* gs = tz + a.rank;                      // [P] the gate's logits (STEP_CHANNEL_RAW)
   float* my = gs + P;                           // [g_rank]
-  const int start = a.seq_start[rq], n = a.seq_len[rq];
+  // (raw columns: every request brings one token)
+  const int start = a.seq_start[rq], n = MODE == STEP_DELTA_RAW || MODE == STEP_CHANNEL_RAW ? 1 : a.seq_len[rq];
   float* row_state = a.state + (size_t)a.slot_ids[rq] * a.state_stride;
   float* Sg = row_state + a.state_offset + (size_t)h * N * P;
   Cols<V> S[R];
