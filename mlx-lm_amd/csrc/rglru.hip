@@ -117,15 +117,15 @@ __device__ __forceinline__ Gated gated(float zr, float zi, float u, float rate) 
   return Gated{a, sqrtf(t > -0.25f ? series : 1.0f - a * a) * sigmoid_f(zi) * u};
 }
 
-// TT: tokens in LDS at a time (64, or 16 for wide parts); four waves: TT / 16 tiles of rows, the
+// TT: tokens in LDS at a time (64, or 16 for wide parts); TH threads: TT / 16 tiles of rows, the waves'
 // remaining factor over the block's 64 channels (every block makes the whole part's convolution).
-template <typename T, int TT>
-__global__ __launch_bounds__(256) void rglru_gates_kernel(RglruArgs p) {
+template <typename T, int TT, int TH>
+__global__ __launch_bounds__(TH) void rglru_gates_kernel(RglruArgs p) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ float2 does[4][64];
-  constexpr int RT = TT / 16, NJ = RT == 4 ? 4 : 1;  // NJ: tiles of sixteen channels a wave
+  constexpr int RT = TT / 16, CW = TH / 64 / RT, NJ = 4 / CW;  // NJ: tiles of sixteen channels a wave
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lg = lane >> 4;
-  const int rt = RT == 4 ? wave : 0, j0 = RT == 4 ? 0 : wave;
+  const int rt = wave % RT, j0 = wave / RT * NJ;
   const int w = p.w, wp = p.wp, ld = wp + 4;
   float* U = lds;  // [TT][ld]
   const int slices = (w + 63) / 64, span = blockIdx.x, part = blockIdx.y / slices, s0 = blockIdx.y % slices * 64, c0 = part * w;
@@ -144,12 +144,12 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(RglruArgs p) {
   for (int t0 = 0; t0 < n; t0 += TT) {
     if (t0 > 0) __syncthreads();  // the tile before is done with U
     if (run) {
-      for (int e = tid; e < TT / CONV_TILE * wp; e += 256) {
+      for (int e = tid; e < TT / CONV_TILE * wp; e += TH) {
         const int t = e / wp * CONV_TILE, c = e % wp, first = t0 + t;
         conv_run(p, ring, row0 + first, lo + first, pos0 + first, c < w ? n - first : -CONV_TAPS, c0 + min(c, w - 1), U + t * ld + c, ld);
       }
     } else {
-      for (int e = tid; e < TT * wp; e += 256) {
+      for (int e = tid; e < TT * wp; e += TH) {
         const int t = e / wp, c = e - t * wp;
         U[t * ld + c] = c < w && t0 + t < n ? conv_at(p, ring, row0 + t0 + t, lo + t0 + t, pos0 + t0 + t, c0 + c) : 0.f;
       }
@@ -400,20 +400,20 @@ extern "C" int rglru_portions(const RglruArgs* args, hipStream_t stream) {
   if (!a.span_req || !a.span_start || !a.span_first || !a.a || !a.b || !a.does || !a.s0) FAIL("rglru_portions: null pointer");
   static bool raised = false;
   if (!raised) {
-    allow(rglru_gates_kernel<float, 64>), allow(rglru_gates_kernel<float, 16>);
-    allow(rglru_gates_kernel<bf16, 64>), allow(rglru_gates_kernel<bf16, 16>);
+    allow(rglru_gates_kernel<float, 64, 1024>), allow(rglru_gates_kernel<float, 16, 256>);
+    allow(rglru_gates_kernel<bf16, 64, 1024>), allow(rglru_gates_kernel<bf16, 16, 256>);
     raised = true;
   }
   const bool wide = gates_lds(64, a.w, a.wp) > 80 * 1024;  // (two blocks a CU)
-  const dim3 grid(a.n_spans, a.B * ((a.w + 63) / 64)), scan(a.n_spans, (a.W + 255) / 256), block(256);
+  const dim3 grid(a.n_spans, a.B * ((a.w + 63) / 64)), scan(a.n_spans, (a.W + 255) / 256), block(256), wide_block(1024);
   const size_t lds = gates_lds(wide ? 16 : 64, a.w, a.wp);
   if (a.dtype == DT_F32) {
-    if (wide) hipLaunchKernelGGL((rglru_gates_kernel<float, 16>), grid, block, lds, stream, a);
-    else hipLaunchKernelGGL((rglru_gates_kernel<float, 64>), grid, block, lds, stream, a);
+    if (wide) hipLaunchKernelGGL((rglru_gates_kernel<float, 16, 256>), grid, block, lds, stream, a);
+    else hipLaunchKernelGGL((rglru_gates_kernel<float, 64, 1024>), grid, wide_block, lds, stream, a);
     hipLaunchKernelGGL(rglru_scan_kernel<float>, scan, block, 0, stream, a);
   } else {
-    if (wide) hipLaunchKernelGGL((rglru_gates_kernel<bf16, 16>), grid, block, lds, stream, a);
-    else hipLaunchKernelGGL((rglru_gates_kernel<bf16, 64>), grid, block, lds, stream, a);
+    if (wide) hipLaunchKernelGGL((rglru_gates_kernel<bf16, 16, 256>), grid, block, lds, stream, a);
+    else hipLaunchKernelGGL((rglru_gates_kernel<bf16, 64, 1024>), grid, wide_block, lds, stream, a);
     hipLaunchKernelGGL(rglru_scan_kernel<bf16>, scan, block, 0, stream, a);
   }
   CHECK_LAUNCH("rglru_portions");
